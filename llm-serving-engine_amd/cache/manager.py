@@ -8,8 +8,9 @@ entry per token (`PagedNeed`: all of them, or a window) or an entry per request
 (`SlotNeed`); a run may need several things at once.  Every paged group has its
 own pool, block tables and, for each field its need names, a tensor [cells, NB,
 *page shape]: what a page holds is the need's business (keys and values for
-attention), the manager only hands pages out and takes them back, and a windowed
-group gives a page back as soon as no later query can read it.  A request's slot
+attention), the manager only hands pages out and takes them back, and a group
+whose readers look back through a window or within a chunk gives a page back as
+soon as no later query can read it.  A request's slot
 (the reference's metadata row) is its block-table row in every group and its
 index into every per-request tensor.
 """
@@ -179,9 +180,7 @@ class CacheManager:
 
     def _first_needed_block(self, group: PageGroup, start: int) -> int:
         """Blocks below this index (and not among the group's kept ones) hold no key that a query at position >= start reads."""
-        if group.need.window is None:
-            return 0
-        return max(0, start - group.need.window + 1) // self.page_size
+        return group.need.first_read(start) // self.page_size
 
     def _kept_blocks(self, group: PageGroup) -> int:
         """The group's first so many blocks hold entries that every later query reads: a window never gives them back."""
@@ -245,7 +244,7 @@ class CacheManager:
         slots = []
         for index, group in enumerate(self.groups):
             table = group.tables[record.slot]
-            if group.need.window is not None:
+            if group.need.window is not None or group.need.chunk is not None:
                 first = min(self._first_needed_block(group, start), first_new)
                 for block in range(max(record.released[index], self._kept_blocks(group)), first):
                     group.pool.free(int(table[block]), request_id)

@@ -1,5 +1,6 @@
 from .model import ArchitectureConfig, ConfigError, KeyReader, Qwen2Config
 from .dafutar import DafutarConfig
+from .dolezen import DolezenConfig
 from .katenex import KatenexConfig
 from .sozavik import SozavikConfig
 from .vagozen import VagozenConfig
@@ -10,6 +11,7 @@ __all__ = [
     "CacheConfig",
     "ConfigError",
     "DafutarConfig",
+    "DolezenConfig",
     "KatenexConfig",
     "KeyReader",
     "Qwen2Config",

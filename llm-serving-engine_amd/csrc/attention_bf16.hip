@@ -26,7 +26,9 @@
 // that owns the newest key rotates that key and stores key and value in their page first.
 // CHANGED: a score is changed before the softmax, for encodings and models that want it (the
 // reference has neither): `soft_cap` > 0 squashes it to cap * tanh(score / cap), and `slopes` (one
-// per query head) then takes slope * (query position - key position) off it.
+// per query head) then takes slope * (query position - key position) off it.  What leaves the scores as they are
+// is a kind of CHANGED of its own, which the fused decode form takes too: a sink in the denominator, and a mask
+// in chunks (a query sees the keys of its own chunk of positions, counted from the sequence's start).
 #include "common.h"
 
 #ifndef HEAD_DIM
@@ -95,11 +97,17 @@ struct FusedDecode {          // what the kernel needs to rotate and store; unus
                               // instead of by the step's row: for the few short requests of a step of long portions
 };
 
+// What CHANGED may be
+#define CHANGED_NOT 0
+#define CHANGED_SCORES 1      // slopes, a soft cap, kept first keys, and what CHANGED_EDGES has
+#define CHANGED_EDGES 2       // sinks and a mask in chunks alone: the scores stay as they are
+
 struct ScoreChange {          // unused unless CHANGED
   const float* slopes;        // [heads], or null
   float soft_cap;             // 0: none
   const float* sinks;         // [heads], or null: exp(sink) more in a head's denominator, once, with no value to it
   int keep_first;             // under a window, a sequence's first so many keys stay visible to every later query; 0: none
+  int chunk;                  // instead of a window: a query sees the keys of its own chunk of so many positions; 0: none
 };
 
 // One step's operands as a lane holds them: its slices of the K rows of the two 16-row tiles and,
@@ -171,7 +179,7 @@ __device__ __forceinline__ void scores_of(const Columns<COLUMN_TILES>& columns, 
 // after `last_key` (slots never written) are kept out of 0 * x.
 // CHANGED: `soft_cap` > 0 squashes a score to cap * tanh(score * scale / cap), as 1 - 2 / (1 + e^(2 score * scale / cap))
 // (right at both ends: e^x = inf gives 1, 0 gives -1), and the column's slope times the key's distance comes off it.
-template <int COLUMN_TILES, bool CHANGED = false>
+template <int COLUMN_TILES, int CHANGED = CHANGED_NOT>
 __device__ __forceinline__ void weigh_and_add(Columns<COLUMN_TILES>& columns, StepLoads& L, const f32x4* s_lo,
                                               const f32x4* s_hi, int key0, int q, bool interior, int last_key,
                                               int v_start, float scale_log2, float soft_cap = 0.f, int keep = 0) {
@@ -184,7 +192,7 @@ __device__ __forceinline__ void weigh_and_add(Columns<COLUMN_TILES>& columns, St
     float x[8];
 #pragma unroll
     for (int i = 0; i < 8; ++i) x[i] = fmaf(i < 4 ? s_lo[t][i] : s_hi[t][i - 4], scale_log2, -reference);
-    if constexpr (CHANGED) {
+    if constexpr (CHANGED == CHANGED_SCORES) {
       if (soft_cap > 0.f) {
         const float cap_log2 = soft_cap * 1.44269504088896f, doubled = 2.f * scale_log2 / soft_cap;
 #pragma unroll
@@ -200,7 +208,7 @@ __device__ __forceinline__ void weigh_and_add(Columns<COLUMN_TILES>& columns, St
     if (!interior) {
       // key0 + 8q + i outside [first, position], counted from the lane's first key (nothing to add per key)
       const int last_seen = columns.position[t] - (key0 + 8 * q), first_seen = columns.first[t] - (key0 + 8 * q);
-      if constexpr (CHANGED) {  // (the sequence's first `keep` keys are seen whatever the window)
+      if constexpr (CHANGED == CHANGED_SCORES) {  // (the sequence's first `keep` keys are seen whatever the window)
         const int kept_seen = keep - (key0 + 8 * q);
 #pragma unroll
         for (int i = 0; i < 8; ++i)
@@ -255,14 +263,14 @@ __device__ __forceinline__ void weigh_and_add(Columns<COLUMN_TILES>& columns, St
       columns.acc[t][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(L.v[d], weights[t], columns.acc[t][d], 0, 0, 0);
 }
 
-template <int COLUMN_TILES, bool FUSED, int WAVES, bool CHANGED = false>
+template <int COLUMN_TILES, bool FUSED, int WAVES, int CHANGED = CHANGED_NOT>
 __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || WAVES > 4) ? 1 : 2) void attention_tiles_kernel(
-    const bf16_t* __restrict__ qkv, int row_width, bf16_t* __restrict__ out, float* __restrict__ partial_acc,
+    const bf16_t* __restrict__ qkv, int row_width, bf16_t* __restrict__ out, int out_stride, float* __restrict__ partial_acc,
     float* __restrict__ partial_ml, bf16_t* __restrict__ keys,
     bf16_t* __restrict__ values, const int* __restrict__ block_tables, int table_width,
     const int* __restrict__ positions, const int* __restrict__ work, int heads, int kv_heads, int tokens_per_tile,
     int page_size, int page_shift, float scale, int window, int splits, FusedDecode fused, ScoreChange change) {
-  static_assert(!(FUSED && CHANGED), "the fused decode form takes plain scores only");
+  static_assert(!(FUSED && CHANGED == CHANGED_SCORES), "the fused decode form leaves the scores as they are");
   extern __shared__ float lds[];  // [WAVES][16 columns][D + 4]
   if (FUSED)  // a short kernel: fetch all arguments in one go rather than each before its first use
     asm volatile("" ::"s"(row_width), "s"(table_width), "s"(heads), "s"(kv_heads), "s"(page_size), "s"(page_shift),
@@ -293,7 +301,7 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
   [[maybe_unused]] float2 new_angle[PAIR_PIECES];
   [[maybe_unused]] int new_slot = -1;
   [[maybe_unused]] int early_k = -1, early_k_hi = -1, early_v = -1;
-  const bool early_pages = FUSED && window <= 0 && splits == 1 && (wave * KEYS + KEYS - 1) / page_size < table_width;
+  const bool early_pages = FUSED && window <= 0 && (CHANGED == CHANGED_NOT || change.chunk <= 0) && splits == 1 && (wave * KEYS + KEYS - 1) / page_size < table_width;
   // (heads up to 128 wide leave the registers for a wave's second step to be asked for together with its first)
   constexpr bool TWO_STEPS = FUSED && HEAD_DIM <= 128;
   [[maybe_unused]] int second_k = -1, second_k_hi = -1, second_v = -1;
@@ -329,7 +337,12 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
     }
   }
   const int last_key = position0 + tokens - 1;
-  const int first_key = window > 0 ? max(0, position0 - window + 1) : 0;
+  // the first key that a query at `position` sees (below 0 while a window reaches before the start); it never moves back
+  auto first_seen_from = [&](int position) {
+    if (CHANGED != CHANGED_NOT && change.chunk > 0) return position - position % change.chunk;
+    return window > 0 ? position - window + 1 : 0;
+  };
+  const int first_key = max(0, first_seen_from(position0));
 
   // this lane's column in each of its column tiles
   Columns<COLUMN_TILES> columns;
@@ -347,8 +360,8 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
     const int safe = min(token, tokens - 1);
     const int head = kv_head * group + head_tile * 16 + head_here;
     column_position[t] = column_live[t] ? position0 + safe : -1;
-    column_first[t] = window > 0 ? column_position[t] - window + 1 : 0;
-    if constexpr (CHANGED) columns.slope[t] = change.slopes ? change.slopes[head] * 1.44269504088896f : 0.f;
+    column_first[t] = first_seen_from(max(column_position[t], 0));
+    if constexpr (CHANGED == CHANGED_SCORES) columns.slope[t] = change.slopes ? change.slopes[head] * 1.44269504088896f : 0.f;
     const bf16_t* q_row = qkv + (size_t)(row0 + safe) * row_width + (size_t)head * D;
 #pragma unroll
     for (int s = 0; s < QK_STEPS; ++s) query[t][s] = load_qk(q_row, KEY_PIECE, s, q);  // a query's row is in one piece
@@ -403,10 +416,10 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
   // steps before the window's first are walked first: the walk counts from step_first - kept_steps, and a step below
   // step_first stands for step (it - step_first + kept_steps) of the sequence's start.  (Kept keys within the window's
   // first step are read there.)  Without kept keys the walk is the window's, as it was.
-  const int keep = CHANGED ? change.keep_first : 0;
-  const int kept_steps = CHANGED ? min((min(keep, first_key) + KEYS - 1) / KEYS, step_first) : 0;
+  const int keep = CHANGED == CHANGED_SCORES ? change.keep_first : 0;
+  const int kept_steps = CHANGED == CHANGED_SCORES ? min((min(keep, first_key) + KEYS - 1) / KEYS, step_first) : 0;
   const int walk_first = step_first - kept_steps;
-  auto real_step = [&](int step) { return CHANGED && step < step_first ? step - walk_first : step; };
+  auto real_step = [&](int step) { return CHANGED == CHANGED_SCORES && step < step_first ? step - walk_first : step; };
   const int per_split = (step_last - walk_first + 1 + splits - 1) / splits;
   const int step_begin = walk_first + blockIdx.z * per_split;
   const int step_end = min(step_last + 1, step_begin + per_split);
@@ -465,7 +478,7 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
   // (a kept key is read where it lies; a key between the kept ones and the window's first counts as outside, and a
   // piece of eight values that begins with a kept key lies in a page that is kept)
   auto held_key = [&](int key) {
-    if constexpr (CHANGED) {
+    if constexpr (CHANGED == CHANGED_SCORES) {
       key = min(key, last_key);
       return key < first_key && key >= keep ? first_key : key;
     } else {
@@ -473,7 +486,7 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
     }
   };
   auto held_piece = [&](int key) {
-    if constexpr (CHANGED) {
+    if constexpr (CHANGED == CHANGED_SCORES) {
       key = min(key, high_limit);
       return key < low_limit && key >= keep ? low_limit : key;
     } else {
@@ -517,6 +530,7 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
   };
 
   const float scale_log2 = scale * 1.44269504088896f;
+  const int every_first = first_seen_from(last_key);  // every column sees the keys from here on (up to its own)
 
   // A wave's next step is requested into the registers of the current one as soon as they are
   // free: the K rows after the first product, the V rows after the second; the page numbers of a
@@ -535,7 +549,7 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
         f32x4 s_lo[COLUMN_TILES], s_hi[COLUMN_TILES];
         scores_of(columns, L, s_lo, s_hi);
         const int key0 = step * KEYS;
-        const bool interior = key0 + KEYS - 1 <= position0 && (window <= 0 || key0 >= last_key - window + 1);
+        const bool interior = key0 + KEYS - 1 <= position0 && key0 >= every_first;
         weigh_and_add(columns, L, s_lo, s_hi, key0, q, interior, last_key,
                       min(max(key0 + 8 * q, low_limit), high_limit), scale_log2);
       };
@@ -574,7 +588,7 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
       scores_of(columns, loads, s_lo, s_hi);
       if (more) fetch_keys(step + WAVES, pages, loads);
       const int key0 = real_step(step) * KEYS;
-      const bool interior = key0 + KEYS - 1 <= position0 && (window <= 0 || key0 >= last_key - window + 1);
+      const bool interior = key0 + KEYS - 1 <= position0 && key0 >= every_first;
       weigh_and_add<COLUMN_TILES, CHANGED>(columns, loads, s_lo, s_hi, key0, q, interior, last_key, held_piece(key0 + 8 * q),
                                            scale_log2, change.soft_cap, keep);
       if (more) fetch_values(step + WAVES, pages, loads);
@@ -627,7 +641,7 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
       const size_t row = (size_t)row0 + token;
       if (splits == 1) {
         float shrink = 1.f;
-        if constexpr (CHANGED) {
+        if constexpr (CHANGED != CHANGED_NOT) {
           if (change.sinks) {  // (in units of log2, as the maxima are)
             const float sink = change.sinks[head] * 1.44269504088896f, top = fmaxf(best, sink);
             shrink = __builtin_amdgcn_exp2f(best - top);
@@ -637,7 +651,7 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
         const float inverse = total > 0.f ? shrink / total : 0.f;
         const bf16x4 rounded = {(bf16_t)(merged[0] * inverse), (bf16_t)(merged[1] * inverse), (bf16_t)(merged[2] * inverse),
                                 (bf16_t)(merged[3] * inverse)};
-        *(bf16x4*)(out + (row * heads + head) * D + d4) = rounded;
+        *(bf16x4*)(out + row * out_stride + head * D + d4) = rounded;
       } else {
         const size_t kept_as = fused.by_item ? (size_t)(gridDim.x - 1 - blockIdx.x) * tokens_per_tile + token : row;
         const size_t slot = (kept_as * heads + head) * splits + blockIdx.z;
@@ -722,18 +736,19 @@ __device__ __forceinline__ void merge_splits(const float* ml, const float* acc, 
 // they are many: a prompt portion's 24,576 pairs in four splits 12 us against 15)
 __global__ __launch_bounds__(MERGE_THREADS) void attention_merge_kernel(const float* __restrict__ partial_acc,
                                                                         const float* __restrict__ partial_ml,
-                                                                        bf16_t* __restrict__ out, int splits,
+                                                                        bf16_t* __restrict__ out, int out_stride, int splits,
                                                                         const float* __restrict__ sinks, int heads) {
   const size_t pair = blockIdx.x;  // row * heads + head
-  const float sink = sinks ? sinks[pair % heads] * 1.44269504088896f : -INFINITY;
-  merge_splits(partial_ml + pair * splits * 2, partial_acc + pair * splits * D, splits, out + pair * D, sink);
+  const unsigned row = blockIdx.x / (unsigned)heads, head = blockIdx.x - row * heads;
+  const float sink = sinks ? sinks[head] * 1.44269504088896f : -INFINITY;
+  merge_splits(partial_ml + pair * splits * 2, partial_acc + pair * splits * D, splits, out + (size_t)row * out_stride + head * D, sink);
 }
 
 // The same for partial results that are kept by work item: workgroup (item, head) merges the item's tokens one
 // after the other (a few), and writes to the rows that the item names.
 __global__ __launch_bounds__(MERGE_THREADS) void attention_merge_items_kernel(const float* __restrict__ partial_acc,
                                                                               const float* __restrict__ partial_ml,
-                                                                              bf16_t* __restrict__ out,
+                                                                              bf16_t* __restrict__ out, int out_stride,
                                                                               const int* __restrict__ work, int splits,
                                                                               int heads, int group, int tokens_per_tile,
                                                                               const float* __restrict__ sinks) {
@@ -743,15 +758,15 @@ __global__ __launch_bounds__(MERGE_THREADS) void attention_merge_items_kernel(co
   const float sink = sinks ? sinks[head] * 1.44269504088896f : -INFINITY;
   for (int token = 0; token < tokens; ++token) {
     const size_t kept_as = ((size_t)blockIdx.x * tokens_per_tile + token) * heads + head;
-    const size_t pair = ((size_t)item[1] + token) * heads + head;
-    merge_splits(partial_ml + kept_as * splits * 2, partial_acc + kept_as * splits * D, splits, out + pair * D, sink);
+    merge_splits(partial_ml + kept_as * splits * 2, partial_acc + kept_as * splits * D, splits,
+                 out + ((size_t)item[1] + token) * out_stride + head * D, sink);
   }
 }
 
-static int launch_merge(float* partial_acc, float* partial_ml, void* out, int splits, size_t pairs, hipStream_t stream,
-                        const float* sinks = nullptr, int heads = 1) {
+static int launch_merge(float* partial_acc, float* partial_ml, void* out, int out_stride, int splits, size_t pairs, int heads,
+                        hipStream_t stream, const float* sinks = nullptr) {
   hipLaunchKernelGGL(attention_merge_kernel, dim3((unsigned)pairs), dim3(pairs >= 4096 ? WAVE : MERGE_THREADS), 0, stream,
-                     partial_acc, partial_ml, (bf16_t*)out, splits, sinks, heads);
+                     partial_acc, partial_ml, (bf16_t*)out, out_stride, splits, sinks, heads);
   return LAUNCH_STATUS();
 }
 
@@ -788,7 +803,7 @@ __device__ __forceinline__ void load_to_lds(const bf16_t* from, unsigned to) {
 
 template <int COLUMN_TILES>
 __global__ __launch_bounds__(256, 2) void attention_portions_kernel(
-    const bf16_t* __restrict__ qkv, int row_width, bf16_t* __restrict__ out, float* __restrict__ partial_acc,
+    const bf16_t* __restrict__ qkv, int row_width, bf16_t* __restrict__ out, int out_stride, float* __restrict__ partial_acc,
     float* __restrict__ partial_ml, const bf16_t* __restrict__ keys,
     const bf16_t* __restrict__ values, const int* __restrict__ block_tables, int table_width,
     const int* __restrict__ positions, const int* __restrict__ work, int heads, int kv_heads, int tokens_per_tile,
@@ -971,7 +986,7 @@ __global__ __launch_bounds__(256, 2) void attention_portions_kernel(
         for (int piece = 0; piece < 8; ++piece) *(f32x4*)(dst + piece * 4) = *(const f32x4*)(from + piece * 4);
         if (quarter == 0) *(float2*)(partial_ml + slot * 2) = mine_ml[column];
       } else {
-        bf16_t* dst = out + ((size_t)(row0 + token) * heads + head) * D + quarter * 32;
+        bf16_t* dst = out + (size_t)(row0 + token) * out_stride + head * D + quarter * 32;
 #pragma unroll
         for (int piece = 0; piece < 4; ++piece) {
           const f32x4 lo = *(const f32x4*)(from + piece * 8);
@@ -988,7 +1003,7 @@ __global__ __launch_bounds__(256, 2) void attention_portions_kernel(
 // `work` holds `items` entries as for llmserve_attention_tiles; an item covers at most 4 * column_tiles
 // column tiles (column_tiles 1 or 2), tokens_per_tile = max(1, 16 / (heads /
 // kv_heads)).  page_size a power of two from 16 on.
-extern "C" int llmserve_attention_portions(const void* qkv, int row_width, void* out, float* partial_acc,
+extern "C" int llmserve_attention_portions(const void* qkv, int row_width, void* out, int out_stride, float* partial_acc,
                                            float* partial_ml, const void* keys,
                                            const void* values, const int* block_tables, int table_width,
                                            const int* positions, const int* work, int items, int column_tiles,
@@ -998,6 +1013,7 @@ extern "C" int llmserve_attention_portions(const void* qkv, int row_width, void*
   if (heads % kv_heads || page_size < 16 || (page_size & (page_size - 1)) != 0 || (column_tiles != 1 && column_tiles != 2))
     return ERR_BAD_ARGUMENT;
   if (splits < 1 || splits > MERGE_SPLITS_MAX || (splits > 1 && (!partial_acc || !partial_ml))) return ERR_BAD_ARGUMENT;
+  if (out_stride < heads * D || out_stride % 8) return ERR_BAD_ARGUMENT;
   if ((long)kv_heads * page_size * D >= (1L << 30)) return ERR_BAD_ARGUMENT;  // a page's bytes are counted in 32 bits
   const int group = heads / kv_heads;
   const int tokens_per_tile = group >= 16 ? 1 : 16 / group;
@@ -1005,20 +1021,20 @@ extern "C" int llmserve_attention_portions(const void* qkv, int row_width, void*
   const dim3 grid(items, kv_heads * ((group + 15) / 16), splits);
   if (column_tiles == 1)
     hipLaunchKernelGGL(attention_portions_kernel<1>, grid, dim3(256), 0, stream, (const bf16_t*)qkv, row_width,
-                       (bf16_t*)out, partial_acc, partial_ml, (const bf16_t*)keys, (const bf16_t*)values, block_tables,
+                       (bf16_t*)out, out_stride, partial_acc, partial_ml, (const bf16_t*)keys, (const bf16_t*)values, block_tables,
                        table_width, positions, work, heads, kv_heads, tokens_per_tile, page_size, page_shift, scale,
                        window, splits);
   else
     hipLaunchKernelGGL(attention_portions_kernel<2>, grid, dim3(256), 0, stream, (const bf16_t*)qkv, row_width,
-                       (bf16_t*)out, partial_acc, partial_ml, (const bf16_t*)keys, (const bf16_t*)values, block_tables,
+                       (bf16_t*)out, out_stride, partial_acc, partial_ml, (const bf16_t*)keys, (const bf16_t*)values, block_tables,
                        table_width, positions, work, heads, kv_heads, tokens_per_tile, page_size, page_shift, scale,
                        window, splits);
   const int status = LAUNCH_STATUS();
   if (status != 0 || splits == 1) return status;
-  return launch_merge(partial_acc, partial_ml, out, splits, (size_t)rows * heads, stream);
+  return launch_merge(partial_acc, partial_ml, out, out_stride, splits, (size_t)rows * heads, heads, stream);
 }
 #else
-extern "C" int llmserve_attention_portions(const void*, int, void*, float*, float*, const void*, const void*, const int*,
+extern "C" int llmserve_attention_portions(const void*, int, void*, int, float*, float*, const void*, const void*, const int*,
                                            int, const int*, const int*, int, int, int, int, int, int, float, int, int,
                                            hipStream_t) {
   return ERR_BAD_ARGUMENT;  // built for head size 128 only
@@ -1029,12 +1045,12 @@ extern "C" int llmserve_attention_portions(const void*, int, void*, float*, floa
 #ifndef FUSED_WAVES
 #define FUSED_WAVES (HEAD_DIM > 128 ? 4 : 8)
 #endif
-template <int COLUMN_TILES, bool FUSED, int WAVES, bool CHANGED = false>
-static int launch_tiles(const void* qkv, int row_width, void* out, float* partial_acc, float* partial_ml,
+template <int COLUMN_TILES, bool FUSED, int WAVES, int CHANGED = CHANGED_NOT>
+static int launch_tiles(const void* qkv, int row_width, void* out, int out_stride, float* partial_acc, float* partial_ml,
                         void* keys, void* values, const int* block_tables, int table_width,
                         const int* positions, const int* work, int tiles, int heads, int kv_heads,
                         int tokens_per_tile, int page_size, float scale, int window, int splits, FusedDecode fused,
-                        hipStream_t stream, ScoreChange change = {nullptr, 0.f, nullptr, 0}) {
+                        hipStream_t stream, ScoreChange change = {nullptr, 0.f, nullptr, 0, 0}) {
   const int group = heads / kv_heads;
   const int page_shift = (page_size & (page_size - 1)) == 0 ? __builtin_ctz(page_size) : -1;
   const int head_tiles = (group + 15) / 16;
@@ -1049,7 +1065,7 @@ static int launch_tiles(const void* qkv, int row_width, void* out, float* partia
     }
   }
   hipLaunchKernelGGL((attention_tiles_kernel<COLUMN_TILES, FUSED, WAVES, CHANGED>), dim3(tiles, kv_heads * head_tiles, splits),
-                     dim3(WAVES * 64), shared, stream, (const bf16_t*)qkv, row_width, (bf16_t*)out, partial_acc,
+                     dim3(WAVES * 64), shared, stream, (const bf16_t*)qkv, row_width, (bf16_t*)out, out_stride, partial_acc,
                      partial_ml, (bf16_t*)keys, (bf16_t*)values, block_tables, table_width, positions, work,
                      heads, kv_heads, tokens_per_tile, page_size, page_shift, scale, window, splits, fused, change);
   return LAUNCH_STATUS();
@@ -1082,20 +1098,23 @@ extern "C" int llmserve_attention_can_fuse(int pairing) {
 // weights.
 // `slopes` (float32 [heads], or null) and `soft_cap` (0 for none) change the scores before the softmax (see the head of
 // this file), `sinks` (float32 [heads], or null) add exp(sink) to a head's denominator, `keep_first` keeps a sequence's first
-// keys visible behind a window; not together with `fuse` & 1.
-extern "C" int llmserve_attention_tiles(const void* qkv, int row_width, void* out, float* partial_acc,
+// keys visible behind a window, `chunk` (0 for none; not together with a window) shows a query the keys of its own chunk of
+// positions; slopes, cap and kept keys not together with `fuse` & 1, sinks not with `fuse` & 2.
+// A row of `out` begins every `out_stride` elements (a multiple of 4 from heads * D on).
+extern "C" int llmserve_attention_tiles(const void* qkv, int row_width, void* out, int out_stride, float* partial_acc,
                                         float* partial_ml, void* keys, void* values,
                                         const int* block_tables, int table_width, const int* positions,
                                         const int* work, int tiles, int column_tiles, int rows, int heads,
                                         int kv_heads, int page_size, float scale, int window, int splits, int fuse,
                                         const float* table, int pairing, const int* slots, const float* slopes,
-                                        float soft_cap, const float* sinks, int keep_first, hipStream_t stream) {
+                                        float soft_cap, const float* sinks, int keep_first, int chunk, hipStream_t stream) {
   if (tiles <= 0) return 0;
-  if (keep_first < 0) return ERR_BAD_ARGUMENT;
+  if (keep_first < 0 || chunk < 0 || (chunk > 0 && window > 0)) return ERR_BAD_ARGUMENT;
+  if (out_stride < heads * D || out_stride % 4) return ERR_BAD_ARGUMENT;
   if (window <= 0) keep_first = 0;  // (without a window every key is seen anyway)
-  const bool changed = slopes != nullptr || soft_cap > 0.f || sinks != nullptr || keep_first > 0;
-  if (soft_cap < 0.f || (changed && (fuse & 1)) || (sinks && (fuse & 2))) return ERR_BAD_ARGUMENT;
-  const ScoreChange change = {slopes, soft_cap, sinks, keep_first};
+  const bool scores = slopes != nullptr || soft_cap > 0.f || keep_first > 0, edges = sinks != nullptr || chunk > 0;
+  if (soft_cap < 0.f || (scores && (fuse & 1)) || (sinks && (fuse & 2))) return ERR_BAD_ARGUMENT;
+  const ScoreChange change = {slopes, soft_cap, sinks, keep_first, chunk};
   if (heads % kv_heads || page_size % 8 || splits < 1 || splits > MERGE_SPLITS_MAX || (splits > 1 && (!partial_acc || !partial_ml)))
     return ERR_BAD_ARGUMENT;
   if ((long)kv_heads * page_size * D >= (1L << 31)) return ERR_BAD_ARGUMENT;  // a page's elements are counted in 32 bits
@@ -1111,33 +1130,28 @@ extern "C" int llmserve_attention_tiles(const void* qkv, int row_width, void* ou
   if (fuse) {
     if (column_tiles != 1 || tiles != rows || !slots || !llmserve_attention_can_fuse(pairing) || (pairing != 0 && !table))
       return ERR_BAD_ARGUMENT;
-    status = launch_tiles<1, true, FUSED_WAVES>(qkv, row_width, out, partial_acc, partial_ml, keys, values, block_tables,
-                                        table_width, positions, work, tiles, heads, kv_heads, tokens_per_tile,
-                                        page_size, scale, window, splits, fused, stream);
-  } else if (changed && column_tiles == 1) {
-    status = launch_tiles<1, false, 4, true>(qkv, row_width, out, partial_acc, partial_ml, keys, values, block_tables,
-                                          table_width, positions, work, tiles, heads, kv_heads, tokens_per_tile,
-                                          page_size, scale, window, splits, fused, stream, change);
-  } else if (changed && column_tiles == 2) {
-    status = launch_tiles<2, false, 4, true>(qkv, row_width, out, partial_acc, partial_ml, keys, values, block_tables,
-                                          table_width, positions, work, tiles, heads, kv_heads, tokens_per_tile,
-                                          page_size, scale, window, splits, fused, stream, change);
+#define LAUNCH_TILES(COLUMN_TILES, FUSED, WAVES, CHANGED)                                                                 \
+  launch_tiles<COLUMN_TILES, FUSED, WAVES, CHANGED>(qkv, row_width, out, out_stride, partial_acc, partial_ml, keys, values, \
+                                                    block_tables, table_width, positions, work, tiles, heads, kv_heads,     \
+                                                    tokens_per_tile, page_size, scale, window, splits, fused, stream, change)
+    status = edges ? LAUNCH_TILES(1, true, FUSED_WAVES, CHANGED_EDGES) : LAUNCH_TILES(1, true, FUSED_WAVES, CHANGED_NOT);
   } else if (column_tiles == 1) {
-    status = launch_tiles<1, false, 4>(qkv, row_width, out, partial_acc, partial_ml, keys, values, block_tables,
-                                    table_width, positions, work, tiles, heads, kv_heads, tokens_per_tile, page_size,
-                                    scale, window, splits, fused, stream);
+    status = scores  ? LAUNCH_TILES(1, false, 4, CHANGED_SCORES)
+             : edges ? LAUNCH_TILES(1, false, 4, CHANGED_EDGES)
+                     : LAUNCH_TILES(1, false, 4, CHANGED_NOT);
   } else if (column_tiles == 2) {
-    status = launch_tiles<2, false, 4>(qkv, row_width, out, partial_acc, partial_ml, keys, values, block_tables,
-                                    table_width, positions, work, tiles, heads, kv_heads, tokens_per_tile, page_size,
-                                    scale, window, splits, fused, stream);
+    status = scores  ? LAUNCH_TILES(2, false, 4, CHANGED_SCORES)
+             : edges ? LAUNCH_TILES(2, false, 4, CHANGED_EDGES)
+                     : LAUNCH_TILES(2, false, 4, CHANGED_NOT);
   } else {
     return ERR_BAD_ARGUMENT;
   }
+#undef LAUNCH_TILES
   if (status != 0 || splits == 1 || unmerged) return status;
   if (by_item) {
     hipLaunchKernelGGL(attention_merge_items_kernel, dim3(tiles, heads), dim3(MERGE_THREADS), 0, stream, partial_acc, partial_ml,
-                       (bf16_t*)out, work, splits, heads, group, tokens_per_tile, sinks);
+                       (bf16_t*)out, out_stride, work, splits, heads, group, tokens_per_tile, sinks);
     return LAUNCH_STATUS();
   }
-  return launch_merge(partial_acc, partial_ml, out, splits, (size_t)rows * heads, stream, sinks, heads);
+  return launch_merge(partial_acc, partial_ml, out, out_stride, splits, (size_t)rows * heads, heads, stream, sinks);
 }

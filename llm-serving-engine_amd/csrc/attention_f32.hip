@@ -7,7 +7,8 @@
 // (the reference has neither): `soft_cap` > 0 squashes it to cap * tanh(score / cap), and `slopes` (one
 // per query head) then adds -slope * (query position - key position).  With `sinks` (one per query head) the
 // softmax's denominator has exp(sink) more, once, with no value to it; it is added where a column's sums are final
-// (in the kernel that merges key splits, where there are splits).
+// (in the kernel that merges key splits, where there are splits).  `chunk` > 0 is a mask instead of a window: a query
+// sees the keys of its own chunk of so many positions, counted from the sequence's start.
 //
 // The unit of work is an item: up to 16 * COLUMN_TILES "columns", the (token, query head) pairs of
 // consecutive tokens of one request that share one kv head, running through the tokens head by head so
@@ -44,11 +45,11 @@ __device__ __forceinline__ f32x4 load4(const float* p) { return *(const f32x4*)p
 // CHANGED: the scores carry a soft cap or a distance bias (a variant of its own, so that the plain one pays nothing)
 template <int COLUMN_TILES, bool CHANGED>
 __global__ __launch_bounds__(WAVES * 64) void attention_f32_kernel(
-    const float* __restrict__ qkv, int row_width, float* __restrict__ out, float* __restrict__ partial_acc,
+    const float* __restrict__ qkv, int row_width, float* __restrict__ out, int out_stride, float* __restrict__ partial_acc,
     float* __restrict__ partial_ml, const float* __restrict__ keys, const float* __restrict__ values,
     const int* __restrict__ block_tables, int table_width, const int* __restrict__ positions,
     const int* __restrict__ work, int heads, int kv_heads, int page_size, float scale_log2, int window, int splits,
-    int columns_total, const float* __restrict__ slopes, float soft_cap, const float* __restrict__ sinks, int keep_first) {
+    int columns_total, const float* __restrict__ slopes, float soft_cap, const float* __restrict__ sinks, int keep_first, int chunk) {
   __shared__ float wave_max[WAVES][COLUMN_TILES][16];
   __shared__ float wave_sum[WAVES][COLUMN_TILES][16];
   __shared__ __attribute__((aligned(16))) float merged[COLUMN_TILES][D_STEPS][64][4];
@@ -61,6 +62,11 @@ __global__ __launch_bounds__(WAVES * 64) void attention_f32_kernel(
   const int i = lane & 15, g = lane >> 4;
   const int* table = block_tables + (size_t)request * table_width;
 
+  // the first key that a query at `position` sees; it never moves back
+  auto first_seen_from = [&](int position) {
+    if (CHANGED && chunk > 0) return position - position % chunk;
+    return window > 0 ? max(0, position - window + 1) : 0;
+  };
   // this lane's column in each tile: its token, head, and the keys it sees, [first, position]
   int position[COLUMN_TILES], first[COLUMN_TILES], token_row[COLUMN_TILES], head[COLUMN_TILES];
   [[maybe_unused]] float slope[COLUMN_TILES];  // of the column's head, in units of log2
@@ -73,7 +79,7 @@ __global__ __launch_bounds__(WAVES * 64) void attention_f32_kernel(
     token_row[t] = first_row + flat / group;
     head[t] = kv_head * group + flat % group;
     position[t] = live ? positions[token_row[t]] : -1;
-    first[t] = window > 0 ? max(0, position[t] - window + 1) : 0;
+    first[t] = first_seen_from(max(position[t], 0));
     if (CHANGED) slope[t] = slopes ? slopes[head[t]] * 1.4426950408889634f : 0.f;
     const float* q = qkv + (size_t)token_row[t] * row_width + head[t] * D + 4 * g;
 #pragma unroll
@@ -86,8 +92,7 @@ __global__ __launch_bounds__(WAVES * 64) void attention_f32_kernel(
   // the item's keys: from the first that its first token sees to its last token's own
   const int last_flat = first_head + columns - 1;
   const int end = positions[first_row + last_flat / group] + 1;
-  const int first_position = positions[first_row];
-  const int begin = window > 0 ? max(0, first_position - window + 1) : 0;
+  const int begin = first_seen_from(positions[first_row]);
   // steps of 16 keys, aligned to 16; the splits share them in contiguous runs, the waves take a run's in turn
   const int step_first = begin / KEYS, step_end = (end + KEYS - 1) / KEYS;
   // The sequence's first `keep` keys stay visible behind a window.  Those of them that lie in steps before the window's
@@ -265,7 +270,7 @@ __global__ __launch_bounds__(WAVES * 64) void attention_f32_kernel(
         const float scale = sum > 0.f ? shrink / sum : 0.f;
 #pragma unroll
         for (int e = 0; e < 4; ++e) result[e] *= scale;
-        *(f32x4*)(out + column * D + 16 * s + 4 * g) = result;
+        *(f32x4*)(out + (size_t)token_row[t] * out_stride + head[t] * D + 16 * s + 4 * g) = result;
       } else {
         *(f32x4*)(partial_acc + ((size_t)split * columns_total + column) * D + 16 * s + 4 * g) = result;
       }
@@ -300,7 +305,7 @@ __device__ __forceinline__ float merge_some(const float* acc, size_t split_strid
   return sum;
 }
 
-__global__ __launch_bounds__(MERGE_THREADS) void attention_f32_merge_kernel(float* __restrict__ out,
+__global__ __launch_bounds__(MERGE_THREADS) void attention_f32_merge_kernel(float* __restrict__ out, int out_stride,
                                                                            const float* __restrict__ partial_acc,
                                                                            const float* __restrict__ partial_ml,
                                                                            int splits, int columns_total,
@@ -325,32 +330,34 @@ __global__ __launch_bounds__(MERGE_THREADS) void attention_f32_merge_kernel(floa
   int first = 0;
   for (; splits - first > 8; first += 32) sum += merge_some<32>(acc, split_stride, first, splits, weight);
   if (first < splits) sum += merge_some<8>(acc, split_stride, first, splits, weight);
-  if (d < D) out[column * D + d] = sum * inverse;
+  if (d < D) out[(column / heads) * out_stride + (column % heads) * D + d] = sum * inverse;
 }
 
 // qkv [tokens, row_width] float32 with the queries in front (heads * D), out [tokens, heads * D]; key pages in
 // pieces ([page, kv_head, D / 8, offset, 8]), value pages transposed in pieces of eight keys ([page, kv_head,
 // page_size / 8, D, 8]; common.h: value_element); work [items, 4].
-// column_tiles 1 or 2; page_size a multiple of 4; slopes and sinks float32 [heads] or null, soft_cap 0 for none.  With splits > 1: partial_acc float32 [splits, tokens * heads, D]
+// A row of `out` begins every `out_stride` elements.  column_tiles 1 or 2; page_size a multiple of 4; slopes and sinks float32 [heads] or null, soft_cap 0 for none.  With splits > 1: partial_acc float32 [splits, tokens * heads, D]
 // and partial_ml [splits, tokens * heads, 2]; every column of the step must belong to an item.
-extern "C" int llmserve_attention_f32(const float* qkv, int row_width, float* out, float* partial_acc, float* partial_ml,
+extern "C" int llmserve_attention_f32(const float* qkv, int row_width, float* out, int out_stride, float* partial_acc, float* partial_ml,
                                       const float* keys, const float* values, const int* block_tables, int table_width,
                                       const int* positions, const int* work, int items, int column_tiles, int tokens,
                                       int heads, int kv_heads, int page_size, float scale, int window, int splits,
-                                      const float* slopes, float soft_cap, const float* sinks, int keep_first, hipStream_t stream) {
+                                      const float* slopes, float soft_cap, const float* sinks, int keep_first, int chunk,
+                                      hipStream_t stream) {
   if (items <= 0 || tokens <= 0) return 0;
-  if (keep_first < 0) return ERR_BAD_ARGUMENT;
+  if (keep_first < 0 || chunk < 0 || (chunk > 0 && (window > 0 || keep_first > 0))) return ERR_BAD_ARGUMENT;
+  if (out_stride < heads * D || out_stride % 4) return ERR_BAD_ARGUMENT;
   if (heads <= 0 || kv_heads <= 0 || heads % kv_heads || page_size <= 0 || page_size % 4 || splits < 1 ||
       splits > MERGE_SPLITS_MAX || (column_tiles != 1 && column_tiles != 2) || (splits > 1 && (!partial_acc || !partial_ml)))
     return ERR_BAD_ARGUMENT;
   const float scale_log2 = scale * 1.4426950408889634f;
   const int columns_total = tokens * heads;
   dim3 grid(items, kv_heads, splits);
-  const bool changed = slopes != nullptr || soft_cap > 0.f || sinks != nullptr || (keep_first > 0 && window > 0);
+  const bool changed = slopes != nullptr || soft_cap > 0.f || sinks != nullptr || (keep_first > 0 && window > 0) || chunk > 0;
 #define LAUNCH_ATTENTION_F32(TILES, CHANGED)                                                                          \
-  hipLaunchKernelGGL((attention_f32_kernel<TILES, CHANGED>), grid, dim3(WAVES * 64), 0, stream, qkv, row_width, out,   \
+  hipLaunchKernelGGL((attention_f32_kernel<TILES, CHANGED>), grid, dim3(WAVES * 64), 0, stream, qkv, row_width, out, out_stride, \
                      partial_acc, partial_ml, keys, values, block_tables, table_width, positions, work, heads,        \
-                     kv_heads, page_size, scale_log2, window, splits, columns_total, slopes, soft_cap, sinks, keep_first)
+                     kv_heads, page_size, scale_log2, window, splits, columns_total, slopes, soft_cap, sinks, keep_first, chunk)
   if (column_tiles == 1 && !changed) LAUNCH_ATTENTION_F32(1, false);
   else if (column_tiles == 1) LAUNCH_ATTENTION_F32(1, true);
   else if (!changed) LAUNCH_ATTENTION_F32(2, false);
@@ -358,7 +365,7 @@ extern "C" int llmserve_attention_f32(const float* qkv, int row_width, float* ou
 #undef LAUNCH_ATTENTION_F32
   int status = LAUNCH_STATUS();
   if (status != 0 || splits == 1) return status;
-  hipLaunchKernelGGL(attention_f32_merge_kernel, dim3(columns_total), dim3(MERGE_THREADS), 0, stream, out, partial_acc, partial_ml,
+  hipLaunchKernelGGL(attention_f32_merge_kernel, dim3(columns_total), dim3(MERGE_THREADS), 0, stream, out, out_stride, partial_acc, partial_ml,
                      splits, columns_total, sinks, heads);
   return LAUNCH_STATUS();
 }

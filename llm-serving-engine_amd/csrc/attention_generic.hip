@@ -9,7 +9,8 @@
 // them (the reference has neither): `soft_cap` > 0 squashes it to cap * tanh(score / cap), and
 // `slopes` (one per query head) then adds -slope * (query position - key position), a bias that
 // grows with distance.  With `sinks` (one per query head) the softmax's denominator has exp(sink) more, once, with
-// no value to it: a key that is not there.
+// no value to it: a key that is not there.  `chunk` > 0 is a mask instead of a window: a query sees the keys of its own chunk of
+// so many positions, counted from the sequence's start.
 #include "common.h"
 
 #define KEYS_PER_TILE 128
@@ -17,11 +18,11 @@
 
 template <typename T>
 __global__ __launch_bounds__(KEYS_PER_TILE) void attention_generic_kernel(
-    const T* __restrict__ qkv, int row_width, T* __restrict__ out, const T* __restrict__ keys,
+    const T* __restrict__ qkv, int row_width, T* __restrict__ out, int out_stride, const T* __restrict__ keys,
     const T* __restrict__ values, const int* __restrict__ block_tables, int table_width,
     const int* __restrict__ token_sequence, const int* __restrict__ positions, int heads, int kv_heads, int dim,
     int page_size, float scale, int window, const float* __restrict__ slopes, float soft_cap, const float* __restrict__ sinks,
-    int keep_first) {
+    int keep_first, int chunk) {
   __shared__ float query[MAX_DIM];
   __shared__ float weights[KEYS_PER_TILE];
   __shared__ float shared[17];
@@ -33,7 +34,7 @@ __global__ __launch_bounds__(KEYS_PER_TILE) void attention_generic_kernel(
   for (int d = threadIdx.x; d < dim; d += blockDim.x) query[d] = to_float(q[d]) * scale;
   __syncthreads();
 
-  const int first = window > 0 ? max(0, position - window + 1) : 0;
+  const int first = chunk > 0 ? position - position % chunk : window > 0 ? max(0, position - window + 1) : 0;
   const float slope = slopes ? slopes[head] : 0.f;
   const int width = key_piece_width(dim);
   const int per_thread = (dim + KEYS_PER_TILE - 1) / KEYS_PER_TILE;  // output dims per thread, <= 4
@@ -89,29 +90,31 @@ __global__ __launch_bounds__(KEYS_PER_TILE) void attention_generic_kernel(
     shrink = expf(running_max - top);
     running_sum = running_sum * shrink + expf(sink - top);
   }
-  T* o = out + ((size_t)token * heads + head) * dim;
+  T* o = out + (size_t)token * out_stride + head * dim;
   for (int i = 0; i < per_thread; ++i) {
     const int d = threadIdx.x + i * KEYS_PER_TILE;
     if (d < dim) o[d] = from_float<T>(acc[i] * shrink / running_sum);
   }
 }
 
-extern "C" int llmserve_attention_generic(const void* qkv, int row_width, void* out, int is_float, const void* keys,
+extern "C" int llmserve_attention_generic(const void* qkv, int row_width, void* out, int out_stride, int is_float, const void* keys,
                                           const void* values, const int* block_tables, int table_width,
                                           const int* token_sequence, const int* positions, int tokens, int heads,
                                           int kv_heads, int dim, int page_size, float scale, int window,
                                           const float* slopes, float soft_cap, const float* sinks, int keep_first,
-                                          hipStream_t stream) {
+                                          int chunk, hipStream_t stream) {
   if (tokens <= 0) return 0;
-  if (dim > MAX_DIM || dim <= 0 || heads % kv_heads || page_size <= 0 || keep_first < 0) return ERR_BAD_ARGUMENT;
+  if (dim > MAX_DIM || dim <= 0 || heads % kv_heads || page_size <= 0 || keep_first < 0 || chunk < 0 ||
+      (chunk > 0 && (window > 0 || keep_first > 0)) || out_stride < heads * dim)
+    return ERR_BAD_ARGUMENT;
   dim3 grid(tokens, heads);
   if (is_float)
     hipLaunchKernelGGL(attention_generic_kernel<float>, grid, dim3(KEYS_PER_TILE), 0, stream, (const float*)qkv,
-                       row_width, (float*)out, (const float*)keys, (const float*)values, block_tables, table_width,
-                       token_sequence, positions, heads, kv_heads, dim, page_size, scale, window, slopes, soft_cap, sinks, keep_first);
+                       row_width, (float*)out, out_stride, (const float*)keys, (const float*)values, block_tables, table_width,
+                       token_sequence, positions, heads, kv_heads, dim, page_size, scale, window, slopes, soft_cap, sinks, keep_first, chunk);
   else
     hipLaunchKernelGGL(attention_generic_kernel<bf16_t>, grid, dim3(KEYS_PER_TILE), 0, stream, (const bf16_t*)qkv,
-                       row_width, (bf16_t*)out, (const bf16_t*)keys, (const bf16_t*)values, block_tables, table_width,
-                       token_sequence, positions, heads, kv_heads, dim, page_size, scale, window, slopes, soft_cap, sinks, keep_first);
+                       row_width, (bf16_t*)out, out_stride, (const bf16_t*)keys, (const bf16_t*)values, block_tables, table_width,
+                       token_sequence, positions, heads, kv_heads, dim, page_size, scale, window, slopes, soft_cap, sinks, keep_first, chunk);
   return LAUNCH_STATUS();
 }

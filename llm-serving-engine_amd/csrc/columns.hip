@@ -7,12 +7,14 @@
 #define ACT_GELU 1
 #define ACT_GELU_TANH 2
 #define ACT_RELU 3
+#define ACT_SQUARED_RELU 5  // (4 is a function of two operands, which the gated products have)
 
 __device__ __forceinline__ float activation_of(int activation, float z) {
   switch (activation) {
     case ACT_GELU: return 0.5f * z * (1.f + erff(z * 0.70710678118654752f));
     case ACT_GELU_TANH: return 0.5f * z * (1.f + tanhf(0.79788456080286536f * (z + 0.044715f * z * z * z)));
     case ACT_RELU: return fmaxf(z, 0.f);
+    case ACT_SQUARED_RELU: return fmaxf(z, 0.f) * fmaxf(z, 0.f);
     default: return z / (1.f + expf(-z));
   }
 }
@@ -80,12 +82,13 @@ extern "C" int llmserve_rotary_table_scaled(const int* positions, const float* f
 
 // ---------------------------------------------------------------------------- rotation of a run of columns per head
 // For every head h: the `width` columns of x from first + h * head_stride go to the columns of out from out_first +
-// h * out_head_stride; of them the first `dims` are rotated in adjacent pairs, (u, v) at columns (2i, 2i + 1) becoming
-// (u cos_i - v sin_i, v cos_i + u sin_i) with the token's table entry i; the others are copied.
+// h * out_head_stride; of them the first `dims` are rotated in pairs, (u, v) at columns (2i, 2i + 1), or with `halves`
+// at columns (i, i + dims / 2), becoming (u cos_i - v sin_i, v cos_i + u sin_i) with the token's table entry i; the
+// others are copied.
 template <typename T>
 __global__ void rotate_columns_kernel(const T* __restrict__ x, int x_stride, int first, int head_stride, int heads, int width,
                                       const float2* __restrict__ table, int dims, T* __restrict__ out, int out_stride,
-                                      int out_first, int out_head_stride) {
+                                      int out_first, int out_head_stride, int halves) {
   const T* row = x + (size_t)blockIdx.x * x_stride + first;
   T* dst = out + (size_t)blockIdx.x * out_stride + out_first;
   const float2* angles = table + (size_t)blockIdx.x * (dims / 2);
@@ -94,9 +97,11 @@ __global__ void rotate_columns_kernel(const T* __restrict__ x, int x_stride, int
     const T* from = row + (size_t)head * head_stride;
     float value = to_float(from[c]);
     if (c < dims) {
-      const float2 turn = angles[c / 2];
-      const float other = to_float(from[c ^ 1]);
-      value = (c & 1) ? value * turn.x + other * turn.y : value * turn.x - other * turn.y;
+      const int half = dims / 2;
+      const bool second = halves ? c >= half : (c & 1) != 0;
+      const float2 turn = angles[halves ? (second ? c - half : c) : c / 2];
+      const float other = to_float(from[halves ? (second ? c - half : c + half) : c ^ 1]);
+      value = second ? value * turn.x + other * turn.y : value * turn.x - other * turn.y;
     }
     dst[(size_t)head * out_head_stride + c] = from_float<T>(value);
   }
@@ -104,7 +109,7 @@ __global__ void rotate_columns_kernel(const T* __restrict__ x, int x_stride, int
 
 extern "C" int llmserve_rotate_columns(const void* x, int is_float, int tokens, int x_stride, int first, int head_stride,
                                        int heads, int width, const float* table, int dims, void* out, int out_stride,
-                                       int out_first, int out_head_stride, hipStream_t stream) {
+                                       int out_first, int out_head_stride, int halves, hipStream_t stream) {
   if (tokens <= 0) return 0;
   if (dims % 2 || dims > width || heads < 1 || first + (heads - 1) * head_stride + width > x_stride ||
       out_first + (heads - 1) * out_head_stride + width > out_stride)
@@ -112,10 +117,10 @@ extern "C" int llmserve_rotate_columns(const void* x, int is_float, int tokens, 
   const int threads = heads * width <= 64 ? 64 : heads * width <= 128 ? 128 : 256;
   if (is_float)
     hipLaunchKernelGGL(rotate_columns_kernel<float>, dim3(tokens), dim3(threads), 0, stream, (const float*)x, x_stride, first,
-                       head_stride, heads, width, (const float2*)table, dims, (float*)out, out_stride, out_first, out_head_stride);
+                       head_stride, heads, width, (const float2*)table, dims, (float*)out, out_stride, out_first, out_head_stride, halves);
   else
     hipLaunchKernelGGL(rotate_columns_kernel<bf16_t>, dim3(tokens), dim3(threads), 0, stream, (const bf16_t*)x, x_stride, first,
-                       head_stride, heads, width, (const float2*)table, dims, (bf16_t*)out, out_stride, out_first, out_head_stride);
+                       head_stride, heads, width, (const float2*)table, dims, (bf16_t*)out, out_stride, out_first, out_head_stride, halves);
   return LAUNCH_STATUS();
 }
 
@@ -165,6 +170,53 @@ extern "C" int llmserve_activate(const void* in, void* out, int is_float, int ro
   else
     hipLaunchKernelGGL(activate_kernel<bf16_t>, dim3(blocks), dim3(256), 0, stream, (const bf16_t*)in, (bf16_t*)out, count, activation);
   return LAUNCH_STATUS();
+}
+
+// out[t, out_first + i] = act(in[t, first + i]) for i < width: a run of a row's columns, to a run of another row's.  A
+// thread takes eight columns where both runs begin and lie on multiples of eight (`octets`), else one.
+template <typename T, bool OCTETS>
+__global__ __launch_bounds__(256) void activate_columns_kernel(const T* __restrict__ in, int in_stride, int first,
+                                                               T* __restrict__ out, int out_stride, int out_first, int width,
+                                                               int activation, unsigned per_row, unsigned total) {
+  typedef T T8 __attribute__((ext_vector_type(8)));
+  const unsigned at = blockIdx.x * 256u + threadIdx.x;
+  if (at >= total) return;
+  const unsigned row = at / per_row, piece = at - row * per_row;
+  const T* from = in + (size_t)row * in_stride + first;
+  T* to = out + (size_t)row * out_stride + out_first;
+  if constexpr (OCTETS) {
+    const T8 value = *(const T8*)(from + piece * 8);
+    T8 result;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) result[i] = from_float<T>(activation_of(activation, to_float(value[i])));
+    *(T8*)(to + piece * 8) = result;
+  } else {
+    to[piece] = from_float<T>(activation_of(activation, to_float(from[piece])));
+  }
+}
+
+template <typename T>
+static int launch_activate_columns(const void* in, int rows, int in_stride, int first, void* out, int out_stride, int out_first,
+                                   int width, int activation, hipStream_t stream) {
+  const bool octets = in_stride % 8 == 0 && first % 8 == 0 && out_stride % 8 == 0 && out_first % 8 == 0 && width % 8 == 0;
+  const unsigned per_row = octets ? width / 8 : width, total = per_row * (unsigned)rows;
+  const dim3 grid((total + 255) / 256), block(256);
+  if (octets)
+    hipLaunchKernelGGL((activate_columns_kernel<T, true>), grid, block, 0, stream, (const T*)in, in_stride, first, (T*)out, out_stride,
+                       out_first, width, activation, per_row, total);
+  else
+    hipLaunchKernelGGL((activate_columns_kernel<T, false>), grid, block, 0, stream, (const T*)in, in_stride, first, (T*)out, out_stride,
+                       out_first, width, activation, per_row, total);
+  return LAUNCH_STATUS();
+}
+
+extern "C" int llmserve_activate_columns(const void* in, int is_float, int rows, int in_stride, int first, void* out, int out_stride,
+                                         int out_first, int width, int activation, hipStream_t stream) {
+  if (rows <= 0 || width <= 0) return 0;
+  if (first < 0 || out_first < 0 || first + width > in_stride || out_first + width > out_stride || (long)rows * width >= (1L << 31))
+    return ERR_BAD_ARGUMENT;
+  return is_float ? launch_activate_columns<float>(in, rows, in_stride, first, out, out_stride, out_first, width, activation, stream)
+                  : launch_activate_columns<bf16_t>(in, rows, in_stride, first, out, out_stride, out_first, width, activation, stream);
 }
 
 // ---------------------------------------------------------------------------- gated add

@@ -4,23 +4,23 @@
 #include "common.h"
 
 // ---------------------------------------------------------------------------- embedding
-// out[t, :] = float(table[ids[t], :])        (reference model.py:293)
+// out[t, :] = float(table[ids[t], :]) * scale        (reference model.py:293, which has no scale)
 template <typename T>
 __global__ void embedding_kernel(const T* __restrict__ table, const int* __restrict__ ids,
-                                 float* __restrict__ out, int hidden) {
+                                 float* __restrict__ out, int hidden, float scale) {
   const size_t row = (size_t)ids[blockIdx.x];
   const T* src = table + row * hidden;
   float* dst = out + (size_t)blockIdx.x * hidden;
-  for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = to_float(src[i]);
+  for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = to_float(src[i]) * scale;
 }
 
 extern "C" int llmserve_embedding(const void* table, int table_is_float, const int* ids, float* out,
-                                  int tokens, int hidden, hipStream_t stream) {
+                                  int tokens, int hidden, float scale, hipStream_t stream) {
   if (tokens <= 0) return 0;
   if (table_is_float)
-    hipLaunchKernelGGL(embedding_kernel<float>, dim3(tokens), dim3(256), 0, stream, (const float*)table, ids, out, hidden);
+    hipLaunchKernelGGL(embedding_kernel<float>, dim3(tokens), dim3(256), 0, stream, (const float*)table, ids, out, hidden, scale);
   else
-    hipLaunchKernelGGL(embedding_kernel<bf16_t>, dim3(tokens), dim3(256), 0, stream, (const bf16_t*)table, ids, out, hidden);
+    hipLaunchKernelGGL(embedding_kernel<bf16_t>, dim3(tokens), dim3(256), 0, stream, (const bf16_t*)table, ids, out, hidden, scale);
   return LAUNCH_STATUS();
 }
 
@@ -379,12 +379,12 @@ extern "C" int llmserve_rotary_table(const int* positions, const float* inverse,
 // reference kv_cache.py:249-266 writes both as [page, offset, kv_head, dim]).
 // slots may be null (nothing is stored); a negative slot skips the token.
 template <typename T>
-__global__ void rotate_and_store_kernel(T* __restrict__ qkv, const float2* __restrict__ table, int pairing, int heads,
+__global__ void rotate_and_store_kernel(T* __restrict__ qkv, int row_stride, const float2* __restrict__ table, int pairing, int heads,
                                         int kv_heads, int dim, T* __restrict__ keys, T* __restrict__ values,
                                         const int* __restrict__ slots, int page_size) {
   const int token = blockIdx.x;
   const int half = dim / 2;
-  T* row = qkv + (size_t)token * (heads + 2 * kv_heads) * dim;
+  T* row = qkv + (size_t)token * row_stride;
   if (pairing != 0) {
     const float2* angles = table + (size_t)token * half;
     const int pairs = (heads + kv_heads) * half;
@@ -420,14 +420,13 @@ __global__ void rotate_and_store_kernel(T* __restrict__ qkv, const float2* __res
 // back, and, for a k head, writes them to the page as well; further threads take eight elements of
 // a v head each.  Threads are dealt to (token, piece) pairs without regard to blocks.
 __global__ __launch_bounds__(256) void rotate_and_store_vector_kernel(
-    bf16_t* __restrict__ qkv, const float2* __restrict__ table, int pairing, int heads, int kv_heads, int dim,
+    bf16_t* __restrict__ qkv, int row_stride, const float2* __restrict__ table, int pairing, int heads, int kv_heads, int dim,
     bf16_t* __restrict__ keys, bf16_t* __restrict__ values, const int* __restrict__ slots, int page_size, int tokens) {
   typedef bf16_t bf16x8 __attribute__((ext_vector_type(8)));
   typedef bf16_t bf16x4 __attribute__((ext_vector_type(4)));
   const int per_head = dim / 16, half = dim / 2;
   const int rotated = (heads + kv_heads) * per_head;
   const size_t id = (size_t)blockIdx.x * 256 + threadIdx.x, rotating = (size_t)tokens * rotated;
-  const int row_width = (heads + 2 * kv_heads) * dim;
   if (id >= rotating) {
     // The values.  A page keeps them transposed in pieces of eight keys (attention sums over keys), so a
     // token's value row is `dim` two-byte stores 16 bytes apart.  A thread therefore takes four dims of eight
@@ -446,7 +445,7 @@ __global__ __launch_bounds__(256) void rotate_and_store_vector_kernel(
     for (int i = 0; i < 8; ++i) {
       const int token = first + min(i, count - 1);
       slot[i] = i < count ? slots[token] : -1;
-      v[i] = *(const bf16x4*)(qkv + (size_t)token * row_width + (size_t)(heads + kv_heads + head) * dim + quad * 4);
+      v[i] = *(const bf16x4*)(qkv + (size_t)token * row_stride + (size_t)(heads + kv_heads + head) * dim + quad * 4);
     }
     bool together = count == 8 && slot[0] >= 0 && slot[0] % 8 == 0 && page_size % 8 == 0;
 #pragma unroll
@@ -470,7 +469,7 @@ __global__ __launch_bounds__(256) void rotate_and_store_vector_kernel(
     return;
   }
   const int token = (int)(id / rotated), piece = (int)(id % rotated);
-  bf16_t* row = qkv + (size_t)token * row_width;
+  bf16_t* row = qkv + (size_t)token * row_stride;
   const int slot = slots ? slots[token] : -1;
   const int head = piece / per_head, p = piece % per_head;
   bf16_t* h = row + head * dim;
@@ -511,26 +510,28 @@ __global__ __launch_bounds__(256) void rotate_and_store_vector_kernel(
   }
 }
 
-extern "C" int llmserve_rotate_and_store(void* qkv, int is_float, const float* table, int pairing, int tokens,
+// A row of qkv (heads, then kv_heads keys, then kv_heads values of `dim`) begins every `row_stride` elements.
+extern "C" int llmserve_rotate_and_store(void* qkv, int row_stride, int is_float, const float* table, int pairing, int tokens,
                                          int heads, int kv_heads, int dim, void* keys, void* values,
                                          const int* slots, int page_size, hipStream_t stream) {
   if (tokens <= 0) return 0;
-  if (dim % 2 || (pairing != 0 && table == nullptr) || pairing < 0 || pairing > 2) return ERR_BAD_ARGUMENT;
-  if (!is_float && dim % 16 == 0) {
+  if (dim % 2 || (pairing != 0 && table == nullptr) || pairing < 0 || pairing > 2 || row_stride < (heads + 2 * kv_heads) * dim)
+    return ERR_BAD_ARGUMENT;
+  if (!is_float && dim % 16 == 0 && row_stride % 8 == 0) {
     // a thread for every 16 elements of a token's q and k heads, then one for every four dims of eight tokens' values
     const size_t threads = (size_t)tokens * (heads + kv_heads) * (dim / 16) +
                            (slots ? (size_t)((tokens + 7) / 8) * kv_heads * (dim / 4) : 0);
     hipLaunchKernelGGL(rotate_and_store_vector_kernel, dim3((unsigned)((threads + 255) / 256)), dim3(256), 0, stream,
-                       (bf16_t*)qkv, (const float2*)table, pairing, heads, kv_heads, dim, (bf16_t*)keys,
+                       (bf16_t*)qkv, row_stride, (const float2*)table, pairing, heads, kv_heads, dim, (bf16_t*)keys,
                        (bf16_t*)values, slots, page_size, tokens);
     return LAUNCH_STATUS();
   }
   if (is_float)
-    hipLaunchKernelGGL(rotate_and_store_kernel<float>, dim3(tokens), dim3(256), 0, stream, (float*)qkv,
+    hipLaunchKernelGGL(rotate_and_store_kernel<float>, dim3(tokens), dim3(256), 0, stream, (float*)qkv, row_stride,
                        (const float2*)table, pairing, heads, kv_heads, dim, (float*)keys, (float*)values, slots,
                        page_size);
   else
-    hipLaunchKernelGGL(rotate_and_store_kernel<bf16_t>, dim3(tokens), dim3(256), 0, stream, (bf16_t*)qkv,
+    hipLaunchKernelGGL(rotate_and_store_kernel<bf16_t>, dim3(tokens), dim3(256), 0, stream, (bf16_t*)qkv, row_stride,
                        (const float2*)table, pairing, heads, kv_heads, dim, (bf16_t*)keys, (bf16_t*)values, slots,
                        page_size);
   return LAUNCH_STATUS();
@@ -549,6 +550,7 @@ extern "C" int llmserve_rotate_and_store(void* qkv, int is_float, const float* t
 // 4: a function of gate and up both, with a limit: g = min(gate, limit), u = clamp(up, -limit, limit),
 // g * sigmoid(1.702 g) * (u + 1)
 #define ACT_LIMITED_SWISH 4
+#define ACT_SQUARED_RELU 5
 
 __device__ __forceinline__ float limited_swish(float gate, float up, float limit) {
   const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
@@ -560,6 +562,7 @@ __device__ __forceinline__ float gate_activation(int activation, float z) {
     case ACT_GELU: return 0.5f * z * (1.f + erff(z * 0.70710678118654752f));
     case ACT_GELU_TANH: return 0.5f * z * (1.f + tanhf(0.79788456080286536f * (z + 0.044715f * z * z * z)));
     case ACT_RELU: return fmaxf(z, 0.f);
+    case ACT_SQUARED_RELU: return fmaxf(z, 0.f) * fmaxf(z, 0.f);
     default: return z / (1.f + expf(-z));
   }
 }
@@ -613,7 +616,7 @@ __global__ __launch_bounds__(256) void silu_mul_vector_kernel(const bf16_t* __re
 extern "C" int llmserve_gate_mul_limit(const void* in, int in_is_float, void* out, int out_is_float, int rows, int width,
                                        int activation, float limit, hipStream_t stream) {
   if (rows <= 0) return 0;
-  if (activation < ACT_SILU || activation > ACT_LIMITED_SWISH || (activation == ACT_LIMITED_SWISH && !(limit > 0.f))) return ERR_BAD_ARGUMENT;
+  if (activation < ACT_SILU || activation > ACT_SQUARED_RELU || (activation == ACT_LIMITED_SWISH && !(limit > 0.f))) return ERR_BAD_ARGUMENT;
   if (activation == ACT_LIMITED_SWISH && !in_is_float && !out_is_float && width % 8 == 0) {
     const size_t octets = (size_t)rows * (width / 8);
     hipLaunchKernelGGL(limited_swish_vector_kernel, dim3((unsigned)((octets + 255) / 256)), dim3(256), 0, stream,

@@ -21,6 +21,7 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 // a function of gate and up both, with a limit (gated results only): g = min(gate, limit), u = clamp(up, -limit, limit),
 // g * sigmoid(1.702 g) * (u + 1)
 #define ACT_LIMITED_SWISH 4
+#define ACT_SQUARED_RELU 5
 
 __device__ __forceinline__ float activation_of(int activation, float z) {
   switch (activation) {
@@ -28,6 +29,7 @@ __device__ __forceinline__ float activation_of(int activation, float z) {
     case ACT_GELU: return 0.5f * z * (1.f + erff(z * 0.70710678118654752f));
     case ACT_GELU_TANH: return 0.5f * z * (1.f + tanhf(0.79788456080286536f * (z + 0.044715f * z * z * z)));
     case ACT_RELU: return fmaxf(z, 0.f);
+    case ACT_SQUARED_RELU: return fmaxf(z, 0.f) * fmaxf(z, 0.f);
     default: return z / (1.f + expf(-z));
   }
 }

@@ -407,7 +407,7 @@ extern "C" int llmserve_assemble_heads(const void* x, int is_float, int tokens, 
                                        void* keys, void* values, const int* slots, int page_size, int pairing, hipStream_t stream) {
   if (tokens <= 0) return 0;
   if (pairing < 1 || pairing > 2) return ERR_BAD_ARGUMENT;
-  if (heads < 1 || kv_heads < 1 || dim < 1 || vdim < 1 || width < dim || width < vdim || norm < 0 || norm > 2 ||
+  if (heads < 1 || kv_heads < 0 || (kv_heads == 0 && slots) || dim < 1 || vdim < 1 || width < dim || width < vdim || norm < 0 || norm > 2 ||
       (norm && (!q_weight || !k_weight)) || rot_dims < 0 || rot_dims % 2 || rot_dims > dim || (rot_dims && !table) ||
       q_first < 0 || k_first < 0 || v_first < 0 || q_first + heads * dim > x_width || k_first + kv_heads * dim > x_width ||
       v_first + kv_heads * vdim > x_width || (other && (other_first < 0 || other_first + kv_heads * vdim > other_width)))

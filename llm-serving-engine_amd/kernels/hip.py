@@ -20,7 +20,7 @@ from .build import _say, load_module
 
 _PAIRINGS = {"none": 0, "adjacent": 1, "half": 2}
 # gate activations of a gated product (csrc/elementwise.hip: gate_activation); the products' fused epilogues know silu alone
-_ACTIVATIONS = {"silu": 0, "gelu": 1, "gelu_tanh": 2, "relu": 3, "limited_swish": 4}  # (the last is a function of gate and up both, with a limit)
+_ACTIVATIONS = {"silu": 0, "gelu": 1, "gelu_tanh": 2, "relu": 3, "limited_swish": 4, "squared_relu": 5}  # (limited_swish is a function of gate and up both, with a limit)
 _GATED_RESULT = 16  # added to an activation's code: the experts' product gates its own result
 
 
@@ -48,10 +48,10 @@ def _pointer(tensor: torch.Tensor | None) -> int | None:
 # Argument types of every entry point: p pointer, i int, f float.  Declared once, so that a call
 # costs no guessing: a decode step is replayed from a graph, but every other step pays per launch.
 _SIGNATURES = {
-    "llmserve_embedding": "pippiip",
+    "llmserve_embedding": "pippiifp",
     "llmserve_add_rms_norm": "ppipipiiifp",
     "llmserve_rotary_table": "pppiip",
-    "llmserve_rotate_and_store": "pipiiiiipppip",
+    "llmserve_rotate_and_store": "piipiiiiipppip",
     "llmserve_silu_mul": "pipiiip",
     "llmserve_gate_mul": "pipiiiip",
     "llmserve_gate_mul_limit": "pipiiiifp",
@@ -68,10 +68,10 @@ _SIGNATURES = {
     "llmserve_gemm_ring": "pppipiiiiiiip",
     "llmserve_gemm_merged": "ppippipiiiip",
     "llmserve_gemm_tiled": "pppipiiiiiip",
-    "llmserve_attention_generic": "pipipppippiiiiifipfpip",
-    "llmserve_attention_f32": "pippppppippiiiiiifiipfpip",
-    "llmserve_attention_tiles": "pippppppippiiiiiifiiipippfpip",
-    "llmserve_attention_portions": "pippppppippiiiiiifiip",
+    "llmserve_attention_generic": "pipiipppippiiiiifipfpiip",
+    "llmserve_attention_f32": "pipipppppippiiiiiifiipfpiip",
+    "llmserve_attention_tiles": "pipipppppippiiiiiifiiipippfpiip",
+    "llmserve_attention_portions": "pipipppppippiiiiiifiip",
     "llmserve_attention_can_fuse": "i",
     "llmserve_argmax": "ppppiip",
     "llmserve_argmax_static": "ppiip",
@@ -80,9 +80,10 @@ _SIGNATURES = {
     "llmserve_add_layer_norm": "ppippipiiifp",
     "llmserve_rms_norm_columns": "piiiiipifpiiiip",
     "llmserve_rotary_table_scaled": "pppiifp",
-    "llmserve_rotate_columns": "piiiiiiipipiiip",
+    "llmserve_rotate_columns": "piiiiiiipipiiiip",
     "llmserve_join_rows": "ppippiiip",
     "llmserve_activate": "ppiiiip",
+    "llmserve_activate_columns": "piiiipiiiip",
     "llmserve_add_gated_rows": "pppiiiip",
     "llmserve_headwise_linear": "piiiiipiiipiiip",
     "llmserve_route": "piipifppiiiiip",
@@ -260,11 +261,11 @@ class HipKernels:
 
     # ------------------------------------------------------------------ elementwise
 
-    def embedding(self, table: torch.Tensor, token_ids: torch.Tensor) -> torch.Tensor:
+    def embedding(self, table: torch.Tensor, token_ids: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
         tokens, hidden = token_ids.shape[0], table.shape[1]
         out = self._empty((tokens, hidden), torch.float32)
         status = self._elementwise.llmserve_embedding(
-            _pointer(table), _is_float(table), _pointer(token_ids), _pointer(out), tokens, hidden, self._stream
+            _pointer(table), _is_float(table), _pointer(token_ids), _pointer(out), tokens, hidden, float(scale), self._stream
         )
         _check(status, "embedding")
         return out
@@ -304,7 +305,7 @@ class HipKernels:
 
     def rotate_and_store(self, qkv, layout, batch, cell, inverse_frequencies, pairing: str) -> None:
         tokens = qkv.shape[0]
-        if qkv.shape[1] != layout.width:
+        if qkv.shape[1] != layout.stride:
             raise KernelError("rotate_and_store: qkv does not have the layout's width")
         store = cell is not None and cell.writable
         group = batch.groups[cell.group] if store else None
@@ -312,7 +313,7 @@ class HipKernels:
             raise KernelError("rotate_and_store: the cell's pages do not fit the layout")
         table = self.rotary_table(batch, inverse_frequencies) if pairing != "none" else None
         status = self._elementwise.llmserve_rotate_and_store(
-            _pointer(qkv), _is_float(qkv), _pointer(table), _PAIRINGS[pairing], tokens, layout.num_heads,
+            _pointer(qkv), layout.stride, _is_float(qkv), _pointer(table), _PAIRINGS[pairing], tokens, layout.num_heads,
             layout.num_kv_heads, layout.head_dim, _pointer(cell.keys if store else None),
             _pointer(cell.values if store else None), _pointer(group.slot_mapping if store else None),
             group.page_size if store else 1, self._stream,
@@ -811,13 +812,14 @@ class HipKernels:
     def paged_attention(
         self, qkv, layout, batch, cell, scale: float, window: int | None, *,
         score_slopes: torch.Tensor | None = None, soft_cap: float | None = None, sinks: torch.Tensor | None = None,
-        keep_first: int = 0,
+        keep_first: int = 0, chunk: int | None = None, out: torch.Tensor | None = None,
     ) -> torch.Tensor:
         """`score_slopes` (float32 [heads]) and `soft_cap` change the scores before the softmax: cap * tanh(score /
         cap), then minus slope * distance; `sinks` (float32 [heads]) add exp(sink) to a head's denominator; with
         `keep_first` a sequence's first so many keys stay visible behind the window, at their own positions.  The
         matrix-core kernels of both precisions take them (in bfloat16 not the forms that fuse the rotation or share
-        keys through LDS)."""
+        keys through LDS).  `chunk` is a mask instead of a window: a query sees the keys of its own chunk of so many positions.
+        With `out` (rows of the run dtype, as wide as the heads or wider) the result is its first columns."""
         tokens = qkv.shape[0]
         group = batch.groups[cell.group]
         if cell.keys.dtype != qkv.dtype:
@@ -831,30 +833,50 @@ class HipKernels:
         keep_first = int(keep_first or 0) if window else 0
         if keep_first < 0 or keep_first != int(getattr(cell.need, "keep_first", 0) or 0):
             raise KernelError("paged_attention: keep_first is what the cell's pages are kept for")
-        out = self._empty((tokens, layout.num_heads * layout.head_dim), qkv.dtype)
+        chunk = int(chunk or 0)
+        if chunk < 0 or (chunk and window):
+            raise KernelError("paged_attention: a mask is a window or chunks")
+        if qkv.shape[1] != layout.stride:
+            raise KernelError("paged_attention: qkv does not have the layout's width")
+        out = self._attention_out(qkv, layout, out)
         dim = layout.head_dim
-        plain_scores = score_slopes is None and soft_cap is None and sinks is None and not keep_first
-        if qkv.dtype == torch.bfloat16 and group.page_size % 8 == 0 and dim % 16 == 0 and 16 <= dim <= 256:
-            changed = None if plain_scores else (score_slopes, float(soft_cap or 0.0), sinks, keep_first)
+        plain_scores = score_slopes is None and soft_cap is None and sinks is None and not keep_first and not chunk
+        aligned = layout.stride % 8 == 0 and out.shape[1] % 8 == 0  # (rows are read and written in pieces of 8 or 16 bytes)
+        if qkv.dtype == torch.bfloat16 and group.page_size % 8 == 0 and dim % 16 == 0 and 16 <= dim <= 256 and aligned:
+            changed = None if plain_scores else (score_slopes, float(soft_cap or 0.0), sinks, keep_first, chunk)
             self._attention_tiles(qkv, out, layout, batch, cell, group, scale, int(window or 0), changed=changed)
             return out
-        if qkv.dtype == torch.float32 and group.page_size % 4 == 0 and dim % 16 == 0 and 16 <= dim <= 256:
-            self._attention_float32(qkv, out, layout, batch, cell, group, scale, int(window or 0), score_slopes, soft_cap, sinks, keep_first)
+        if qkv.dtype == torch.float32 and group.page_size % 4 == 0 and dim % 16 == 0 and 16 <= dim <= 256 and aligned:
+            self._attention_float32(qkv, out, layout, batch, cell, group, scale, int(window or 0), score_slopes, soft_cap, sinks, keep_first, chunk)
             return out
         if qkv.dtype == torch.bfloat16:
             why = f"head size {dim} and pages of {group.page_size}"
             self._tell_once(f"generic attention: {why}", f"bfloat16 attention runs on the generic kernel, not on the matrix cores: {why}")
         status = self._attention_generic.llmserve_attention_generic(
-            _pointer(qkv), layout.width, _pointer(out), _is_float(qkv), _pointer(cell.keys), _pointer(cell.values),
+            _pointer(qkv), layout.stride, _pointer(out), out.shape[1], _is_float(qkv), _pointer(cell.keys), _pointer(cell.values),
             _pointer(group.block_tables), group.width, _pointer(batch.token_sequence), _pointer(batch.positions),
             tokens, layout.num_heads, layout.num_kv_heads, dim, group.page_size,
-            scale, int(window or 0), _pointer(score_slopes), float(soft_cap or 0.0), _pointer(sinks), keep_first, self._stream,
+            scale, int(window or 0), _pointer(score_slopes), float(soft_cap or 0.0), _pointer(sinks), keep_first, chunk, self._stream,
         )
         _check(status, "paged_attention")
         return out
 
+    def _attention_out(self, qkv, layout, out) -> torch.Tensor:
+        wanted = layout.num_heads * layout.head_dim
+        if out is None:
+            return self._empty((qkv.shape[0], wanted), qkv.dtype)
+        if out.dtype != qkv.dtype or out.ndim != 2 or out.shape[0] != qkv.shape[0] or out.shape[1] < wanted:
+            raise KernelError("paged_attention: the rows to write are of the queries' type, one a token, and wide enough")
+        return out
+
+    @staticmethod
+    def _walked_keys(batch, window: int, keep_first: int, chunk: int) -> int:
+        """The most keys that one query of the step walks."""
+        reach = window + keep_first if window else chunk
+        return min(batch.max_context_length, reach) if reach else batch.max_context_length
+
     def _attention_float32(self, qkv, out, layout, batch, cell, group, scale: float, window: int, score_slopes=None, soft_cap=None, sinks=None,
-                           keep_first: int = 0) -> None:
+                           keep_first: int = 0, chunk: int = 0) -> None:
         """The 32-bit path's attention on the matrix cores: an item is 16 (decoding) or 32 columns of one
         request, (token, head) pairs running through the tokens head by head whatever the number of heads; few
         items over long contexts are cut into key splits that a second kernel merges."""
@@ -872,17 +894,17 @@ class HipKernels:
         # walk is as long as its steps are many: where the chip has room for more workgroups the keys are split
         # until a wave has two steps or so (a decode step of 8 requests over 530 keys: 61 us unsplit; the merge
         # kernel costs about 5).
-        steps = -(-batch.max_context_length // 16)
+        steps = -(-self._walked_keys(batch, window, keep_first, chunk) // 16)
         splits = max(1, min(32, 1024 // (items * kv_heads), steps // 8))
         partial_acc = partial_ml = None
         if splits > 1:
             partial_acc = self._empty((splits, tokens * heads, dim), torch.float32)
             partial_ml = self._empty((splits, tokens * heads, 2), torch.float32)
         status = self._attention_f32[dim].llmserve_attention_f32(
-            _pointer(qkv), layout.width, _pointer(out), _pointer(partial_acc), _pointer(partial_ml), _pointer(cell.keys),
+            _pointer(qkv), layout.stride, _pointer(out), out.shape[1], _pointer(partial_acc), _pointer(partial_ml), _pointer(cell.keys),
             _pointer(cell.values), _pointer(group.block_tables), group.width, _pointer(batch.positions), _pointer(work),
             items, column_tiles, tokens, heads, kv_heads, group.page_size, scale, window, splits, _pointer(score_slopes),
-            float(soft_cap or 0.0), _pointer(sinks), keep_first, self._stream,
+            float(soft_cap or 0.0), _pointer(sinks), keep_first, chunk, self._stream,
         )
         _check(status, "paged_attention")
 
@@ -893,12 +915,12 @@ class HipKernels:
         store inside the same kernel.  With `unmerged` (a step of single tokens whose reader merges
         key splits itself) the keys are split more finely and the splits are returned as they are
         (their results in bfloat16, laid out for `gemm_merged`; their maxima and sums in float32; how
-        many), instead of `out`.  `changed` = (slopes or None, soft cap or 0.0, sinks or None, kept first keys or 0): scores
-        changed before the softmax, a sink in its denominator, or a sequence's first keys kept visible behind the window, which neither
-        `fuse` nor the kernel that shares keys through LDS takes."""
-        if changed is not None and fuse is not None:
-            raise KernelError("paged_attention: the fused decode form takes plain scores only")
-        slopes, soft_cap, sinks, keep_first = changed if changed is not None else (None, 0.0, None, 0)
+        many), instead of `out`.  `changed` = (slopes or None, soft cap or 0.0, sinks or None, kept first keys or 0, chunk or 0): scores
+        changed before the softmax, a sink in its denominator, a sequence's first keys kept visible behind the window, or a mask
+        in chunks, which the kernel that shares keys through LDS does not take; `fuse` takes sinks and chunks alone."""
+        slopes, soft_cap, sinks, keep_first, chunk = changed if changed is not None else (None, 0.0, None, 0, 0)
+        if fuse is not None and (slopes is not None or soft_cap or keep_first):
+            raise KernelError("paged_attention: the fused decode form leaves the scores as they are")
         library = self._attention_library(layout.head_dim)
         heads, kv_heads = layout.num_heads, layout.num_kv_heads
         per_tile = max(1, 16 // (heads // kv_heads))
@@ -948,7 +970,7 @@ class HipKernels:
                 partial_acc = self._empty((tokens * heads * splits * layout.head_dim,), torch.float32)
                 partial_ml = self._empty((tokens * heads * splits * 2,), torch.float32)
             status = library.llmserve_attention_portions(
-                _pointer(qkv), layout.width, _pointer(out), _pointer(partial_acc), _pointer(partial_ml), _pointer(cell.keys),
+                _pointer(qkv), layout.stride, _pointer(out), out.shape[1], _pointer(partial_acc), _pointer(partial_ml), _pointer(cell.keys),
                 _pointer(cell.values), _pointer(group.block_tables), group.width, _pointer(batch.positions), _pointer(work),
                 items, 2, tokens, heads, kv_heads, group.page_size, scale, window, splits, self._stream,
             )
@@ -989,7 +1011,7 @@ class HipKernels:
                 # requests over 4,096 keys 40.6 / 47.4, over 2,500 27.2 / 33.4, over 1,500 18.8 / 21.8; 32 over
                 # 8,192 44.0 / 47.0; 16 over 16,384 43.9 / 48.1; up to 8 requests as before).
                 blocks = items * kv_heads * head_tiles
-                steps = -(-batch.max_context_length // 32)
+                steps = -(-self._walked_keys(batch, window, keep_first, chunk) // 32)
                 splits = max(1, min(-(-steps // 32), max(1, 192 // blocks), 64))
                 if unmerged:
                     # Nothing merges in a kernel of its own here, so a split costs only what its reader pays to
@@ -1025,10 +1047,10 @@ class HipKernels:
                     partial_ml = self._empty((held * heads * splits * 2,), torch.float32)
             table, pairing = fuse if fuse is not None else (None, "none")
             status = library.llmserve_attention_tiles(
-                _pointer(qkv), layout.width, _pointer(out), _pointer(partial_acc), _pointer(partial_ml),
+                _pointer(qkv), layout.stride, _pointer(out), out.shape[1], _pointer(partial_acc), _pointer(partial_ml),
                 _pointer(cell.keys), _pointer(cell.values), _pointer(group.block_tables), group.width, _pointer(batch.positions), _pointer(work), items, column_tiles, tokens, heads, kv_heads,
                 group.page_size, scale, window, splits, (1 if fuse is not None else 0) + (2 if unmerged else 0) + (4 if by_item else 0),
-                _pointer(table), _PAIRINGS[pairing], _pointer(group.slot_mapping), _pointer(slopes), soft_cap, _pointer(sinks), keep_first, self._stream,
+                _pointer(table), _PAIRINGS[pairing], _pointer(group.slot_mapping), _pointer(slopes), soft_cap, _pointer(sinks), keep_first, chunk, self._stream,
             )
             _check(status, "paged_attention")
             if unmerged and splits > 1:
@@ -1037,18 +1059,20 @@ class HipKernels:
 
     def rotate_store_attend(
         self, qkv, layout, batch, cell, inverse_frequencies, pairing: str, scale: float, window: int | None,
-        project: LinearWeights | None = None,
+        project: LinearWeights | None = None, *, sinks: torch.Tensor | None = None, chunk: int | None = None, out: torch.Tensor | None = None,
     ) -> torch.Tensor:
         """`rotate_and_store` followed by `paged_attention`; one kernel when every request of
         the step brings a single token and the MFMA kernel takes the sizes.  With `project`, the result
         is `linear(that, project, float32, partial=True)`: for up to 16 single tokens at head size 128
         the attention leaves its key splits unmerged and the product merges them as it loads its x."""
-        out, projected = self._rotate_store_attend(qkv, layout, batch, cell, inverse_frequencies, pairing, scale, window, project)
+        if project is not None and out is not None:
+            raise KernelError("rotate_store_attend: the result goes to given rows or through a product")
+        out, projected = self._rotate_store_attend(qkv, layout, batch, cell, inverse_frequencies, pairing, scale, window, project, sinks, chunk, out)
         if project is None or projected:
             return out
         return self.linear(out, project, out_dtype=torch.float32, partial=True)
 
-    def _rotate_store_attend(self, qkv, layout, batch, cell, inverse_frequencies, pairing, scale, window, project):
+    def _rotate_store_attend(self, qkv, layout, batch, cell, inverse_frequencies, pairing, scale, window, project, sinks, chunk, out):
         """(the attention's output, False) or, where the key splits were left to the product, (the product's, True)."""
         group = batch.groups[cell.group]
         dim = layout.head_dim
@@ -1060,13 +1084,21 @@ class HipKernels:
             and group.page_size % 8 == 0
             and dim % 16 == 0
             and 16 <= dim <= 256
+            and layout.stride % 8 == 0
+            and (out is None or out.shape[1] % 8 == 0)
             and self._attention_library(dim).llmserve_attention_can_fuse(_PAIRINGS[pairing])
         ):
-            out = self._empty((qkv.shape[0], layout.num_heads * dim), qkv.dtype)
+            if sinks is not None and (sinks.dtype != torch.float32 or sinks.shape != (layout.num_heads,)):
+                raise KernelError("paged_attention: sinks is one float32 per query head")
+            if qkv.shape[1] != layout.stride or (chunk and window) or int(getattr(cell.need, "keep_first", 0) or 0):
+                raise KernelError("rotate_store_attend: rows of the layout's width, a window or chunks, and no kept first keys")
+            out = self._attention_out(qkv, layout, out)
             table = self.rotary_table(batch, inverse_frequencies) if pairing != "none" else None
             rows = qkv.shape[0]
             merging = (
                 project is not None
+                and sinks is None
+                and not chunk
                 and self.merge_in_product
                 and dim == 128
                 and rows <= 16
@@ -1080,7 +1112,8 @@ class HipKernels:
                 # 3.29 / 3.67 with the merging kernel): what decides is the weight, so the gate is its size.
                 and project.weight.numel() * project.weight.element_size() <= self.merge_weight_bytes
             )
-            left = self._attention_tiles(qkv, out, layout, batch, cell, group, scale, int(window or 0), fuse=(table, pairing), unmerged=merging)
+            left = self._attention_tiles(qkv, out, layout, batch, cell, group, scale, int(window or 0), fuse=(table, pairing), unmerged=merging,
+                                         changed=(None, 0.0, sinks, 0, int(chunk or 0)) if sinks is not None or chunk else None)
             if left is None:
                 return out, False
             split_x, split_ml, splits = left
@@ -1096,7 +1129,7 @@ class HipKernels:
             _check(status, "linear over unmerged key splits")
             return result, True
         self.rotate_and_store(qkv, layout, batch, cell, inverse_frequencies, pairing)
-        return self.paged_attention(qkv, layout, batch, cell, scale, window), False
+        return self.paged_attention(qkv, layout, batch, cell, scale, window, sinks=sinks, chunk=chunk, out=out), False
 
     # ------------------------------------------------------------------ layer norm, runs of columns
 
@@ -1131,13 +1164,16 @@ class HipKernels:
         _check(status, "rms_norm_columns")
         return out
 
-    def rotate_columns(self, x, first: int, head_stride: int, heads: int, width: int, table, dims: int, out, out_first: int, out_head_stride: int):
+    def rotate_columns(self, x, first: int, head_stride: int, heads: int, width: int, table, dims: int, out, out_first: int, out_head_stride: int,
+                       pairing: str = "adjacent"):
         tokens = x.shape[0]
+        if pairing not in ("adjacent", "half"):
+            raise KernelError(f"rotate_columns: no kernel turns pairs that are {pairing!r}")
         if out.dtype != x.dtype or out.shape[0] != tokens or table.shape != (tokens, dims // 2, 2) or table.dtype != torch.float32:
             raise KernelError("rotate_columns: rows of one type, and a table entry for every pair of every token")
         status = self._library_of("columns").llmserve_rotate_columns(
             _pointer(x), _is_float(x), tokens, x.shape[1], first, head_stride, heads, width, _pointer(table), dims, _pointer(out),
-            out.shape[1], out_first, out_head_stride, self._stream,
+            out.shape[1], out_first, out_head_stride, 1 if pairing == "half" else 0, self._stream,
         )
         _check(status, "rotate_columns")
         return out
@@ -1154,9 +1190,33 @@ class HipKernels:
         _check(status, "join_rows")
         return out
 
+    @staticmethod
+    def _plain_activation(activation: str, what: str) -> int:
+        if activation not in _ACTIVATIONS or activation == "limited_swish":
+            known = ", ".join(name for name in _ACTIVATIONS if name != "limited_swish")
+            raise KernelError(f"{what}: no kernel applies the activation {activation!r} (known: {known})")
+        return _ACTIVATIONS[activation]
+
+    def activated_linear(self, x, weights: LinearWeights, activation: str, first: int = 0, out=None, out_first: int = 0):
+        """The product, and the activation on its columns from `first` on, written to a tensor of their own or to the
+        columns of `out` from `out_first`."""
+        code = self._plain_activation(activation, "activated_linear")
+        width = weights.out_features - first
+        if not 0 <= first < weights.out_features:
+            raise KernelError("activated_linear: the activation begins at a column of the product")
+        if out is None:
+            out = self._empty((x.shape[0], width), self.dtype)
+        if out.dtype != self.dtype or out.shape[0] != x.shape[0] or not 0 <= out_first <= out.shape[1] - width:
+            raise KernelError("activated_linear: the rows to write are of the run dtype, one a token, and wide enough")
+        rows = self.linear(x, weights)
+        status = self._library_of("columns").llmserve_activate_columns(
+            _pointer(rows), _is_float(rows), rows.shape[0], rows.shape[1], first, _pointer(out), out.shape[1], out_first, width, code, self._stream
+        )
+        _check(status, "activated_linear")
+        return rows, out
+
     def activate(self, x, activation: str) -> torch.Tensor:
-        if activation not in _ACTIVATIONS:
-            raise KernelError(f"activate: no kernel applies the activation {activation!r} (known: {', '.join(_ACTIVATIONS)})")
+        self._plain_activation(activation, "activate")
         out = torch.empty_like(x)
         status = self._library_of("columns").llmserve_activate(
             _pointer(x), _pointer(out), _is_float(x), x.shape[0], x.shape[1], _ACTIVATIONS[activation], self._stream
@@ -1474,7 +1534,7 @@ class HipKernels:
         )
         _check(status, "assemble_heads")
         if store and not here:
-            layout = types.SimpleNamespace(num_heads=heads, num_kv_heads=kv_heads, head_dim=width, width=(heads + 2 * kv_heads) * width)
+            layout = types.SimpleNamespace(num_heads=heads, num_kv_heads=kv_heads, head_dim=width, stride=out.shape[1])
             self.rotate_and_store(out, layout, batch, cell, None, "none")
         return out
 

@@ -23,8 +23,8 @@ class Kernels(Protocol):
     def queued_to_device(self, tensor: torch.Tensor) -> torch.Tensor:
         """As `to_device`, for small per-step inputs: the host does not wait for work queued before."""
 
-    def embedding(self, table: torch.Tensor, token_ids: torch.Tensor) -> torch.Tensor:
-        """float32 rows [T, hidden] of `table` at `token_ids`."""
+    def embedding(self, table: torch.Tensor, token_ids: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
+        """float32 rows [T, hidden] of `table` at `token_ids`, times `scale`."""
 
     def add_rms_norm(
         self, hidden: torch.Tensor, delta: torch.Tensor | None, weight: torch.Tensor, eps: float
@@ -36,7 +36,7 @@ class Kernels(Protocol):
 
     def prepare_gated_linear(self, gate: torch.Tensor, up: torch.Tensor, activation: str = "silu", limit: float | None = None) -> Any:
         """Gate and up weights [I, K] in whatever layout `gated_linear` wants; `activation` is the gate's
-        (silu, gelu, gelu_tanh, relu), and one the library has no kernel for is refused here, by name.
+        (silu, gelu, gelu_tanh, relu, squared_relu), and one the library has no kernel for is refused here, by name.
         "limited_swish" is a function of gate and up both and has a `limit`: g = min(gate, limit), u = clamp(up,
         -limit, limit), and the result is g * sigmoid(1.702 g) * (u + 1)."""
 
@@ -49,18 +49,27 @@ class Kernels(Protocol):
     def gated_linear(self, x: torch.Tensor, weights: Any) -> torch.Tensor:
         """act(x Wg^T) * (x Wu^T) -> [T, I] in the run dtype."""
 
+    def activated_linear(
+        self, x: torch.Tensor, weights: Any, activation: str, first: int = 0, out: torch.Tensor | None = None, out_first: int = 0,
+    ) -> tuple[torch.Tensor | None, torch.Tensor]:
+        """y = x W^T + bias [T, N]; its columns from `first` on, through the activation, to a new [T, N - first] tensor or to
+        the columns of `out`'s rows from `out_first` -> (rows whose first `first` columns are y's, with or without more behind
+        them; the tensor that holds the activated columns), both in the run dtype."""
+
     def rotate_and_store(
         self, qkv: torch.Tensor, layout: Any, batch: Any, cell: Any,
         inverse_frequencies: torch.Tensor | None, pairing: str,
     ) -> None:
-        """Rotary on the q and k heads of `qkv` in place; k and v into the cell's pages if it is writable."""
+        """Rotary on the q and k heads of `qkv` in place; k and v into the cell's pages if it is writable.  (`layout.stride`
+        columns a row of qkv, of which the layout's heads are the first.)"""
 
     def paged_attention(
         self, qkv: torch.Tensor, layout: Any, batch: Any, cell: Any, scale: float, window: int | None, *,
         score_slopes: torch.Tensor | None = None, soft_cap: float | None = None, sinks: torch.Tensor | None = None,
-        keep_first: int = 0,
+        keep_first: int = 0, chunk: int | None = None, out: torch.Tensor | None = None,
     ) -> torch.Tensor:
-        """Attention of the q heads of `qkv` over the cell's pages -> [T, heads * head_dim].
+        """Attention of the q heads of `qkv` over the cell's pages -> [T, heads * head_dim], or the first columns of `out`'s
+        rows.  With `chunk` (and no window) a query at p sees the keys at k <= p with k // chunk == p // chunk.
         Before the softmax a score s of a query at position p for a key at position k may be changed,
         for encodings and models that want it (Qwen2 wants neither): with `soft_cap`, to
         soft_cap * tanh(s / soft_cap); with `score_slopes` (float32, one per query head), by
@@ -72,7 +81,7 @@ class Kernels(Protocol):
     def rotate_store_attend(
         self, qkv: torch.Tensor, layout: Any, batch: Any, cell: Any,
         inverse_frequencies: torch.Tensor | None, pairing: str, scale: float, window: int | None,
-        project: Any = None,
+        project: Any = None, *, sinks: torch.Tensor | None = None, chunk: int | None = None, out: torch.Tensor | None = None,
     ) -> torch.Tensor:
         """`rotate_and_store` followed by `paged_attention` (a library may fuse them); with `project` (what
         `prepare_linear` returned), followed by `linear(that, project, float32, partial=True)`, whose result
@@ -100,10 +109,11 @@ class Kernels(Protocol):
 
     def rotate_columns(
         self, x: torch.Tensor, first: int, head_stride: int, heads: int, width: int, table: torch.Tensor, dims: int,
-        out: torch.Tensor, out_first: int, out_head_stride: int,
+        out: torch.Tensor, out_first: int, out_head_stride: int, pairing: str = "adjacent",
     ) -> torch.Tensor:
         """For every head h: `width` columns of x from first + h * head_stride to out from out_first + h *
-        out_head_stride; the first `dims` of them rotated in adjacent pairs by the token's table row, the rest copied."""
+        out_head_stride; the first `dims` of them rotated in pairs (`pairing` "adjacent": (2i, 2i + 1); "half": (i, i + dims /
+        2)) by the token's table row, the rest copied."""
 
     def prepare_headwise_linear(self, weight: torch.Tensor) -> Any:
         """[heads, N, K] weights in whatever layout `headwise_linear` wants."""
@@ -119,7 +129,7 @@ class Kernels(Protocol):
         """[hidden + delta | embedded] in the run dtype, [T, 2 hidden]."""
 
     def activate(self, x: torch.Tensor, activation: str) -> torch.Tensor:
-        """act(x) elementwise (silu, gelu, gelu_tanh, relu), in x's type."""
+        """act(x) elementwise (silu, gelu, gelu_tanh, relu, squared_relu), in x's type."""
 
     def add_gated_rows(self, target: torch.Tensor, rows: torch.Tensor, gates: torch.Tensor, column: int, squash: str) -> torch.Tensor:
         """target += squash(gates[:, column]) * rows, float32, in place."""

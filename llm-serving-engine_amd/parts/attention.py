@@ -3,7 +3,7 @@
 from __future__ import annotations
 
 from dataclasses import dataclass
-from typing import Any
+from typing import Any, ClassVar
 
 import torch
 
@@ -16,9 +16,21 @@ class Mixer(Part):
     in the run dtype and returns the float32 rows [T, hidden] to add to the
     residual stream, or partial sums [parts, T, hidden] of them (whoever adds
     them to the stream adds the parts in order).  `cell` is what `cache_need`
-    asked for."""
+    asked for.
+
+    A mixer that begins and ends with a product may leave both to the block around it, which joins them with those
+    of another sublayer that reads the same rows (`ParallelBlock`).  Such a mixer has `joins` True and a field
+    `joined` in its spec; built with it set, it prepares neither product and shows them instead: `opening`, a list of
+    (weight [N, hidden], bias or None), whose results side by side are the first columns of the rows that `mix(projected,
+    batch, cell, out)` reads; and `closing`, (weight [hidden, K], bias or None), whose operand `mix` writes to the first
+    K columns of `out`'s rows."""
+
+    joins: ClassVar[bool] = False
 
     def forward(self, x: torch.Tensor, batch, cell) -> torch.Tensor:
+        raise NotImplementedError
+
+    def mix(self, projected: torch.Tensor, batch, cell, out: torch.Tensor) -> None:
         raise NotImplementedError
 
 

@@ -10,6 +10,7 @@ by registering a class: nothing else changes.
 
 from __future__ import annotations
 
+import math
 from dataclasses import dataclass
 from typing import Any, ClassVar
 
@@ -59,10 +60,25 @@ class CacheNeed:
 class PagedNeed(CacheNeed):
     """An entry per token.  A subclass has a field `window` (keys at most that are ever read again, None:
     all), may have a field `keep_first` (so many entries at a request's start are read for ever, whatever the
-    window), and says what one page holds."""
+    window) and one `chunk` (instead of a window: a query reads the entries of its own chunk of so many positions,
+    counted from the request's start), and says what one page holds."""
 
     window: int | None = None
     keep_first: int = 0
+    chunk: int | None = None
+
+    def first_read(self, position: int) -> int:
+        """No query at `position` or later reads an entry before the one returned (the first `keep_first` aside)."""
+        if self.window is not None:
+            return max(0, position - self.window + 1)
+        if self.chunk is not None:
+            return position - position % self.chunk
+        return 0
+
+    def shared_with(self, other: "CacheNeed") -> "CacheNeed | None":
+        """The need of one cell that runs with this need and with `other` both read: None where the two differ in what an
+        entry is, else one that keeps entries as long as either asks."""
+        return self if other == self else None
 
     def page_fields(self, page_size: int) -> dict[str, tuple[int, ...]]:
         """name -> shape of ONE page of that field.  The cache keeps each field as a tensor
@@ -97,6 +113,27 @@ class PagedKeyValue(PagedNeed):
     head_dim: int
     window: int | None = None
     keep_first: int = 0
+    chunk: int | None = None
+
+    def __post_init__(self) -> None:
+        if self.window is not None and self.chunk is not None:
+            raise ValueError("keys and values are read through a window or in chunks, not both")
+
+    def shared_with(self, other: CacheNeed) -> "PagedKeyValue | None":
+        if not isinstance(other, PagedKeyValue) or (other.num_kv_heads, other.head_dim) != (self.num_kv_heads, self.head_dim):
+            return None
+        if other == self:
+            return self
+        window = chunk = None
+        if self.window is not None and other.window is not None:
+            window = max(self.window, other.window)
+        elif self.keep_first or other.keep_first:
+            return None
+        elif self.chunk is not None and other.chunk is not None:
+            chunk = math.lcm(self.chunk, other.chunk)  # a chunk of either size lies in one of these
+        if self.keep_first != other.keep_first:  # (readers say what a cell keeps: those of one cell agree on it)
+            return None
+        return PagedKeyValue(self.num_kv_heads, self.head_dim, window, self.keep_first, chunk)
 
     def page_fields(self, page_size: int) -> dict[str, tuple[int, ...]]:
         width = key_piece_width(self.head_dim)
@@ -210,3 +247,13 @@ def under(tensors: dict[str, Any], prefix: str) -> dict[str, Any]:
 
 def prefixed(tensors: dict[str, Any], prefix: str) -> dict[str, Any]:
     return {prefix + name: value for name, value in tensors.items()}
+
+
+def side_by_side(products: list[tuple[torch.Tensor, torch.Tensor | None]]) -> tuple[list[torch.Tensor], list[torch.Tensor] | None]:
+    """(weight [N, K], bias or None) of several products over the same rows, as one product's lists of weights and of
+    biases: zeros where only some have a bias, None where none has."""
+    known = [bias for _, bias in products if bias is not None]
+    if not known:
+        return [weight for weight, _ in products], None
+    biases = [torch.zeros((weight.shape[0],), dtype=known[0].dtype, device=known[0].device) if bias is None else bias for weight, bias in products]
+    return [weight for weight, _ in products], biases

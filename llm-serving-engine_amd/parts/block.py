@@ -2,12 +2,13 @@
 
 from __future__ import annotations
 
+import dataclasses
 from dataclasses import dataclass
 from typing import Any
 
 import torch
 
-from .base import BLOCKS, FEED_FORWARDS, MIXERS, NORMS, CacheNeed, Part, TensorSpec, prefixed, under
+from .base import BLOCKS, FEED_FORWARDS, MIXERS, NORMS, CacheNeed, Part, TensorSpec, prefixed, side_by_side, under
 
 
 class Block(Part):
@@ -226,3 +227,79 @@ class SandwichBlock(Block):
         )
         fed = self.feed_forward.forward(normed, batch)
         return PendingNormed(fed, self.feed_forward_out, self.feed_forward_out_eps, kernels)
+
+
+@dataclass(frozen=True)
+class ParallelBlockSpec:
+    """h += mixer(norm(h)) + feed_forward(norm(h)): one norm, whose rows both sublayers read.  A layer without a feed-forward
+    has `feed_forward` None.  The `*_name` fields are the prefixes of the members' tensors below the layer's own prefix."""
+
+    norm: Any
+    mixer: Any
+    feed_forward: Any
+    norm_name: str = "norm1"
+    mixer_name: str = "mix."
+    feed_forward_name: str = "mlp."
+    kind: str = "parallel"
+
+
+@BLOCKS.register("parallel")
+class ParallelBlock(Block):
+    """Where mixer and feed-forward both begin and end with a product (`joins`), the two first products are one over the
+    weights side by side, and the two last ones are one over the operands side by side, W_o m + W_d a = [W_o | W_d] [m; a]:
+    the sum of the sublayers is made in the product's float32 accumulators, and a layer is two launches of products
+    instead of four and no add.  Else the results are added by a kernel."""
+
+    @classmethod
+    def _members(cls, spec: ParallelBlockSpec):
+        members = [(spec.norm_name, NORMS, spec.norm), (spec.mixer_name, MIXERS, spec.mixer)]
+        if spec.feed_forward is not None:
+            members.append((spec.feed_forward_name, FEED_FORWARDS, spec.feed_forward))
+        return members
+
+    @classmethod
+    def tensors(cls, spec: ParallelBlockSpec) -> dict[str, TensorSpec]:
+        found: dict[str, TensorSpec] = {}
+        for name, registry, member in cls._members(spec):
+            found.update(prefixed(registry.tensors(member), name))
+        return found
+
+    @classmethod
+    def cache_need(cls, spec: ParallelBlockSpec) -> CacheNeed:
+        return MIXERS.cache_need(spec.mixer)
+
+    def __init__(self, spec: ParallelBlockSpec, tensors, kernels) -> None:
+        super().__init__(spec, tensors, kernels)
+        may_join = spec.feed_forward is not None and all(
+            getattr(registry.get(member), "joins", False) and hasattr(member, "joined") for _, registry, member in self._members(spec)[1:]
+        )
+        members = [(name, registry, dataclasses.replace(member, joined=True) if may_join and registry is not NORMS else member)
+                   for name, registry, member in self._members(spec)]
+        built = [registry.build(member, under(tensors, name), kernels) for name, registry, member in members]
+        self.norm, self.mixer = built[:2]
+        self.feed_forward = built[2] if spec.feed_forward is not None else None
+        self.replayable = all(part.replayable for part in built)
+        self.opening = None
+        if may_join:
+            mixer, feed_forward = self.mixer, self.feed_forward
+            self.split = sum(weight.shape[0] for weight, _ in mixer.opening)  # columns of the first product that the mixer reads
+            self.opening = kernels.prepare_linear(*side_by_side(mixer.opening + feed_forward.opening))
+            weights, biases = zip(mixer.closing, feed_forward.closing)
+            self.mixed_width, self.inner_width = weights[0].shape[1], sum(weight.shape[1] for weight in weights)
+            biases = [bias for bias in biases if bias is not None]
+            if len(biases) > 1:
+                biases = [biases[0].float() + biases[1].float()]
+            self.closing = kernels.prepare_linear([torch.cat(weights, dim=1)], biases or None)
+
+    def forward(self, hidden, delta, batch, cell) -> torch.Tensor:
+        kernels = self.kernels
+        normed = self.norm.forward(hidden, delta)
+        if self.opening is not None:
+            inner = kernels.new_rows(normed.shape[0], self.inner_width)  # [the mixer's | the feed-forward's]
+            projected, _ = kernels.activated_linear(normed, self.opening, self.feed_forward.activation, self.split, out=inner, out_first=self.mixed_width)
+            self.mixer.mix(projected, batch, cell, inner)
+            return kernels.linear(inner, self.closing, out_dtype=torch.float32, partial=True)
+        mixed = self.mixer.forward(normed, batch, cell)
+        if self.feed_forward is None:
+            return mixed
+        return kernels.add_scaled(mixed, 1.0, self.feed_forward.forward(normed, batch), 1.0)

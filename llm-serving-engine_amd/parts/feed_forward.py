@@ -57,3 +57,44 @@ class GatedMLP(FeedForward):
     def forward(self, x: torch.Tensor, batch) -> torch.Tensor:
         activated = self.kernels.gated_linear(x, self.gate_up)
         return self.kernels.linear(activated, self.down, out_dtype=torch.float32, partial=True)
+
+
+@dataclass(frozen=True)
+class DenseMLPSpec:
+    """`names`: the tensors' names below the part's prefix: up, down.  `joined`: as a mixer's (`Mixer`): both products are
+    the block's."""
+
+    hidden_size: int
+    intermediate_size: int
+    activation: str = "squared_relu"
+    names: tuple[str, str] = ("up", "down")
+    joined: bool = False
+    kind: str = "dense_mlp"
+
+
+@FEED_FORWARDS.register("dense_mlp")
+class DenseMLP(FeedForward):
+    """down(act(up(x))) without biases."""
+
+    joins = True
+
+    @classmethod
+    def tensors(cls, spec: DenseMLPSpec) -> dict[str, TensorSpec]:
+        up, down = spec.names
+        return {
+            up: TensorSpec((spec.intermediate_size, spec.hidden_size)),
+            down: TensorSpec((spec.hidden_size, spec.intermediate_size)),
+        }
+
+    def __init__(self, spec: DenseMLPSpec, tensors, kernels) -> None:
+        super().__init__(spec, tensors, kernels)
+        up, down = (tensors[name] for name in spec.names)
+        self.activation = spec.activation
+        self.opening, self.closing = [(up, None)], (down, None)
+        if not spec.joined:
+            self.up = kernels.prepare_linear([up], None)
+            self.down = kernels.prepare_linear([down], None)
+
+    def forward(self, x: torch.Tensor, batch) -> torch.Tensor:
+        _, inner = self.kernels.activated_linear(x, self.up, self.activation)
+        return self.kernels.linear(inner, self.down, out_dtype=torch.float32, partial=True)

@@ -8,7 +8,7 @@ from typing import Any
 
 import torch
 
-from .base import BLOCKS, LOGIT_PARTS, NORMS, PASS_PARTS, STREAM_PARTS, CacheNeed, TensorSpec, prefixed, under
+from .base import BLOCKS, LOGIT_PARTS, NORMS, PASS_PARTS, STREAM_PARTS, CacheNeed, PagedNeed, TensorSpec, prefixed, under
 
 
 @dataclass(frozen=True)
@@ -22,7 +22,8 @@ class LayerRun:
     """One entry of the run order.  `layer` indexes `ModelSpec.layers`; a layer
     may be named by several entries (its tensors are shared, each run has a
     cache cell of its own).  With `reads` set, the run uses the cell of that
-    earlier entry of the run order instead, and stores nothing.  With `enters` set, the run is
+    earlier entry of the run order instead, and stores nothing (the cell keeps entries as long as the run that
+    fills it or one that reads it asks: they may look back differently far).  With `enters` set, the run is
     the first of a pass (its number: 0, 1, ...) through layers that the model walks several times, and
     the model's `pass_entry` part acts on the stream before it."""
 
@@ -56,6 +57,8 @@ class ModelSpec:
     output_parts: tuple[NamedPart, ...] = ()
     # the part that stands before every run with `enters` set (a kind of PASS_PARTS)
     pass_entry: NamedPart | None = None
+    # the embedded rows are the table's times this
+    embedding_scale: float = 1.0
     # tensors that a model folder may hold and the model does not use
     ignored_tensors: tuple[str, ...] = ()
 
@@ -70,12 +73,21 @@ class ModelSpec:
                     raise ValueError(f"run {index} reads the cache of run {run.reads}, which is not earlier")
                 if self.run_order[run.reads].reads is not None:
                     raise ValueError(f"run {index} reads run {run.reads}, which owns no cache")
-                if self.cell_need(run.reads) != self.cell_need(index):
-                    raise ValueError(f"run {index} and run {run.reads} need different caches")
+                self.cell_need(index)  # (refuses runs that cannot share a cell)
 
-    def cell_need(self, run_index: int) -> CacheNeed:
-        block = self.layers[self.run_order[run_index].layer].block
-        return BLOCKS.cache_need(block)
+    def cell_need(self, run_index: int) -> "CacheNeed | dict[str, CacheNeed] | None":
+        """What the run's cell has to be: what the run itself needs, joined with what the runs that read its cell need."""
+        owner = self.run_order[run_index].reads
+        owner = run_index if owner is None else owner
+        need = BLOCKS.cache_need(self.layers[self.run_order[owner].layer].block)
+        for index, run in enumerate(self.run_order):
+            if run.reads == owner:
+                other = BLOCKS.cache_need(self.layers[run.layer].block)
+                joined = need.shared_with(other) if isinstance(need, PagedNeed) else need if other == need else None
+                if joined is None and other != need:
+                    raise ValueError(f"run {index} and run {owner} need different caches")
+                need = joined
+        return need
 
     def tensors(self) -> dict[str, TensorSpec]:
         """Every tensor of the model by its name in the model folder."""
@@ -103,6 +115,7 @@ class DecoderModel:
         self.spec = spec
         self.kernels = kernels
         self.embedding = tensors[spec.embedding_name]
+        self._embedding_scale = (float(spec.embedding_scale),) if spec.embedding_scale != 1.0 else ()
         self.layers = [
             BLOCKS.build(layer.block, under(tensors, layer.prefix), kernels) for layer in spec.layers
         ]
@@ -123,7 +136,7 @@ class DecoderModel:
         self.observer = None
 
     def _run_layers(self, batch, cells: list):
-        hidden = self.kernels.embedding(self.embedding, batch.token_ids)
+        hidden = self.kernels.embedding(self.embedding, batch.token_ids, *self._embedding_scale)
         for part in self.input_parts:  # (in place, or a new stream of another shape: copies side by side)
             changed = part.forward(hidden, batch)
             hidden = hidden if changed is None else changed

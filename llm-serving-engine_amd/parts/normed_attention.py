@@ -1,15 +1,16 @@
-"""Attention over a sliding window whose queries and keys are normed, with the options some designs put around
-it: heads rotated in part, capped scores, a sink in the softmax's denominator, values blended with an earlier
-layer's, and a gate a head on the result."""
+"""Attention over a sliding window or in chunks whose queries and keys may be normed, with the options some designs put
+around it: heads rotated in part, capped scores, a sink in the softmax's denominator, values blended with an earlier
+layer's, keys and values read from an earlier layer's cache, and a gate a head on the result."""
 
 from __future__ import annotations
 
+import dataclasses
 from dataclasses import dataclass
 
 import torch
 
 from .attention import Mixer
-from .base import MIXERS, PagedKeyValue, TensorSpec
+from .base import MIXERS, PagedKeyValue, TensorSpec, side_by_side
 from .position import HeadLayout, LinearScaling, WavelengthScaling, YarnScaling, rotary_frequencies
 
 
@@ -28,7 +29,12 @@ class NormedAttentionSpec:
     `values`: None, "give" (the step's values are shown to later layers under `values_name`) or "take" (v <- (1 - a) v
     + a v_given with the learned number a; the blended v is what is cached).
     `keep_first`: under a window, the first so many tokens of a sequence stay visible to every later query, at their
-    own positions (a query at p sees the keys at j <= p with p - j < window or j < keep_first)."""
+    own positions (a query at p sees the keys at j <= p with p - j < window or j < keep_first).
+    `chunk`: instead of a window, a query at p sees the keys at j <= p with j // chunk == p // chunk.
+    `own_keys` False: the layer has no key and value projections, it attends over the cell of the earlier layer run that its
+    `LayerRun.reads` names, with queries of its own.
+    `bias` is of the q, k and v projections, `out_bias` of the last.  `joined`: the first and the last product are the
+    block's (`Mixer`)."""
 
     hidden_size: int
     num_heads: int
@@ -50,7 +56,16 @@ class NormedAttentionSpec:
     values: str | None = None
     values_name: str = "values"
     keep_first: int = 0
+    chunk: int | None = None
+    own_keys: bool = True
+    out_bias: bool = False
+    joined: bool = False
     kind: str = "normed_attention"
+
+    @property
+    def stored_heads(self) -> int:
+        """Key/value heads that the layer projects and stores itself."""
+        return self.num_kv_heads if self.own_keys else 0
 
     @property
     def head_width(self) -> int:
@@ -66,19 +81,23 @@ class NormedAttention(Mixer):
 
     The heads go to the engine's paged attention as rows of `head_width`: a key's or value's columns beyond its own
     size are zeros, which change neither a score nor a result's own columns, and the output projection's weight has
-    zero columns where the results do.  Norms, angles, cosines and sines, the blend and the gate are float32."""
+    zero columns where the results do.  Norms, angles, cosines and sines, the blend and the gate are float32.  Where the
+    projections are already such rows (sizes of `head_width`, nothing to do to a head) the attention reads them as they lie."""
+
+    joins = True
 
     @classmethod
     def tensors(cls, spec: NormedAttentionSpec) -> dict[str, TensorSpec]:
         q_size, k_size, v_size = spec.num_heads * spec.dim, spec.num_kv_heads * spec.dim, spec.num_kv_heads * spec.vdim
-        found = {
-            "q": TensorSpec((q_size, spec.hidden_size)),
-            "k": TensorSpec((k_size, spec.hidden_size)),
-            "v": TensorSpec((v_size, spec.hidden_size)),
-            "o": TensorSpec((spec.hidden_size, spec.num_heads * spec.vdim)),
-        }
+        found = {"q": TensorSpec((q_size, spec.hidden_size)), "o": TensorSpec((spec.hidden_size, spec.num_heads * spec.vdim))}
+        if spec.own_keys:
+            found.update({"k": TensorSpec((k_size, spec.hidden_size)), "v": TensorSpec((v_size, spec.hidden_size))})
         if spec.bias:
-            found.update({"q.b": TensorSpec((q_size,), role="bias"), "k.b": TensorSpec((k_size,), role="bias"), "v.b": TensorSpec((v_size,), role="bias")})
+            found["q.b"] = TensorSpec((q_size,), role="bias")
+            if spec.own_keys:
+                found.update({"k.b": TensorSpec((k_size,), role="bias"), "v.b": TensorSpec((v_size,), role="bias")})
+        if spec.out_bias:
+            found["o.b"] = TensorSpec((spec.hidden_size,), role="bias")
         if spec.norm == "head":
             found.update({"q.norm": TensorSpec((spec.dim,), role="norm"), "k.norm": TensorSpec((spec.dim,), role="norm")})
         elif spec.norm == "row":
@@ -93,7 +112,9 @@ class NormedAttention(Mixer):
 
     @classmethod
     def cache_need(cls, spec: NormedAttentionSpec) -> PagedKeyValue:
-        return PagedKeyValue(spec.num_kv_heads, spec.head_width, spec.window, spec.keep_first if spec.window is not None else 0)
+        return PagedKeyValue(
+            spec.num_kv_heads, spec.head_width, spec.window, spec.keep_first if spec.window is not None else 0, spec.chunk,
+        )
 
     def __init__(self, spec: NormedAttentionSpec, tensors, kernels) -> None:
         super().__init__(spec, tensors, kernels)
@@ -107,16 +128,21 @@ class NormedAttention(Mixer):
             raise ValueError("normed attention: the rotated dimensions are an even number within dim")
         if spec.keep_first < 0:
             raise ValueError("normed attention: keep_first counts tokens")
+        if spec.window is not None and spec.chunk is not None:
+            raise ValueError("normed attention: a mask is a window or chunks")
+        if not spec.own_keys and (spec.norm is not None or spec.values is not None or spec.gate):
+            raise ValueError("normed attention: norms, blended values and gates are of layers with keys of their own")
+        if spec.joined and spec.gate:
+            raise ValueError("normed attention: gates are made beside the queries by the layer's own product")
         self.keep_first = spec.keep_first if spec.window is not None else 0
         heads, width = spec.num_heads, spec.head_width
-        self.layout = HeadLayout(heads, spec.num_kv_heads, width)
-        names = ["q", "k", "v"] + (["g"] if spec.gate else [])
-        biases = None
-        if spec.bias:
-            biases = [tensors["q.b"], tensors["k.b"], tensors["v.b"]]
-            if spec.gate:
-                biases.append(torch.zeros((heads,), dtype=biases[0].dtype, device=biases[0].device))
-        self.inputs = kernels.prepare_linear([tensors[name] for name in names], biases)  # [q | k | v | gates]
+        self.layout = HeadLayout(heads, spec.num_kv_heads, width, None if spec.own_keys else heads * width)
+        # nothing to do to the projections' heads: they are what the attention reads
+        self.direct = spec.norm is None and not spec.rot_dims and spec.values != "take" and spec.dim == spec.vdim == width and not spec.gate
+        names = ["q", "k", "v"] if spec.own_keys else ["q"]
+        self.opening = [(tensors[name], tensors[name + ".b"] if spec.bias else None) for name in names]
+        if spec.gate:
+            self.opening.append((tensors["g"], None))
         self.q_norm = tensors.get("q.norm") if spec.norm else None
         self.k_norm = tensors.get("k.norm") if spec.norm else None
         self.blend = float(tensors["vmix"].float()) if spec.values == "take" else 0.0
@@ -126,7 +152,10 @@ class NormedAttention(Mixer):
             wide = torch.zeros((spec.hidden_size, heads, width), dtype=out.dtype, device=out.device)
             wide[:, :, : spec.vdim] = out.view(spec.hidden_size, heads, spec.vdim)
             out = wide.view(spec.hidden_size, heads * width)
-        self.out = kernels.prepare_linear([out.contiguous()], None)
+        self.closing = (out.contiguous(), tensors["o.b"] if spec.out_bias else None)
+        if not spec.joined:
+            self.inputs = kernels.prepare_linear(*side_by_side(self.opening))  # [q | k | v | gates]
+            self.out = kernels.prepare_linear([self.closing[0]], [self.closing[1]] if spec.out_bias else None)
         self.frequencies = None
         if spec.rot_dims:
             shared = kernels.__dict__.setdefault("_rotary_frequencies", {})
@@ -138,8 +167,21 @@ class NormedAttention(Mixer):
 
     def forward(self, x: torch.Tensor, batch, cell) -> torch.Tensor:
         kernels, spec = self.kernels, self.spec
-        q_size, k_size, v_size = spec.num_heads * spec.dim, spec.num_kv_heads * spec.dim, spec.num_kv_heads * spec.vdim
         projected = kernels.linear(x, self.inputs)  # [T, q | k | v | gates]
+        plain = spec.soft_cap is None and self.sinks is None and not spec.gate and not self.keep_first and spec.chunk is None and spec.own_keys
+        if plain:  # the output projection goes with the attention: a kernel library may fuse the two
+            rows, layout = self._rows(projected, batch, None)
+            return kernels.rotate_store_attend(rows, layout, batch, cell, None, "none", spec.scale, spec.window, project=self.out)
+        mixed = self.mix(projected, batch, cell, None)
+        if spec.gate:
+            kernels.scale_heads(mixed, spec.num_heads, spec.head_width, projected, spec.num_heads * spec.dim + spec.stored_heads * (spec.dim + spec.vdim), "sigmoid")
+        return kernels.linear(mixed, self.out, out_dtype=torch.float32, partial=True)
+
+    def _rows(self, projected, batch, cell):
+        """Per token the heads' queries, keys and values as the attention reads them (normed, turned, blended, widened),
+        and their layout; with a `cell` the keys and values are stored too, unless the rows are the projections."""
+        kernels, spec = self.kernels, self.spec
+        q_size, k_size, v_size = spec.num_heads * spec.dim, spec.stored_heads * spec.dim, spec.stored_heads * spec.vdim
         given = None
         if spec.values == "give":
             batch.computed[("given values", spec.values_name)] = (projected, q_size + k_size, v_size)
@@ -147,21 +189,32 @@ class NormedAttention(Mixer):
             given = batch.computed.get(("given values", spec.values_name))
             if given is None or given[2] != v_size:
                 raise RuntimeError("normed attention: no earlier layer of this step gave values of this size")
+        if self.direct and projected.shape[1] % 8 == 0:
+            return projected, dataclasses.replace(self.layout, row_stride=projected.shape[1])
         table = kernels.rotary_table(batch, self.frequencies, self.magnitude) if spec.rot_dims else None
-        # per token the heads' queries, keys and values as the attention reads them: normed, turned, blended, widened
-        plain = spec.soft_cap is None and self.sinks is None and not spec.gate and not self.keep_first
         rows = kernels.assemble_heads(
-            projected, 0, q_size, q_size + k_size, spec.num_heads, spec.num_kv_heads, spec.dim, spec.vdim, spec.head_width,
+            projected, 0, q_size, q_size + k_size, spec.num_heads, spec.stored_heads, spec.dim, spec.vdim, spec.head_width,
             spec.norm, self.q_norm, self.k_norm, spec.eps, table, spec.rot_dims,
             given[0] if given else None, given[1] if given else 0, self.blend,
-            batch=batch, cell=None if plain else cell,  # (with plain scores the attention below stores, and may fuse that)
-            pairing=spec.pairing,
+            batch=batch, cell=cell if spec.own_keys else None, pairing=spec.pairing,
         )
-        if plain:
-            return kernels.rotate_store_attend(rows, self.layout, batch, cell, None, "none", spec.scale, spec.window, project=self.out)
-        mixed = kernels.paged_attention(
-            rows, self.layout, batch, cell, spec.scale, spec.window, soft_cap=spec.soft_cap, sinks=self.sinks, keep_first=self.keep_first,
+        return rows, self.layout
+
+    def mix(self, projected: torch.Tensor, batch, cell, out: torch.Tensor | None) -> torch.Tensor:
+        kernels, spec = self.kernels, self.spec
+        scores_as_they_are = spec.soft_cap is None and not self.keep_first
+        if self.direct and scores_as_they_are and spec.own_keys:
+            rows, layout = self._rows(projected, batch, None)
+            if rows is projected:  # keys and values are stored by the attention's own kernel where it can
+                return kernels.rotate_store_attend(
+                    rows, layout, batch, cell, None, "none", spec.scale, spec.window, sinks=self.sinks, chunk=spec.chunk, out=out,
+                )
+            kernels.rotate_and_store(rows, layout, batch, cell, None, "none")
+        else:
+            rows, layout = self._rows(projected, batch, cell)
+            if rows is projected and spec.own_keys:
+                kernels.rotate_and_store(rows, layout, batch, cell, None, "none")
+        return kernels.paged_attention(
+            rows, layout, batch, cell, spec.scale, spec.window, soft_cap=spec.soft_cap, sinks=self.sinks, keep_first=self.keep_first,
+            chunk=spec.chunk, out=out,
         )
-        if spec.gate:
-            kernels.scale_heads(mixed, spec.num_heads, spec.head_width, projected, q_size + k_size + v_size, "sigmoid")
-        return kernels.linear(mixed, self.out, out_dtype=torch.float32, partial=True)

@@ -12,15 +12,22 @@ from .base import POSITIONS, Part
 
 @dataclass(frozen=True)
 class HeadLayout:
-    """How one token's projected row is laid out: q heads, then k heads, then v heads."""
+    """How one token's projected row is laid out: q heads, then k heads, then v heads, and, where a row is
+    `row_stride` wide, other things behind them (or the q heads alone, for attention over keys that are cached)."""
 
     num_heads: int
     num_kv_heads: int
     head_dim: int
+    row_stride: int | None = None
 
     @property
     def width(self) -> int:
         return (self.num_heads + 2 * self.num_kv_heads) * self.head_dim
+
+    @property
+    def stride(self) -> int:
+        """Elements from one token's row to the next."""
+        return self.width if self.row_stride is None else self.row_stride
 
 
 @dataclass(frozen=True)

@@ -25,6 +25,15 @@ def _limited_swish(gate, up, limit):
     return g * torch.sigmoid(1.702 * g) * (up.clamp(-limit, limit) + 1.0)
 
 
+_ACTIVATIONS = {
+    "silu": torch.nn.functional.silu,
+    "gelu": torch.nn.functional.gelu,
+    "gelu_tanh": lambda z: torch.nn.functional.gelu(z, approximate="tanh"),
+    "relu": torch.relu,
+    "squared_relu": lambda z: torch.relu(z) ** 2,
+}
+
+
 class TorchKernels:
     def __init__(self, dtype: torch.dtype = torch.float32) -> None:
         self.device = torch.device("cpu")
@@ -37,8 +46,8 @@ class TorchKernels:
     def queued_to_device(self, tensor):
         return tensor
 
-    def embedding(self, table, token_ids):
-        return table[token_ids.long()].float()
+    def embedding(self, table, token_ids, scale=1.0):
+        return table[token_ids.long()].float() * scale
 
     def add_rms_norm(self, hidden, delta, weight, eps):
         if delta is not None:
@@ -52,8 +61,7 @@ class TorchKernels:
         return _Linear(weight, bias)
 
     def prepare_gated_linear(self, gate, up, activation="silu", limit=None):
-        acts = {"silu": torch.nn.functional.silu, "gelu": torch.nn.functional.gelu, "relu": torch.relu,
-                "gelu_tanh": lambda z: torch.nn.functional.gelu(z, approximate="tanh")}
+        acts = _ACTIVATIONS
         if activation == "limited_swish":
             if limit is None or not limit > 0:
                 raise ValueError("gated_linear: limited_swish has a positive limit")
@@ -78,7 +86,8 @@ class TorchKernels:
     def rotate_and_store(self, qkv, layout, batch, cell, inverse_frequencies, pairing):
         tokens = qkv.shape[0]
         heads, kv_heads, dim = layout.num_heads, layout.num_kv_heads, layout.head_dim
-        view = qkv.view(tokens, heads + 2 * kv_heads, dim)
+        assert qkv.shape[1] == layout.stride
+        view = qkv[:, : layout.width].unflatten(1, (heads + 2 * kv_heads, dim))  # (a view: what is turned is written back)
         if pairing != "none":
             angles = batch.positions.float()[:, None] * inverse_frequencies[None, :]
             cos, sin = angles.cos()[:, None, :], angles.sin()[:, None, :]
@@ -99,17 +108,19 @@ class TorchKernels:
             cell.put_key_rows(pages, offsets, view[:, heads : heads + kv_heads])  # pages are [kv, dim / w, offset, w]
             cell.put_value_rows(pages, offsets, view[:, heads + kv_heads :])  # pages are [kv, offset / v, dim, v]
 
-    def paged_attention(self, qkv, layout, batch, cell, scale, window, *, score_slopes=None, soft_cap=None, sinks=None, keep_first=0):
+    def paged_attention(self, qkv, layout, batch, cell, scale, window, *, score_slopes=None, soft_cap=None, sinks=None, keep_first=0,
+                        chunk=None, out=None):
         tokens = qkv.shape[0]
         heads, kv_heads, dim = layout.num_heads, layout.num_kv_heads, layout.head_dim
-        queries = qkv.view(tokens, heads + 2 * kv_heads, dim)[:, :heads].float()
+        assert qkv.shape[1] == layout.stride
+        queries = qkv[:, : heads * dim].unflatten(1, (heads, dim)).float()
         group = batch.groups[cell.group]
-        out = torch.zeros(tokens, heads, dim)
+        given, out = out, torch.zeros(tokens, heads, dim)
         row = 0
-        for b, chunk in enumerate(batch.chunks):
+        for b, portion in enumerate(batch.chunks):
             table = group.block_tables[b].long()
-            for position in range(chunk.start, chunk.start + chunk.count):
-                first = 0 if window is None else max(0, position - window + 1)
+            for position in range(portion.start, portion.start + portion.count):
+                first = position // chunk * chunk if chunk else 0 if window is None else max(0, position - window + 1)
                 where = torch.arange(first, position + 1)
                 if keep_first and first > 0:  # the sequence's first tokens stay visible, at their own positions
                     where = torch.cat([torch.arange(0, min(keep_first, first)), where])
@@ -130,11 +141,16 @@ class TorchKernels:
                 else:
                     out[row] = torch.einsum("hn,nhd->hd", torch.softmax(scores, dim=-1), values)
                 row += 1
-        return out.reshape(tokens, heads * dim).to(self.dtype)
+        result = out.reshape(tokens, heads * dim).to(self.dtype)
+        if given is None:
+            return result
+        given[:, : heads * dim] = result
+        return given
 
-    def rotate_store_attend(self, qkv, layout, batch, cell, inverse_frequencies, pairing, scale, window, project=None):
+    def rotate_store_attend(self, qkv, layout, batch, cell, inverse_frequencies, pairing, scale, window, project=None, *, sinks=None, chunk=None,
+                            out=None):
         self.rotate_and_store(qkv, layout, batch, cell, inverse_frequencies, pairing)
-        mixed = self.paged_attention(qkv, layout, batch, cell, scale, window)
+        mixed = self.paged_attention(qkv, layout, batch, cell, scale, window, sinks=sinks, chunk=chunk, out=out)
         return mixed if project is None else self.linear(mixed, project, out_dtype=torch.float32, partial=True)
 
     def gather_rows(self, hidden, delta, rows):
@@ -193,14 +209,15 @@ class TorchKernels:
         angles = batch.positions.float()[:, None] * frequencies.float()[None, :]
         return torch.stack([angles.cos() * magnitude, angles.sin() * magnitude], dim=-1)
 
-    def rotate_columns(self, x, first, head_stride, heads, width, table, dims, out, out_first, out_head_stride):
+    def rotate_columns(self, x, first, head_stride, heads, width, table, dims, out, out_first, out_head_stride, pairing="adjacent"):
+        one, two = (slice(0, dims, 2), slice(1, dims, 2)) if pairing == "adjacent" else (slice(0, dims // 2), slice(dims // 2, dims))
         cos, sin = table[..., 0], table[..., 1]
         for head in range(heads):
             part = x[:, first + head * head_stride : first + head * head_stride + width].float()
             turned = part.clone()
-            a, b = part[:, 0:dims:2], part[:, 1:dims:2]
-            turned[:, 0:dims:2] = a * cos - b * sin
-            turned[:, 1:dims:2] = b * cos + a * sin
+            a, b = part[:, one], part[:, two]
+            turned[:, one] = a * cos - b * sin
+            turned[:, two] = b * cos + a * sin
             out[:, out_first + head * out_head_stride : out_first + head * out_head_stride + width] = turned.to(out.dtype)
         return out
 
@@ -222,9 +239,15 @@ class TorchKernels:
         return torch.cat([now, embedded], dim=-1).to(self.dtype)
 
     def activate(self, x, activation):
-        acts = {"silu": torch.nn.functional.silu, "gelu": torch.nn.functional.gelu, "relu": torch.relu,
-                "gelu_tanh": lambda z: torch.nn.functional.gelu(z, approximate="tanh")}
-        return acts[activation](x.float()).to(x.dtype)
+        return _ACTIVATIONS[activation](x.float()).to(x.dtype)
+
+    def activated_linear(self, x, weights, activation, first=0, out=None, out_first=0):
+        rows = self.linear(x, weights)  # (rounded to the run dtype before the activation)
+        width = rows.shape[1] - first
+        if out is None:
+            out = torch.zeros((x.shape[0], width), dtype=self.dtype)
+        out[:, out_first : out_first + width] = self.activate(rows[:, first:], activation)
+        return rows, out
 
     def add_gated_rows(self, target, rows, gates, column, squash):
         assert squash == "sigmoid"
