@@ -43,6 +43,11 @@ and number of layer runs (the engine's other decoder with the delta rule and rou
 
 measures the fifth (configs/vagozen-w1536.json, configs/vagozen-w3584.json) beside the Sozavik models (window attention, a
 decaying state, norms behind the sublayers), the Dafutar models (latent attention, experts, layers walked twice) and the Qwen2 models.
+
+    python bench.py --op dolezen
+
+measures the sixth (configs/dolezen-w1536.json, configs/dolezen-w3584.json) beside the Sozavik models (window attention with
+a sink), the Vagozen models (latent attention) and the Qwen2 models.
 """
 
 from __future__ import annotations
@@ -84,7 +89,7 @@ def parse() -> argparse.Namespace:
                         help="leave out decoding at contexts of 8k and 30k (batch 8) and 4k (batch 64), and the long prompts")
     parser.add_argument("--skip-other-models", action="store_true",
                         help="leave out the float32 run and the 7B and 32B layer sizes")
-    parser.add_argument("--op", choices=("decode-attention", "prefill-attention", "dafutar", "sozavik", "katenex", "vagozen"), default=None,
+    parser.add_argument("--op", choices=("decode-attention", "prefill-attention", "dafutar", "sozavik", "katenex", "vagozen", "dolezen"), default=None,
                         help="measure one operation alone instead, as the reference's kernel benchmark does")
     return parser.parse_args()
 
@@ -441,6 +446,8 @@ def main() -> int:
         return katenex_table(args)
     if args.op == "vagozen":
         return vagozen_table(args)
+    if args.op == "dolezen":
+        return dolezen_table(args)
 
     import torch
 
@@ -597,6 +604,14 @@ def vagozen_table(args) -> int:
     two layer sizes beside the Sozavik, the Dafutar and the Qwen2 of the same width, number of layer runs and vocabulary,
     measured as `dafutar_table` measures."""
     return beside_qwen2(args, "vagozen", "Vagozen", also=("sozavik", "dafutar"))
+
+
+def dolezen_table(args) -> int:
+    """The Dolezen decoder (one norm for mixer and feed-forward; layers of attention in chunks with a sink, every other one of
+    them over an earlier layer's keys and values, and of latent attention over a window; squared relu) at two layer sizes
+    beside the Sozavik, the Vagozen and the Qwen2 of the same width, number of layer runs and vocabulary, measured as
+    `dafutar_table` measures."""
+    return beside_qwen2(args, "dolezen", "Dolezen", also=("sozavik", "vagozen"))
 
 
 def beside_qwen2(args, name: str, title: str, also: tuple[str, ...] = ()) -> int:
