@@ -28,7 +28,28 @@ __device__ __forceinline__ bf16x8 load8_stream(const bf16_t* p) { return *(const
 #define TARGET_WAVES 2048
 #endif
 
-// GATED in the kernels for up to 64 rows below: 0 a plain product, 1 silu(gate) * up, 2 relu(gate) * up
+// GATED in the kernels for up to 64 rows below: 0 a plain product, 1 silu(gate) * up, 2 relu(gate) * up, 3 a plain product
+// whose columns from `Tail::first` on are activated (relu(z)^2) and go to rows of their own
+struct Tail {
+  bf16_t* rows;  // column n of row m, n >= first, goes to rows[m * stride + n - first]; a column below `first` to out[m * first + n]
+  int first, stride;
+};
+
+template <typename TO>
+__device__ __forceinline__ void store_with_tail(TO* out, const Tail& tail, int m, int n_first, int N, f32x4 total) {
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int n = n_first + i;
+    if (n >= N) break;
+    if (n < tail.first) {
+      out[(size_t)m * tail.first + n] = from_float<TO>(total[i]);
+    } else {
+      const float z = fmaxf(total[i], 0.f);
+      tail.rows[(size_t)m * tail.stride + n - tail.first] = (bf16_t)(z * z);
+    }
+  }
+}
+
 template <int GATED>
 __device__ __forceinline__ float gate_value(float gate) {
   return GATED == 2 ? fmaxf(gate, 0.f) : gate / (1.f + expf(-gate));
@@ -39,7 +60,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_kernel(const bf16_t* _
                                                                  const bf16_t* __restrict__ w,
                                                                  const void* __restrict__ bias, int bias_is_float,
                                                                  TO* __restrict__ out, int M, int N, int K,
-                                                                 int k_split) {
+                                                                 int k_split, Tail tail) {
   extern __shared__ float partial[];  // [WAVES][MT][64 lanes][4]
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int r = lane & 15, g = lane >> 4;
@@ -132,7 +153,9 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_kernel(const bf16_t* _
     for (int i = 0; i < 4; ++i)
       total[i] += __uint_as_float((unsigned)bias_high[i] << 16 | (bias_is_float ? (unsigned)bias_low[i] : 0u));
   }
-  if (GATED) {
+  if (GATED == 3) {
+    store_with_tail(out, tail, m, n_first, N, total);
+  } else if (GATED) {
     TO* dst = out + (size_t)m * (N / 2) + n_first / 2;
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
@@ -151,31 +174,31 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_kernel(const bf16_t* _
 
 template <int WAVES, int MT, typename TO, int GATED>
 static int launch_skinny(const void* x, const void* w, const void* bias, int bias_is_float, void* out, int M, int N,
-                         int K, int splits, hipStream_t stream) {
+                         int K, int splits, hipStream_t stream, Tail tail = {}) {
   const size_t lds = (size_t)WAVES * MT * 64 * 4 * sizeof(float);
   hipLaunchKernelGGL((gemm_skinny_kernel<WAVES, MT, TO, GATED>), dim3((N + 15) / 16, splits), dim3(WAVES * 64), lds,
-                     stream, (const bf16_t*)x, (const bf16_t*)w, bias, bias_is_float, (TO*)out, M, N, K, K / splits);
+                     stream, (const bf16_t*)x, (const bf16_t*)w, bias, bias_is_float, (TO*)out, M, N, K, K / splits, tail);
   return LAUNCH_STATUS();
 }
 
 template <int WAVES, typename TO, int GATED>
 static int pick_tiles(const void* x, const void* w, const void* bias, int bias_is_float, void* out, int M, int N, int K,
-                      int splits, hipStream_t stream) {
-  if (M <= 16) return launch_skinny<WAVES, 1, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream);
-  if (M <= 32) return launch_skinny<WAVES, 2, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream);
-  return launch_skinny<WAVES, 4, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream);
+                      int splits, hipStream_t stream, Tail tail = {}) {
+  if (M <= 16) return launch_skinny<WAVES, 1, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream, tail);
+  if (M <= 32) return launch_skinny<WAVES, 2, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream, tail);
+  return launch_skinny<WAVES, 4, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream, tail);
 }
 
 template <typename TO, int GATED>
 static int pick_waves(const void* x, const void* w, const void* bias, int bias_is_float, void* out, int M, int N, int K,
-                      int splits, hipStream_t stream) {
+                      int splits, hipStream_t stream, Tail tail = {}) {
   // enough waves to cover the chip (about 2,048), but no more than there are 128-wide groups of K
   const int tiles = (N + 15) / 16 * splits, groups = max(1, K / splits / (STEP * GROUP));
   int waves = 4;
   while (waves < 16 && waves * tiles < TARGET_WAVES && waves * 2 <= groups) waves *= 2;
-  if (waves == 4) return pick_tiles<4, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream);
-  if (waves == 8) return pick_tiles<8, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream);
-  return pick_tiles<16, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream);
+  if (waves == 4) return pick_tiles<4, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream, tail);
+  if (waves == 8) return pick_tiles<8, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream, tail);
+  return pick_tiles<16, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream, tail);
 }
 
 // gemm_pair: gemm_skinny for up to 16 rows of x with NT tiles of 16 weight rows a wave, which share
@@ -189,7 +212,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_pair_kernel(const bf16_t* __r
                                                                const bf16_t* __restrict__ w,
                                                                const void* __restrict__ bias, int bias_is_float,
                                                                TO* __restrict__ out, int M, int N, int K,
-                                                               int k_split) {
+                                                               int k_split, Tail tail) {
   extern __shared__ float partial[];  // [WAVES][NT][64 lanes][4]
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int r = lane & 15, g = lane >> 4;
@@ -254,7 +277,9 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_pair_kernel(const bf16_t* __r
   if (m >= M) return;
 #pragma unroll
   for (int i = 0; i < 4; ++i) total[i] += bias_here[i];
-  if (GATED) {
+  if (GATED == 3) {
+    store_with_tail(out, tail, m, n_first, N, total);
+  } else if (GATED) {
     TO* dst = out + (size_t)m * (N / 2) + n_first / 2;
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
@@ -273,10 +298,10 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_pair_kernel(const bf16_t* __r
 
 template <int NT, typename TO, int GATED>
 static int launch_pair(const void* x, const void* w, const void* bias, int bias_is_float, void* out, int M, int N,
-                       int K, int splits, hipStream_t stream) {
+                       int K, int splits, hipStream_t stream, Tail tail = {}) {
   const size_t lds = (size_t)4 * NT * 64 * 4 * sizeof(float);
   hipLaunchKernelGGL((gemm_pair_kernel<4, NT, TO, GATED>), dim3((N + 16 * NT - 1) / (16 * NT), splits), dim3(256), lds,
-                     stream, (const bf16_t*)x, (const bf16_t*)w, bias, bias_is_float, (TO*)out, M, N, K, K / splits);
+                     stream, (const bf16_t*)x, (const bf16_t*)w, bias, bias_is_float, (TO*)out, M, N, K, K / splits, tail);
   return LAUNCH_STATUS();
 }
 
@@ -324,7 +349,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_stream_kernel(const bf16_t* _
                                                                  const bf16_t* __restrict__ w,
                                                                  const void* __restrict__ bias, int bias_is_float,
                                                                  TO* __restrict__ out, int M, int N, int K,
-                                                                 int k_split) {
+                                                                 int k_split, Tail tail) {
   extern __shared__ __attribute__((aligned(16))) unsigned char stream_lds[];
   constexpr int OPERANDS = (NT + MT) * G;                // of one group: the weight tiles' steps, then x's
   constexpr int STAGE_BYTES = OPERANDS * STREAM_CHUNK;
@@ -427,7 +452,9 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_stream_kernel(const bf16_t* _
 #pragma unroll
       for (int i = 0; i < 4; ++i) total[i] += load_as_float(bias, bias_is_float, min(n_first + i, N - 1));
     }
-    if (GATED) {
+    if (GATED == 3) {
+      store_with_tail(out, tail, m, n_first, N, total);
+    } else if (GATED) {
       TO* dst = out + (size_t)m * (N / 2) + n_first / 2;
 #pragma unroll
       for (int i = 0; i < 2; ++i) {
@@ -447,7 +474,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_stream_kernel(const bf16_t* _
 
 template <int WAVES, int NT, int MT, int G, typename TO, int GATED>
 static int launch_stream(const void* x, const void* w, const void* bias, int bias_is_float, void* out, int M, int N,
-                         int K, int splits, hipStream_t stream) {
+                         int K, int splits, hipStream_t stream, Tail tail = {}) {
   const size_t stages = (size_t)WAVES * STREAM_STAGES * (NT + MT) * G * STREAM_CHUNK;
   const size_t sums = (size_t)WAVES * NT * MT * 64 * 4 * sizeof(float);
   const size_t lds = stages > sums ? stages : sums;
@@ -462,7 +489,7 @@ static int launch_stream(const void* x, const void* w, const void* bias, int bia
   }
   hipLaunchKernelGGL((gemm_stream_kernel<WAVES, NT, MT, G, TO, GATED>), dim3((N + 16 * NT - 1) / (16 * NT), splits),
                      dim3(WAVES * 64), lds, stream, (const bf16_t*)x, (const bf16_t*)w, bias, bias_is_float, (TO*)out, M,
-                     N, K, K / splits);
+                     N, K, K / splits, tail);
   return LAUNCH_STATUS();
 }
 
@@ -475,7 +502,7 @@ static int launch_stream(const void* x, const void* w, const void* bias, int bia
 // M <= 16, K / splits a multiple of 128.
 template <typename TO, int GATED>
 static int pick_stream(const void* x, const void* w, const void* bias, int bias_is_float, void* out, int M, int N, int K,
-                       int splits, hipStream_t stream, int nt = 0, int g = 0) {
+                       int splits, hipStream_t stream, int nt = 0, int g = 0, Tail tail = {}) {
   const long tiles = (N + 15) / 16;
   if (M > 16) {
     // 17 to 64 rows: two or four tiles of x.  nt, g: 0 = by the sizes, else as asked (measurements)
@@ -483,7 +510,7 @@ static int pick_stream(const void* x, const void* w, const void* bias, int bias_
     if (g == 0) g = 1;
 #define ROWS_CASE(NT_, MT_, G_)                                                                              \
   if (nt == NT_ && g == G_ && M <= 16 * MT_)                                                                 \
-    return launch_stream<4, NT_, MT_, G_, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream);
+    return launch_stream<4, NT_, MT_, G_, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream, tail);
     ROWS_CASE(1, 2, 1)
     ROWS_CASE(2, 2, 1)
     ROWS_CASE(1, 2, 2)
@@ -501,8 +528,8 @@ static int pick_stream(const void* x, const void* w, const void* bias, int bias_
   // 7B and 32B sizes: 11.6 -> 10.6 and 20.0 -> 17.5 us); with K cut over workgroups one tile is as good or
   // better (the 32B sizes' o in two parts: 13.5 us against 16.9)
   if (splits == 1 && tiles >= 256 && tiles < 1024 && tiles * K >= 1000000L)
-    return launch_stream<4, 2, 1, 2, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream);
-  return launch_stream<4, 1, 1, 4, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream);
+    return launch_stream<4, 2, 1, 2, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream, tail);
+  return launch_stream<4, 1, 1, 4, TO, GATED>(x, w, bias, bias_is_float, out, M, N, K, splits, stream, tail);
 }
 
 // The same product as llmserve_gemm_skinny, always through gemm_stream (tests and measurements); up to 64 rows.
@@ -1544,11 +1571,8 @@ extern "C" int llmserve_gemm_tiled(const void* x, const void* w, const void* bia
 // `gated` (1: silu(gate) * up, 2: relu(gate) * up) an even N.  Any N.  With splits > 1 (float32 out, not gated, K / splits a multiple of
 // 32) `out` is [splits, M, N]: slice s holds the sums over the s-th part of K (the bias in slice 0),
 // and whoever reads it adds the slices in order.
-extern "C" int llmserve_gemm_skinny(const void* x, const void* w, const void* bias, int bias_is_float, void* out,
-                                    int out_is_float, int gated, int M, int N, int K, int splits,
-                                    hipStream_t stream) {
-  if (M <= 0 || N <= 0) return 0;
-  if (M > 64 || K <= 0 || K % STEP || (gated && N % 2) || gated > 2 || splits < 1) return ERR_BAD_ARGUMENT;
+static int skinny_entry(const void* x, const void* w, const void* bias, int bias_is_float, void* out, int out_is_float, int gated,
+                        int M, int N, int K, int splits, hipStream_t stream, Tail tail) {
   if (splits > 1 && (gated || !out_is_float || K % splits || (K / splits) % STEP)) return ERR_BAD_ARGUMENT;
   if (M <= 16 && (K / splits) % (STEP * GROUP) == 0) {
     // several weight tiles a wave where a wave has many groups of K to walk (or x is all 16 rows) and
@@ -1561,6 +1585,7 @@ extern "C" int llmserve_gemm_skinny(const void* x, const void* w, const void* bi
                                                                                                             : 1;
     // Two tiles or one: through LDS (gemm_stream), unless many rows of x meet a long walk over K.
     if (share != 4 && !(share == 2 && M > 8 && per_wave >= 4)) {
+      if (gated == 3) return pick_stream<bf16_t, 3>(x, w, bias, bias_is_float, out, M, N, K, 1, stream, 0, 0, tail);
       if (gated == 2)
         return out_is_float ? pick_stream<float, 2>(x, w, bias, bias_is_float, out, M, N, K, 1, stream)
                             : pick_stream<bf16_t, 2>(x, w, bias, bias_is_float, out, M, N, K, 1, stream);
@@ -1572,6 +1597,7 @@ extern "C" int llmserve_gemm_skinny(const void* x, const void* w, const void* bi
     }
 #define PAIR_CASE(NT)                                                                                              \
   if (share == NT) {                                                                                               \
+    if (gated == 3) return launch_pair<NT, bf16_t, 3>(x, w, bias, bias_is_float, out, M, N, K, 1, stream, tail);   \
     if (gated == 2)                                                                                                \
       return out_is_float ? launch_pair<NT, float, 2>(x, w, bias, bias_is_float, out, M, N, K, 1, stream)          \
                           : launch_pair<NT, bf16_t, 2>(x, w, bias, bias_is_float, out, M, N, K, 1, stream);        \
@@ -1596,6 +1622,7 @@ extern "C" int llmserve_gemm_skinny(const void* x, const void* w, const void* bi
     return out_is_float ? pick_stream<float, false>(x, w, bias, bias_is_float, out, M, N, K, splits, stream, 1, g)
                         : pick_stream<bf16_t, false>(x, w, bias, bias_is_float, out, M, N, K, 1, stream, 1, g);
   }
+  if (gated == 3) return pick_waves<bf16_t, 3>(x, w, bias, bias_is_float, out, M, N, K, 1, stream, tail);
   if (gated == 2)
     return out_is_float ? pick_waves<float, 2>(x, w, bias, bias_is_float, out, M, N, K, 1, stream)
                         : pick_waves<bf16_t, 2>(x, w, bias, bias_is_float, out, M, N, K, 1, stream);
@@ -1604,4 +1631,21 @@ extern "C" int llmserve_gemm_skinny(const void* x, const void* w, const void* bi
                         : pick_waves<bf16_t, true>(x, w, bias, bias_is_float, out, M, N, K, 1, stream);
   return out_is_float ? pick_waves<float, false>(x, w, bias, bias_is_float, out, M, N, K, splits, stream)
                       : pick_waves<bf16_t, false>(x, w, bias, bias_is_float, out, M, N, K, 1, stream);
+}
+
+extern "C" int llmserve_gemm_skinny(const void* x, const void* w, const void* bias, int bias_is_float, void* out,
+                                    int out_is_float, int gated, int M, int N, int K, int splits,
+                                    hipStream_t stream) {
+  if (M <= 0 || N <= 0) return 0;
+  if (M > 64 || K <= 0 || K % STEP || (gated && N % 2) || gated > 2 || splits < 1) return ERR_BAD_ARGUMENT;
+  return skinny_entry(x, w, bias, bias_is_float, out, out_is_float, gated, M, N, K, splits, stream, Tail{});
+}
+
+// The same for a bfloat16 result in two places: columns below `first` to out [M, first] (may be null where first is 0), the
+// others, as relu(z)^2, to the first N - first columns of `tail`, whose rows begin every `tail_stride` elements.
+extern "C" int llmserve_gemm_skinny_tail(const void* x, const void* w, const void* bias, int bias_is_float, void* out, int first,
+                                         void* tail, int tail_stride, int M, int N, int K, hipStream_t stream) {
+  if (M <= 0 || N <= 0) return 0;
+  if (M > 64 || K <= 0 || K % STEP || first < 0 || first >= N || tail_stride < N - first || !tail || (first && !out)) return ERR_BAD_ARGUMENT;
+  return skinny_entry(x, w, bias, bias_is_float, out, 0, 3, M, N, K, 1, stream, Tail{(bf16_t*)tail, first, tail_stride});
 }

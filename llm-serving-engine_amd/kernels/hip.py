@@ -62,6 +62,7 @@ _SIGNATURES = {
     "llmserve_gemm_generic": "pipipipiiiip",
     "llmserve_gemm_f32": "ppppiiiiip",
     "llmserve_gemm_skinny": "pppipiiiiiip",
+    "llmserve_gemm_skinny_tail": "pppipipiiiip",
     "llmserve_gemm_stream": "pppipiiiiiip",
     "llmserve_gemm_stream_shaped": "pppipiiiiiiiip",
     "llmserve_gemm_medium": "pppipiiiiiip",
@@ -132,6 +133,22 @@ class LinearWeights:
 
     weight: torch.Tensor
     bias: torch.Tensor | None
+    _transposed: torch.Tensor | None = None
+    _float_bias: torch.Tensor | None = None
+
+    @property
+    def transposed(self) -> torch.Tensor:
+        """The weight as [K, N] rows, made when a product over slices of K first asks for it: the library's batched product
+        takes a right operand whose rows lie as they are read."""
+        if self._transposed is None:
+            self._transposed = self.weight.t().contiguous()
+        return self._transposed
+
+    @property
+    def float_bias(self) -> torch.Tensor:
+        if self._float_bias is None:
+            self._float_bias = self.bias.float()
+        return self._float_bias
 
     @property
     def out_features(self) -> int:
@@ -562,16 +579,21 @@ class HipKernels:
             streaming = "medium"
         if streaming is None and self._library(x, weights):
             if (out_dtype or self.dtype) == torch.float32:  # float32 straight from the accumulators
-                cuts = self._library_splits(rows, weights.out_features, inner) if partial and bias is None else 1
+                cuts = self._library_splits(rows, weights.out_features, inner) if partial else 1
                 if cuts > 1:
                     # The library does not cut a long K over workgroups by itself (the down projection of the 7B
                     # sizes at 2,048 rows: 342 us in one piece, 217 in two; at 136 rows 103 and 43 in eight).  As a
                     # strided batch of `cuts` products over slices of K it does, and the batch is the partial sums.
+                    # (Over the weight's transpose, which lies in such slices whatever `cuts` is: as fast as over views of
+                    # the weight itself, 62.5 us against 61.8 at 2,048 rows of K 10,496 x N 1,536, where one piece takes 82.)
                     slices = x.view(rows, cuts, inner // cuts).transpose(0, 1)
-                    weight_slices = weights.weight.view(weights.out_features, cuts, inner // cuts).permute(1, 2, 0)
-                    return torch.bmm(slices, weight_slices, out_dtype=torch.float32)
+                    weight_slices = weights.transposed.view(cuts, inner // cuts, weights.out_features)
+                    parts = torch.bmm(slices, weight_slices, out_dtype=torch.float32)
+                    if bias is not None:
+                        parts[0].add_(weights.float_bias)
+                    return parts
                 out = torch.mm(x, weights.weight.t(), out_dtype=torch.float32)
-                return out if bias is None else out.add_(bias.float())
+                return out if bias is None else out.add_(weights.float_bias)
             if bias is not None and bias.dtype != x.dtype:
                 return (torch.mm(x, weights.weight.t(), out_dtype=torch.float32) + bias).to(torch.bfloat16)
             return torch.nn.functional.linear(x, weights.weight, bias)
@@ -1202,12 +1224,24 @@ class HipKernels:
         columns of `out` from `out_first`."""
         code = self._plain_activation(activation, "activated_linear")
         width = weights.out_features - first
-        if not 0 <= first < weights.out_features:
-            raise KernelError("activated_linear: the activation begins at a column of the product")
+        if not 0 <= first < weights.out_features or x.shape[1] != weights.in_features or not (out is None or out.is_contiguous()):
+            raise KernelError("activated_linear: the activation begins at a column of the product, and rows are contiguous")
         if out is None:
             out = self._empty((x.shape[0], width), self.dtype)
         if out.dtype != self.dtype or out.shape[0] != x.shape[0] or not 0 <= out_first <= out.shape[1] - width:
             raise KernelError("activated_linear: the rows to write are of the run dtype, one a token, and wide enough")
+        streaming = self._streaming(x, weights)
+        if activation == "squared_relu" and (streaming == "skinny" or (streaming == "ring" and x.shape[0] <= 8)):
+            # the kernels for a few rows (a decode step) apply it in their epilogue and store the two runs of columns apart
+            # (up to 8 rows the ring is not far enough ahead of them on a large weight to pay a launch more)
+            rows = self._empty((x.shape[0], first), self.dtype) if first else None
+            status = self._gemm_bf16.llmserve_gemm_skinny_tail(
+                _pointer(x), _pointer(weights.weight), _pointer(weights.bias), _is_float(weights.bias) if weights.bias is not None else 0,
+                _pointer(rows), first, out.data_ptr() + out_first * out.element_size(), out.shape[1], x.shape[0], weights.out_features,
+                weights.in_features, self._stream,
+            )
+            _check(status, "activated_linear")
+            return rows, out
         rows = self.linear(x, weights)
         status = self._library_of("columns").llmserve_activate_columns(
             _pointer(rows), _is_float(rows), rows.shape[0], rows.shape[1], first, _pointer(out), out.shape[1], out_first, width, code, self._stream
