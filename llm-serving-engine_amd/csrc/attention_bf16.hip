@@ -295,7 +295,8 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
   // back.  So everything the start of the kernel needs is asked for here at once, before anything is
   // used: the pieces of the token's key and value row (one wave will store them; which one depends on the
   // position, so all ask), the angles, and the pages of this wave's first step, looked up as if that
-  // step lay wholly inside the context and the context's first key were in sight (if not, they are looked up again below).
+  // step lay wholly inside the context and the context's first key were in sight (if not, they are looked up again below:
+  // a page behind a mask may have been given back, and its entry in the table is no page).
   constexpr int PAIR_PIECES = (D / 2 + WAVE - 1) / WAVE, VALUE_PIECES = (D + WAVE - 1) / WAVE;
   [[maybe_unused]] bf16_t new_a[PAIR_PIECES], new_b[PAIR_PIECES], new_v[VALUE_PIECES];
   [[maybe_unused]] float2 new_angle[PAIR_PIECES];
@@ -538,7 +539,7 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
   if (step_begin + wave < step_end) {
     const int step0 = step_begin + wave;
     StepLoads loads;
-    StepPages pages = early_pages && step_begin == 0 && step0 < step_last ? StepPages{early_k, early_k_hi, early_v} : pages_of(step0);
+    StepPages pages = early_pages && first_key == 0 && step0 < step_last ? StepPages{early_k, early_k_hi, early_v} : pages_of(step0);
     fetch_keys(step0, pages, loads);
     fetch_values(step0, pages, loads);
     if constexpr (TWO_STEPS) {
@@ -557,7 +558,7 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
       const int step1 = step0 + WAVES;
       if (step1 < step_end) {
         const StepPages pages1 =
-            second_pages && step_begin == 0 && step1 < step_last ? StepPages{second_k, second_k_hi, second_v} : pages_of(step1);
+            second_pages && first_key == 0 && step1 < step_last ? StepPages{second_k, second_k_hi, second_v} : pages_of(step1);
         fetch_keys(step1, pages1, ahead);
         fetch_values(step1, pages1, ahead);
       }
