@@ -89,9 +89,10 @@ class NormedAttention(Mixer):
     @classmethod
     def tensors(cls, spec: NormedAttentionSpec) -> dict[str, TensorSpec]:
         q_size, k_size, v_size = spec.num_heads * spec.dim, spec.num_kv_heads * spec.dim, spec.num_kv_heads * spec.vdim
-        found = {"q": TensorSpec((q_size, spec.hidden_size)), "o": TensorSpec((spec.hidden_size, spec.num_heads * spec.vdim))}
+        found = {"q": TensorSpec((q_size, spec.hidden_size))}
         if spec.own_keys:
             found.update({"k": TensorSpec((k_size, spec.hidden_size)), "v": TensorSpec((v_size, spec.hidden_size))})
+        found["o"] = TensorSpec((spec.hidden_size, spec.num_heads * spec.vdim))
         if spec.bias:
             found["q.b"] = TensorSpec((q_size,), role="bias")
             if spec.own_keys:

@@ -1032,11 +1032,11 @@ def test_attention_at_random_step_shapes(dtype, draws):
     shared_entry, tiles_entry = library.llmserve_attention_portions, library.llmserve_attention_tiles
 
     def counted_shared(*arguments):
-        ways["shared in runs" if arguments[18] > 1 else "shared whole"] += 1  # (splits)
+        ways["shared in runs" if arguments[19] > 1 else "shared whole"] += 1  # (splits)
         return shared_entry(*arguments)
 
     def counted_tiles(*arguments):
-        splits, fuse = arguments[19], arguments[20]
+        splits, fuse = arguments[20], arguments[21]
         ways["by item" if fuse & 4 and splits > 1 else "tiles split" if splits > 1 else "tiles"] += 1
         return tiles_entry(*arguments)
 

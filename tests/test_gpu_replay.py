@@ -384,7 +384,7 @@ def test_long_portions_at_many_heads_beside_a_decoded_token(tmp_path_factory):
         return shared_entry(*arguments)
 
     def counted_tiles(*arguments):
-        calls["by item"] += 1 if arguments[20] & 4 and arguments[19] > 1 else 0  # (fuse, splits)
+        calls["by item"] += 1 if arguments[21] & 4 and arguments[20] > 1 else 0  # (fuse, splits)
         return tiles_entry(*arguments)
 
     library.llmserve_attention_portions, library.llmserve_attention_tiles = counted_shared, counted_tiles
