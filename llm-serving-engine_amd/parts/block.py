@@ -248,7 +248,8 @@ class ParallelBlock(Block):
     """Where mixer and feed-forward both begin and end with a product (`joins`), the two first products are one over the
     weights side by side, and the two last ones are one over the operands side by side, W_o m + W_d a = [W_o | W_d] [m; a]:
     the sum of the sublayers is made in the product's float32 accumulators, and a layer is two launches of products
-    instead of four and no add.  Else the results are added by a kernel."""
+    instead of four and no add.  Else (or where the operands side by side make rows of no multiple of eight) the results
+    are added by a kernel."""
 
     @classmethod
     def _members(cls, spec: ParallelBlockSpec):
@@ -273,19 +274,24 @@ class ParallelBlock(Block):
         may_join = spec.feed_forward is not None and all(
             getattr(registry.get(member), "joins", False) and hasattr(member, "joined") for _, registry, member in self._members(spec)[1:]
         )
-        members = [(name, registry, dataclasses.replace(member, joined=True) if may_join and registry is not NORMS else member)
-                   for name, registry, member in self._members(spec)]
-        built = [registry.build(member, under(tensors, name), kernels) for name, registry, member in members]
+
+        def build(joined: bool):
+            return [registry.build(dataclasses.replace(member, joined=True) if joined and registry is not NORMS else member, under(tensors, name), kernels)
+                    for name, registry, member in self._members(spec)]
+
+        built = build(may_join)
+        if may_join:
+            weights, biases = zip(built[1].closing, built[2].closing)
+            self.mixed_width, self.inner_width = weights[0].shape[1], sum(weight.shape[1] for weight in weights)
+            if self.inner_width % 8:  # rows that begin anywhere: the matrix cores' attention writes pieces of eight elements
+                may_join, built = False, build(False)
         self.norm, self.mixer = built[:2]
         self.feed_forward = built[2] if spec.feed_forward is not None else None
         self.replayable = all(part.replayable for part in built)
         self.opening = None
         if may_join:
-            mixer, feed_forward = self.mixer, self.feed_forward
-            self.split = sum(weight.shape[0] for weight, _ in mixer.opening)  # columns of the first product that the mixer reads
-            self.opening = kernels.prepare_linear(*side_by_side(mixer.opening + feed_forward.opening))
-            weights, biases = zip(mixer.closing, feed_forward.closing)
-            self.mixed_width, self.inner_width = weights[0].shape[1], sum(weight.shape[1] for weight in weights)
+            self.split = sum(weight.shape[0] for weight, _ in self.mixer.opening)  # columns of the first product that the mixer reads
+            self.opening = kernels.prepare_linear(*side_by_side(self.mixer.opening + self.feed_forward.opening))
             biases = [bias for bias in biases if bias is not None]
             if len(biases) > 1:
                 biases = [biases[0].float() + biases[1].float()]
