@@ -27,11 +27,11 @@ WIDE = cases.config_of(
         (cases.attention(heads=8, kv_heads=2, dim=128, vdim=128, chunk=70, scale=0.09), 384),
         (cases.latent(heads=4, dim=32, rot_dim=32, vdim=64, q_rank=96, kv_rank=128, scale=0.12, window=45), 256),
         (cases.attention(heads=4, kv_heads=2, dim=128, vdim=128, chunk=52, scale=0.1, kv_from=0), 128),
-        (cases.attention(heads=4, kv_heads=4, dim=64, vdim=80, chunk=33, scale=0.15), 96),
+        (cases.attention(heads=3, kv_heads=3, dim=48, vdim=80, chunk=33, scale=0.15), 96),
         (cases.latent(heads=2, dim=64, rot_dim=16, vdim=32, q_rank=64, kv_rank=96, scale=0.12, window=130, dims=8), None),
-        (cases.attention(heads=8, kv_heads=4, dim=64, vdim=80, chunk=99, scale=0.12, kv_from=3), 200),
+        (cases.attention(heads=6, kv_heads=3, dim=48, vdim=80, chunk=99, scale=0.12, kv_from=3), 200),
     ],
-    vocab=300, width=256, scale=4.0,
+    vocab=300, width=288, scale=4.0,
 )
 
 
