@@ -26,7 +26,7 @@ import torch
 
 from ..config.serving import CacheConfig
 from .cell import CacheCell
-from ..parts.base import CacheNeed, PagedNeed, SlotNeed
+from ..parts.base import PagedNeed, SlotNeed, needs_by_name
 from ..parts.model import ModelSpec
 from .pool import CacheFullError, PagePool
 
@@ -98,12 +98,11 @@ class CacheManager:
         self._state_needs: list[SlotNeed] = []
         by_need: dict[PagedNeed, int] = {}
         for index, run in enumerate(spec.run_order):
-            if run.reads is not None:
-                self._cell_of_run.append(self._cell_of_run[run.reads])
-                continue
             entries: dict[str | None, tuple[str, int, int]] = {}
-            for name, need in self._named(spec.cell_need(index), index).items():
-                if isinstance(need, PagedNeed):
+            for name, need in needs_by_name(spec.cell_need(index)).items():
+                if run.takes(name):
+                    entries[name] = self._cell_of_run[run.reads][name]
+                elif isinstance(need, PagedNeed):
                     if need not in by_need:
                         by_need[need] = len(self.groups)
                         tables = np.full((config.max_sequences, self.max_blocks_per_sequence), -1, np.int32)
@@ -127,17 +126,6 @@ class CacheManager:
                     (len(group.cells), config.num_blocks, *shape), dtype=dtype, device=self.device
                 )
 
-    @staticmethod
-    def _named(need: "CacheNeed | dict[str, CacheNeed] | None", run: int) -> dict[str | None, CacheNeed]:
-        """A run's needs by name: none, one (under None), or the several its block named."""
-        if need is None:
-            return {}
-        if isinstance(need, dict):
-            if any(not isinstance(name, str) for name in need):
-                raise TypeError(f"run {run}: several cache needs are named by strings")
-            return {name: value for name, value in need.items() if value is not None}
-        return {None: need}
-
     # ------------------------------------------------------------------ views
 
     def _cell(self, entry: tuple[str, int, int], writable: bool) -> CacheCell:
@@ -152,13 +140,13 @@ class CacheManager:
         nothing, or the cells by name for a run whose block named several needs."""
         views: list[CacheCell | dict[str, CacheCell] | None] = []
         for index, entries in enumerate(self._cell_of_run):
-            writable = self.spec.run_order[index].reads is None
+            run = self.spec.run_order[index]
             if not entries:
                 views.append(None)
             elif None in entries:
-                views.append(self._cell(entries[None], writable))
+                views.append(self._cell(entries[None], not run.takes(None)))
             else:
-                views.append({name: self._cell(entry, writable) for name, entry in entries.items()})
+                views.append({name: self._cell(entry, not run.takes(name)) for name, entry in entries.items()})
         return views
 
     # ------------------------------------------------------------------ requests

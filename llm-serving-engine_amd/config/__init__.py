@@ -1,6 +1,7 @@
 from .model import ArchitectureConfig, ConfigError, KeyReader, Qwen2Config
 from .dafutar import DafutarConfig
 from .dolezen import DolezenConfig
+from .dubesun import DubesunConfig
 from .katenex import KatenexConfig
 from .sozavik import SozavikConfig
 from .vagozen import VagozenConfig
@@ -12,6 +13,7 @@ __all__ = [
     "ConfigError",
     "DafutarConfig",
     "DolezenConfig",
+    "DubesunConfig",
     "KatenexConfig",
     "KeyReader",
     "Qwen2Config",

@@ -28,7 +28,11 @@
 // reference has neither): `soft_cap` > 0 squashes it to cap * tanh(score / cap), and `slopes` (one
 // per query head) then takes slope * (query position - key position) off it.  What leaves the scores as they are
 // is a kind of CHANGED of its own, which the fused decode form takes too: a sink in the denominator, and a mask
-// in chunks (a query sees the keys of its own chunk of positions, counted from the sequence's start).
+// in chunks (a query sees the keys of its own chunk of positions, counted from the sequence's start).  Two more kinds write
+// their results finished, heads of `vdim` side by side: CHANGED_BIAS adds a learned bias by distance to the scores and may
+// multiply the results with a gate an element; CHANGED_MAPS is differential attention: a query and a key are two maps side by
+// side, a wave's two column tiles are the two maps of the same columns, each multiplied with its own half of the keys, and the
+// difference of the two results is normed before it is written.
 #include "common.h"
 
 #ifndef HEAD_DIM
@@ -101,6 +105,8 @@ struct FusedDecode {          // what the kernel needs to rotate and store; unus
 #define CHANGED_NOT 0
 #define CHANGED_SCORES 1      // slopes, a soft cap, kept first keys, and what CHANGED_EDGES has
 #define CHANGED_EDGES 2       // sinks and a mask in chunks alone: the scores stay as they are
+#define CHANGED_BIAS 3        // a bias by distance on the scores, a gate an element on the results
+#define CHANGED_MAPS 4        // two maps a head over the same values, the second taken off the first
 
 struct ScoreChange {          // unused unless CHANGED
   const float* slopes;        // [heads], or null
@@ -108,7 +114,44 @@ struct ScoreChange {          // unused unless CHANGED
   const float* sinks;         // [heads], or null: exp(sink) more in a head's denominator, once, with no value to it
   int keep_first;             // under a window, a sequence's first so many keys stay visible to every later query; 0: none
   int chunk;                  // instead of a window: a query sees the keys of its own chunk of so many positions; 0: none
+  const float* bias;          // [heads][reach + BIAS_SPARE] by distance (common.h: bias_element), or null
+  int reach;
 };
+
+struct Finish {               // how CHANGED_BIAS and CHANGED_MAPS write a result: heads of `vdim` side by side
+  int vdim;
+  const bf16_t* gates;        // CHANGED_BIAS: a result's element is multiplied with the sigmoid of gates[row][first + its column]; or null
+  int gate_stride, gate_first;
+  float factor, eps, out_scale;  // CHANGED_MAPS: d = map 1 - factor * map 2, then d / sqrt(mean(d^2) + eps) * out_scale
+};
+
+// four results of one head, from dimension d4 on, to their row (16-byte aligned where vdim is a multiple of 4)
+__device__ __forceinline__ void write_finished(const Finish& f, bf16_t* row_out, const bf16_t* row_gates, int head, int d4, f32x4 v) {
+  if (d4 >= f.vdim) return;
+  const int column = head * f.vdim + d4;
+  const bool whole = f.vdim % 4 == 0;
+  if (row_gates) {
+    const bf16_t* g = row_gates + column;
+    float gate[4];
+    if (whole && (f.gate_stride | f.gate_first) % 4 == 0) {
+      const bf16x4 raw = *(const bf16x4*)g;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) gate[i] = (float)raw[i];
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) gate[i] = d4 + i < f.vdim ? (float)g[i] : 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] *= __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(gate[i] * -1.44269504088896f));
+  }
+  if (whole) {
+    *(bf16x4*)(row_out + column) = (bf16x4){(bf16_t)v[0], (bf16_t)v[1], (bf16_t)v[2], (bf16_t)v[3]};
+  } else {
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (d4 + i < f.vdim) row_out[column + i] = (bf16_t)v[i];
+  }
+}
 
 // One step's operands as a lane holds them: its slices of the K rows of the two 16-row tiles and,
 // for every 16-row tile of V^T, eight consecutive keys of its row.
@@ -154,7 +197,10 @@ struct Columns {
 };
 
 // First product of a step, for all column tiles: after it the K rows are no longer needed.
-template <int COLUMN_TILES>
+// CHANGED_MAPS: tile t meets the t-th half of the keys alone (a step of the product that straddles the middle is of both,
+// and a query has zeros in the other half of it).
+constexpr int STEP_WIDTH = WIDE ? 32 : 16;  // elements of a head a step of the first product takes
+template <int COLUMN_TILES, int CHANGED = CHANGED_NOT>
 __device__ __forceinline__ void scores_of(const Columns<COLUMN_TILES>& columns, const StepLoads& L, f32x4* s_lo,
                                           f32x4* s_hi) {
 #pragma unroll
@@ -163,6 +209,7 @@ __device__ __forceinline__ void scores_of(const Columns<COLUMN_TILES>& columns, 
     s_hi[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int s = 0; s < QK_STEPS; ++s) {
+      if (CHANGED == CHANGED_MAPS && (t == 0 ? s * STEP_WIDTH >= D / 2 : (s + 1) * STEP_WIDTH <= D / 2)) continue;
       s_lo[t] = mfma_qk(L.k_lo[s], columns.query[t][s], s_lo[t]);
       s_hi[t] = mfma_qk(L.k_hi[s], columns.query[t][s], s_hi[t]);
     }
@@ -182,7 +229,8 @@ __device__ __forceinline__ void scores_of(const Columns<COLUMN_TILES>& columns, 
 template <int COLUMN_TILES, int CHANGED = CHANGED_NOT>
 __device__ __forceinline__ void weigh_and_add(Columns<COLUMN_TILES>& columns, StepLoads& L, const f32x4* s_lo,
                                               const f32x4* s_hi, int key0, int q, bool interior, int last_key,
-                                              int v_start, float scale_log2, float soft_cap = 0.f, int keep = 0) {
+                                              int v_start, float scale_log2, float soft_cap = 0.f, int keep = 0,
+                                              const float (*bias)[8] = nullptr) {
   bf16x8 weights[COLUMN_TILES];
 #pragma unroll
   for (int t = 0; t < COLUMN_TILES; ++t) {
@@ -204,6 +252,10 @@ __device__ __forceinline__ void weigh_and_add(Columns<COLUMN_TILES>& columns, St
       const float distance = (float)(columns.position[t] - (key0 + 8 * q));  // of the lane's first key
 #pragma unroll
       for (int i = 0; i < 8; ++i) x[i] -= columns.slope[t] * (distance - (float)i);
+    }
+    if constexpr (CHANGED == CHANGED_BIAS) {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) x[i] = fmaf(bias[t][i], 1.44269504088896f, x[i]);
     }
     if (!interior) {
       // key0 + 8q + i outside [first, position], counted from the lane's first key (nothing to add per key)
@@ -269,8 +321,9 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
     float* __restrict__ partial_ml, bf16_t* __restrict__ keys,
     bf16_t* __restrict__ values, const int* __restrict__ block_tables, int table_width,
     const int* __restrict__ positions, const int* __restrict__ work, int heads, int kv_heads, int tokens_per_tile,
-    int page_size, int page_shift, float scale, int window, int splits, FusedDecode fused, ScoreChange change) {
-  static_assert(!(FUSED && CHANGED == CHANGED_SCORES), "the fused decode form leaves the scores as they are");
+    int page_size, int page_shift, float scale, int window, int splits, FusedDecode fused, ScoreChange change, Finish finish) {
+  static_assert(!FUSED || CHANGED == CHANGED_NOT || CHANGED == CHANGED_EDGES, "the fused decode form leaves the scores as they are");
+  static_assert(CHANGED != CHANGED_MAPS || COLUMN_TILES == 2, "a column tile a map");
   extern __shared__ float lds[];  // [WAVES][16 columns][D + 4]
   if (FUSED)  // a short kernel: fetch all arguments in one go rather than each before its first use
     asm volatile("" ::"s"(row_width), "s"(table_width), "s"(heads), "s"(kv_heads), "s"(page_size), "s"(page_shift),
@@ -348,6 +401,7 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
   // this lane's column in each of its column tiles
   Columns<COLUMN_TILES> columns;
   bool column_live[COLUMN_TILES];
+  [[maybe_unused]] const float* column_bias[COLUMN_TILES];
   auto& column_position = columns.position;
   auto& column_first = columns.first;
   auto& query = columns.query;
@@ -357,7 +411,7 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
 #pragma unroll
   for (int t = 0; t < COLUMN_TILES; ++t) {
     int token, head_here;
-    map.of(t, c, token, head_here, column_live[t]);
+    map.of(CHANGED == CHANGED_MAPS ? 0 : t, c, token, head_here, column_live[t]);
     const int safe = min(token, tokens - 1);
     const int head = kv_head * group + head_tile * 16 + head_here;
     column_position[t] = column_live[t] ? position0 + safe : -1;
@@ -366,6 +420,16 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
     const bf16_t* q_row = qkv + (size_t)(row0 + safe) * row_width + (size_t)head * D;
 #pragma unroll
     for (int s = 0; s < QK_STEPS; ++s) query[t][s] = load_qk(q_row, KEY_PIECE, s, q);  // a query's row is in one piece
+    if constexpr (CHANGED == CHANGED_BIAS) {
+      column_bias[t] = change.bias + (size_t)head * (change.reach + BIAS_SPARE);
+      columns.slope[t] = column_bias[t][0];  // of every distance beyond the table's reach
+    }
+#if HEAD_DIM % 32 == 0
+    if constexpr (CHANGED == CHANGED_MAPS && D / 2 % 32 != 0) {  // the step that straddles the middle: zeros in the other map's half
+      constexpr int middle = D / 2 / 32;
+      if ((q >= 2) != (t == 1)) query[t][middle].v = (bf16x8){};
+    }
+#endif
 #if HEAD_DIM % 32 == 0
     if (FUSED && fused.pairing != 0) {  // the queries come unrotated: rotate them here, in float32
       const float2* angles = fused.table + (size_t)(row0 + safe) * (D / 2);
@@ -586,12 +650,30 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
     for (int step = step0; step < step_end; step += WAVES) {
       const bool more = step + WAVES < step_end;
       f32x4 s_lo[COLUMN_TILES], s_hi[COLUMN_TILES];
-      scores_of(columns, loads, s_lo, s_hi);
-      if (more) fetch_keys(step + WAVES, pages, loads);
       const int key0 = real_step(step) * KEYS;
+      [[maybe_unused]] float bias[COLUMN_TILES][8];
+      if constexpr (CHANGED == CHANGED_BIAS) {
+        if (position0 - (key0 + KEYS - 1) >= change.reach - 1) {  // all of the step's keys lie beyond the table's reach
+#pragma unroll
+          for (int t = 0; t < COLUMN_TILES; ++t)
+#pragma unroll
+            for (int i = 0; i < 8; ++i) bias[t][i] = columns.slope[t];
+        } else {
+          typedef float f32x4_anywhere __attribute__((ext_vector_type(4), aligned(4)));
+#pragma unroll
+          for (int t = 0; t < COLUMN_TILES; ++t) {
+            const float* at = column_bias[t] + bias_element(column_position[t] - (key0 + 8 * q), change.reach);
+            const f32x4_anywhere lo = *(const f32x4_anywhere*)at, hi = *(const f32x4_anywhere*)(at + 4);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) bias[t][i] = i < 4 ? lo[i] : hi[i - 4];
+          }
+        }
+      }
+      scores_of<COLUMN_TILES, CHANGED>(columns, loads, s_lo, s_hi);
+      if (more) fetch_keys(step + WAVES, pages, loads);
       const bool interior = key0 + KEYS - 1 <= position0 && key0 >= every_first;
       weigh_and_add<COLUMN_TILES, CHANGED>(columns, loads, s_lo, s_hi, key0, q, interior, last_key, held_piece(key0 + 8 * q),
-                                           scale_log2, change.soft_cap, keep);
+                                           scale_log2, change.soft_cap, keep, bias);
       if (more) fetch_values(step + WAVES, pages, loads);
       if (step + 2 * WAVES < step_end) pages = pages_of(step + 2 * WAVES);
     }
@@ -603,6 +685,9 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
   // (a column's row is D sums, then its maximum and its sum of weights; rows 16 bytes apart in the banks, so that a
   // lane's four sums of a tile go and come as one 16-byte piece)
   constexpr int STRIDE = D + 4;
+  // (CHANGED_MAPS: a thread's pieces of the first map's results stay here until it has the second's)
+  constexpr int HELD = CHANGED == CHANGED_MAPS ? (16 * (D / 4) + WAVES * 64 - 1) / (WAVES * 64) : 1;
+  [[maybe_unused]] f32x4 held[HELD];
 #pragma unroll
   for (int t = 0; t < COLUMN_TILES; ++t) {
     float sum = running_sum[t];
@@ -613,11 +698,14 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
     for (int d = 0; d < D_TILES; ++d) *(f32x4*)(mine + d * 16 + 4 * q) = acc[t][d];
     if (q == 0) *(float2*)(mine + D) = make_float2(running_max[t], sum);
     __syncthreads();
-    for (int index = threadIdx.x; index < 16 * (D / 4); index += WAVES * 64) {
+#pragma unroll
+    for (int turn = 0; turn < (16 * (D / 4) + WAVES * 64 - 1) / (WAVES * 64); ++turn) {
+      const int index = threadIdx.x + turn * WAVES * 64;
+      if (index >= 16 * (D / 4)) continue;
       const int column = index / (D / 4), d4 = (index % (D / 4)) * 4;
       int token, head_here;
       bool live;
-      map.of(t, column, token, head_here, live);
+      map.of(CHANGED == CHANGED_MAPS ? 0 : t, column, token, head_here, live);
       if (!live) continue;
       float2 theirs_ml[WAVES];
       f32x4 theirs_acc[WAVES];
@@ -650,12 +738,20 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
           }
         }
         const float inverse = total > 0.f ? shrink / total : 0.f;
-        const bf16x4 rounded = {(bf16_t)(merged[0] * inverse), (bf16_t)(merged[1] * inverse), (bf16_t)(merged[2] * inverse),
-                                (bf16_t)(merged[3] * inverse)};
-        *(bf16x4*)(out + row * out_stride + head * D + d4) = rounded;
+        if constexpr (CHANGED == CHANGED_MAPS) {
+          if (t == 0) held[turn] = merged * inverse;
+          else held[turn] -= merged * (inverse * finish.factor);
+        } else if constexpr (CHANGED == CHANGED_BIAS) {
+          write_finished(finish, out + row * out_stride, finish.gates ? finish.gates + row * finish.gate_stride + finish.gate_first : nullptr,
+                         head, d4, merged * inverse);
+        } else {
+          const bf16x4 rounded = {(bf16_t)(merged[0] * inverse), (bf16_t)(merged[1] * inverse), (bf16_t)(merged[2] * inverse),
+                                  (bf16_t)(merged[3] * inverse)};
+          *(bf16x4*)(out + row * out_stride + head * D + d4) = rounded;
+        }
       } else {
         const size_t kept_as = fused.by_item ? (size_t)(gridDim.x - 1 - blockIdx.x) * tokens_per_tile + token : row;
-        const size_t slot = (kept_as * heads + head) * splits + blockIdx.z;
+        const size_t slot = (CHANGED == CHANGED_MAPS ? (kept_as * heads + head) * 2 + t : kept_as * heads + head) * splits + blockIdx.z;
         if (fused.unmerged) {
           // for the product that merges: [head][split][piece of 8][16 rows][8], the rows of a piece side by
           // side, so that the four lanes of its loads that hold four rows' share of a piece read 64 bytes
@@ -674,6 +770,34 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
       }
     }
     __syncthreads();
+  }
+  if constexpr (CHANGED == CHANGED_MAPS) {
+    if (splits > 1) return;
+    // a column's sum of squares, over the threads that hold its pieces (dimensions beyond vdim are zeros)
+    constexpr int PIECES = D / 4, SQUARES = PIECES + 1;
+#pragma unroll
+    for (int turn = 0; turn < HELD; ++turn) {
+      const int index = threadIdx.x + turn * WAVES * 64;
+      if (index >= 16 * PIECES) continue;
+      const f32x4 v = held[turn];
+      lds[(index / PIECES) * SQUARES + index % PIECES] = v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int turn = 0; turn < HELD; ++turn) {
+      const int index = threadIdx.x + turn * WAVES * 64;
+      if (index >= 16 * PIECES) continue;
+      const int column = index / PIECES, d4 = (index % PIECES) * 4;
+      int token, head_here;
+      bool live;
+      map.of(0, column, token, head_here, live);
+      if (!live) continue;
+      float squares = 0.f;
+      for (int i = 0; i < PIECES; ++i) squares += lds[column * SQUARES + i];
+      const float normed = finish.out_scale * rsqrtf(squares / (float)finish.vdim + finish.eps);
+      write_finished(finish, out + ((size_t)row0 + token) * out_stride, nullptr, kv_head * group + head_tile * 16 + head_here, d4,
+                     held[turn] * normed);
+    }
   }
 }
 
@@ -762,6 +886,43 @@ __global__ __launch_bounds__(MERGE_THREADS) void attention_merge_items_kernel(co
     merge_splits(partial_ml + kept_as * splits * 2, partial_acc + kept_as * splits * D, splits,
                  out + ((size_t)item[1] + token) * out_stride + head * D, sink);
   }
+}
+
+// The kinds that write finished results: workgroup (row, head), a thread a dimension; every lane of every wave calls
+// merged_value, which gives dimension min(d, D - 1) of the splits' merged result.
+__device__ __forceinline__ float merged_value(const float* ml, const float* acc, int splits, int d) {
+  const int lane = threadIdx.x & (WAVE - 1);
+  const float2 mine = lane < splits ? *(const float2*)(ml + (size_t)lane * 2) : make_float2(-INFINITY, 0.f);
+  const float best = wave_max(mine.x);
+  const float weight = mine.x == -INFINITY ? 0.f : exp2f(mine.x - best);
+  const float total = wave_sum(mine.y * weight);
+  const float* mine_acc = acc + min(d, D - 1);
+  float sum = 0.f;
+  int first = 0;
+  for (; splits - first > 8; first += 32) sum += merge_some<32>(mine_acc, first, splits, weight);
+  if (first < splits) sum += merge_some<8>(mine_acc, first, splits, weight);
+  return total > 0.f ? sum / total : 0.f;
+}
+
+template <bool MAPS>
+__global__ __launch_bounds__(MERGE_THREADS) void attention_merge_finish_kernel(const float* __restrict__ partial_acc,
+                                                                               const float* __restrict__ partial_ml,
+                                                                               bf16_t* __restrict__ out, int out_stride, int splits,
+                                                                               int heads, Finish finish) {
+  __shared__ float shared[17];
+  const size_t row = blockIdx.x / (unsigned)heads;
+  const int head = blockIdx.x - (unsigned)row * heads, d = threadIdx.x;
+  const size_t pair = (size_t)blockIdx.x * (MAPS ? 2 : 1);
+  float v = merged_value(partial_ml + pair * splits * 2, partial_acc + pair * splits * D, splits, d);
+  if (MAPS) {
+    v -= finish.factor * merged_value(partial_ml + (pair + 1) * splits * 2, partial_acc + (pair + 1) * splits * D, splits, d);
+    const float squares = block_sum(d < finish.vdim ? v * v : 0.f, shared);
+    v *= finish.out_scale * rsqrtf(squares / (float)finish.vdim + finish.eps);
+  }
+  if (d >= finish.vdim) return;
+  const int column = head * finish.vdim + d;
+  if (!MAPS && finish.gates) v /= 1.f + expf(-(float)finish.gates[row * finish.gate_stride + finish.gate_first + column]);
+  out[row * out_stride + column] = (bf16_t)v;
 }
 
 static int launch_merge(float* partial_acc, float* partial_ml, void* out, int out_stride, int splits, size_t pairs, int heads,
@@ -1051,7 +1212,7 @@ static int launch_tiles(const void* qkv, int row_width, void* out, int out_strid
                         void* keys, void* values, const int* block_tables, int table_width,
                         const int* positions, const int* work, int tiles, int heads, int kv_heads,
                         int tokens_per_tile, int page_size, float scale, int window, int splits, FusedDecode fused,
-                        hipStream_t stream, ScoreChange change = {nullptr, 0.f, nullptr, 0, 0}) {
+                        hipStream_t stream, ScoreChange change, Finish finish) {
   const int group = heads / kv_heads;
   const int page_shift = (page_size & (page_size - 1)) == 0 ? __builtin_ctz(page_size) : -1;
   const int head_tiles = (group + 15) / 16;
@@ -1068,7 +1229,7 @@ static int launch_tiles(const void* qkv, int row_width, void* out, int out_strid
   hipLaunchKernelGGL((attention_tiles_kernel<COLUMN_TILES, FUSED, WAVES, CHANGED>), dim3(tiles, kv_heads * head_tiles, splits),
                      dim3(WAVES * 64), shared, stream, (const bf16_t*)qkv, row_width, (bf16_t*)out, out_stride, partial_acc,
                      partial_ml, (bf16_t*)keys, (bf16_t*)values, block_tables, table_width, positions, work,
-                     heads, kv_heads, tokens_per_tile, page_size, page_shift, scale, window, splits, fused, change);
+                     heads, kv_heads, tokens_per_tile, page_size, page_shift, scale, window, splits, fused, change, finish);
   return LAUNCH_STATUS();
 }
 
@@ -1101,21 +1262,33 @@ extern "C" int llmserve_attention_can_fuse(int pairing) {
 // this file), `sinks` (float32 [heads], or null) add exp(sink) to a head's denominator, `keep_first` keeps a sequence's first
 // keys visible behind a window, `chunk` (0 for none; not together with a window) shows a query the keys of its own chunk of
 // positions; slopes, cap and kept keys not together with `fuse` & 1, sinks not with `fuse` & 2.
-// A row of `out` begins every `out_stride` elements (a multiple of 4 from heads * D on).
+// `bias` (float32 [heads][reach + BIAS_SPARE], common.h: bias_element, or null) adds a bias by distance to the scores, `gates`
+// (bfloat16 rows of `gate_stride`, or null) multiplies a result's element with the sigmoid of column gate_first + its own;
+// `maps` 2: differential attention, column_tiles 2 with work items made for one column tile, partial results twice as many
+// ([rows * heads * 2 * splits ..]); each of the three writes heads of `vdim` side by side, and goes with no other change.
+// A row of `out` begins every `out_stride` elements (a multiple of 4 from heads * D, or heads * vdim, on).
 extern "C" int llmserve_attention_tiles(const void* qkv, int row_width, void* out, int out_stride, float* partial_acc,
                                         float* partial_ml, void* keys, void* values,
                                         const int* block_tables, int table_width, const int* positions,
                                         const int* work, int tiles, int column_tiles, int rows, int heads,
                                         int kv_heads, int page_size, float scale, int window, int splits, int fuse,
                                         const float* table, int pairing, const int* slots, const float* slopes,
-                                        float soft_cap, const float* sinks, int keep_first, int chunk, hipStream_t stream) {
+                                        float soft_cap, const float* sinks, int keep_first, int chunk, const float* bias, int reach,
+                                        int maps, int vdim, float factor, float eps, float out_scale, const void* gates,
+                                        int gate_stride, int gate_first, hipStream_t stream) {
   if (tiles <= 0) return 0;
   if (keep_first < 0 || chunk < 0 || (chunk > 0 && window > 0)) return ERR_BAD_ARGUMENT;
-  if (out_stride < heads * D || out_stride % 4) return ERR_BAD_ARGUMENT;
+  const bool finished = vdim > 0;
+  if (out_stride < heads * (finished ? vdim : D) || (out_stride % 4 && (!finished || vdim % 4 == 0))) return ERR_BAD_ARGUMENT;
+  if (vdim > D || (maps != 1 && maps != 2) || (!finished && (bias || gates || maps == 2)) || (bias && reach < 1)) return ERR_BAD_ARGUMENT;
+  if (finished && ((maps == 1) == (bias == nullptr) || fuse || slopes || soft_cap != 0.f || sinks || keep_first > 0 || chunk > 0)) return ERR_BAD_ARGUMENT;
+  if (maps == 2 && (D % 32 || gates || column_tiles != 2 || window > 0)) return ERR_BAD_ARGUMENT;
+  if (gates && (gate_first < 0 || gate_first + heads * vdim > gate_stride)) return ERR_BAD_ARGUMENT;
+  const Finish finish = {vdim, (const bf16_t*)gates, gate_stride, gate_first, factor, eps, out_scale};
   if (window <= 0) keep_first = 0;  // (without a window every key is seen anyway)
   const bool scores = slopes != nullptr || soft_cap > 0.f || keep_first > 0, edges = sinks != nullptr || chunk > 0;
   if (soft_cap < 0.f || (scores && (fuse & 1)) || (sinks && (fuse & 2))) return ERR_BAD_ARGUMENT;
-  const ScoreChange change = {slopes, soft_cap, sinks, keep_first, chunk};
+  const ScoreChange change = {slopes, soft_cap, sinks, keep_first, chunk, bias, reach};
   if (heads % kv_heads || page_size % 8 || splits < 1 || splits > MERGE_SPLITS_MAX || (splits > 1 && (!partial_acc || !partial_ml)))
     return ERR_BAD_ARGUMENT;
   if ((long)kv_heads * page_size * D >= (1L << 31)) return ERR_BAD_ARGUMENT;  // a page's elements are counted in 32 bits
@@ -1134,8 +1307,22 @@ extern "C" int llmserve_attention_tiles(const void* qkv, int row_width, void* ou
 #define LAUNCH_TILES(COLUMN_TILES, FUSED, WAVES, CHANGED)                                                                 \
   launch_tiles<COLUMN_TILES, FUSED, WAVES, CHANGED>(qkv, row_width, out, out_stride, partial_acc, partial_ml, keys, values, \
                                                     block_tables, table_width, positions, work, tiles, heads, kv_heads,     \
-                                                    tokens_per_tile, page_size, scale, window, splits, fused, stream, change)
+                                                    tokens_per_tile, page_size, scale, window, splits, fused, stream, change, finish)
     status = edges ? LAUNCH_TILES(1, true, FUSED_WAVES, CHANGED_EDGES) : LAUNCH_TILES(1, true, FUSED_WAVES, CHANGED_NOT);
+  } else if (finished) {
+#if HEAD_DIM % 32 == 0
+    if (maps == 2) status = LAUNCH_TILES(2, false, 4, CHANGED_MAPS);
+    else
+#endif
+    status = column_tiles == 1 ? LAUNCH_TILES(1, false, 4, CHANGED_BIAS) : LAUNCH_TILES(2, false, 4, CHANGED_BIAS);
+    if (status != 0 || splits == 1) return status;
+    if (maps == 2)
+      hipLaunchKernelGGL(attention_merge_finish_kernel<true>, dim3((unsigned)rows * heads), dim3(MERGE_THREADS), 0, stream, partial_acc,
+                         partial_ml, (bf16_t*)out, out_stride, splits, heads, finish);
+    else
+      hipLaunchKernelGGL(attention_merge_finish_kernel<false>, dim3((unsigned)rows * heads), dim3(MERGE_THREADS), 0, stream, partial_acc,
+                         partial_ml, (bf16_t*)out, out_stride, splits, heads, finish);
+    return LAUNCH_STATUS();
   } else if (column_tiles == 1) {
     status = scores  ? LAUNCH_TILES(1, false, 4, CHANGED_SCORES)
              : edges ? LAUNCH_TILES(1, false, 4, CHANGED_EDGES)

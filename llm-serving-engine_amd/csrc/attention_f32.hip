@@ -8,7 +8,9 @@
 // per query head) then adds -slope * (query position - key position).  With `sinks` (one per query head) the
 // softmax's denominator has exp(sink) more, once, with no value to it; it is added where a column's sums are final
 // (in the kernel that merges key splits, where there are splits).  `chunk` > 0 is a mask instead of a window: a query
-// sees the keys of its own chunk of so many positions, counted from the sequence's start.
+// sees the keys of its own chunk of so many positions, counted from the sequence's start.  `bias` (common.h: bias_element) is
+// added to a score by the distance between query and key.  With `maps` = m > 1 a query row holds m maps side by side, each
+// meets its own part of the keys and is an attention of its own: head h is map h % m of the queries' head h / m.
 //
 // The unit of work is an item: up to 16 * COLUMN_TILES "columns", the (token, query head) pairs of
 // consecutive tokens of one request that share one kv head, running through the tokens head by head so
@@ -49,7 +51,8 @@ __global__ __launch_bounds__(WAVES * 64) void attention_f32_kernel(
     float* __restrict__ partial_ml, const float* __restrict__ keys, const float* __restrict__ values,
     const int* __restrict__ block_tables, int table_width, const int* __restrict__ positions,
     const int* __restrict__ work, int heads, int kv_heads, int page_size, float scale_log2, int window, int splits,
-    int columns_total, const float* __restrict__ slopes, float soft_cap, const float* __restrict__ sinks, int keep_first, int chunk) {
+    int columns_total, const float* __restrict__ slopes, float soft_cap, const float* __restrict__ sinks, int keep_first, int chunk,
+    int maps, const float* __restrict__ bias, int reach) {
   __shared__ float wave_max[WAVES][COLUMN_TILES][16];
   __shared__ float wave_sum[WAVES][COLUMN_TILES][16];
   __shared__ __attribute__((aligned(16))) float merged[COLUMN_TILES][D_STEPS][64][4];
@@ -81,12 +84,16 @@ __global__ __launch_bounds__(WAVES * 64) void attention_f32_kernel(
     position[t] = live ? positions[token_row[t]] : -1;
     first[t] = first_seen_from(max(position[t], 0));
     if (CHANGED) slope[t] = slopes ? slopes[head[t]] * 1.4426950408889634f : 0.f;
-    const float* q = qkv + (size_t)token_row[t] * row_width + head[t] * D + 4 * g;
+    const int of_map = D / maps, map_first = head[t] % maps * of_map;
+    const float* q = qkv + (size_t)token_row[t] * row_width + head[t] / maps * D + 4 * g;
 #pragma unroll
     for (int s = 0; s < D_STEPS; ++s) {
       query[t][s] = load4(q + 16 * s);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) query[t][s][e] *= scale_log2;
+      for (int e = 0; e < 4; ++e) {
+        const int d = 16 * s + 4 * g + e;
+        query[t][s][e] = d >= map_first && d < map_first + of_map ? query[t][s][e] * scale_log2 : 0.f;
+      }
     }
   }
   // the item's keys: from the first that its first token sees to its last token's own
@@ -176,6 +183,7 @@ __global__ __launch_bounds__(WAVES * 64) void attention_f32_kernel(
         if (CHANGED) {  // scores are kept in units of log2: the cap is applied to the score itself
           if (soft_cap > 0.f) s4[e] = soft_cap * 1.4426950408889634f * tanhf(s4[e] * 0.6931471805599453f / soft_cap);
           s4[e] -= slope[t] * (float)(position[t] - key);
+          if (bias) s4[e] += bias[(size_t)head[t] * (reach + BIAS_SPARE) + bias_element(position[t] - key, reach)] * 1.4426950408889634f;
         }
         s4[e] = seen ? s4[e] : -INFINITY;
         best = fmaxf(best, s4[e]);
@@ -343,21 +351,23 @@ extern "C" int llmserve_attention_f32(const float* qkv, int row_width, float* ou
                                       const int* positions, const int* work, int items, int column_tiles, int tokens,
                                       int heads, int kv_heads, int page_size, float scale, int window, int splits,
                                       const float* slopes, float soft_cap, const float* sinks, int keep_first, int chunk,
-                                      hipStream_t stream) {
+                                      int maps, const float* bias, int reach, hipStream_t stream) {
   if (items <= 0 || tokens <= 0) return 0;
   if (keep_first < 0 || chunk < 0 || (chunk > 0 && (window > 0 || keep_first > 0))) return ERR_BAD_ARGUMENT;
   if (out_stride < heads * D || out_stride % 4) return ERR_BAD_ARGUMENT;
+  if (maps < 1 || heads % maps || D % maps || (bias && reach < 1)) return ERR_BAD_ARGUMENT;
   if (heads <= 0 || kv_heads <= 0 || heads % kv_heads || page_size <= 0 || page_size % 4 || splits < 1 ||
       splits > MERGE_SPLITS_MAX || (column_tiles != 1 && column_tiles != 2) || (splits > 1 && (!partial_acc || !partial_ml)))
     return ERR_BAD_ARGUMENT;
   const float scale_log2 = scale * 1.4426950408889634f;
   const int columns_total = tokens * heads;
   dim3 grid(items, kv_heads, splits);
-  const bool changed = slopes != nullptr || soft_cap > 0.f || sinks != nullptr || (keep_first > 0 && window > 0) || chunk > 0;
+  const bool changed = slopes != nullptr || soft_cap > 0.f || sinks != nullptr || (keep_first > 0 && window > 0) || chunk > 0 || bias != nullptr;
 #define LAUNCH_ATTENTION_F32(TILES, CHANGED)                                                                          \
   hipLaunchKernelGGL((attention_f32_kernel<TILES, CHANGED>), grid, dim3(WAVES * 64), 0, stream, qkv, row_width, out, out_stride, \
                      partial_acc, partial_ml, keys, values, block_tables, table_width, positions, work, heads,        \
-                     kv_heads, page_size, scale_log2, window, splits, columns_total, slopes, soft_cap, sinks, keep_first, chunk)
+                     kv_heads, page_size, scale_log2, window, splits, columns_total, slopes, soft_cap, sinks, keep_first, chunk, \
+                     maps, bias, reach)
   if (column_tiles == 1 && !changed) LAUNCH_ATTENTION_F32(1, false);
   else if (column_tiles == 1) LAUNCH_ATTENTION_F32(1, true);
   else if (!changed) LAUNCH_ATTENTION_F32(2, false);

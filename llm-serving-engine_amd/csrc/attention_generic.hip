@@ -10,7 +10,9 @@
 // `slopes` (one per query head) then adds -slope * (query position - key position), a bias that
 // grows with distance.  With `sinks` (one per query head) the softmax's denominator has exp(sink) more, once, with
 // no value to it: a key that is not there.  `chunk` > 0 is a mask instead of a window: a query sees the keys of its own chunk of
-// so many positions, counted from the sequence's start.
+// so many positions, counted from the sequence's start.  `bias` (common.h: bias_element) is added to a score by the distance
+// between query and key.  With `maps` = m > 1 a query row holds m maps side by side, each meets its own part of the keys and
+// is an attention of its own: head h is map h % m of the queries' head h / m.
 #include "common.h"
 
 #define KEYS_PER_TILE 128
@@ -22,7 +24,7 @@ __global__ __launch_bounds__(KEYS_PER_TILE) void attention_generic_kernel(
     const T* __restrict__ values, const int* __restrict__ block_tables, int table_width,
     const int* __restrict__ token_sequence, const int* __restrict__ positions, int heads, int kv_heads, int dim,
     int page_size, float scale, int window, const float* __restrict__ slopes, float soft_cap, const float* __restrict__ sinks,
-    int keep_first, int chunk) {
+    int keep_first, int chunk, int maps, const float* __restrict__ bias, int reach) {
   __shared__ float query[MAX_DIM];
   __shared__ float weights[KEYS_PER_TILE];
   __shared__ float shared[17];
@@ -30,8 +32,10 @@ __global__ __launch_bounds__(KEYS_PER_TILE) void attention_generic_kernel(
   const int kv_head = head / (heads / kv_heads);
   const int position = positions[token];
   const int* table = block_tables + (size_t)token_sequence[token] * table_width;
-  const T* q = qkv + (size_t)token * row_width + head * dim;
-  for (int d = threadIdx.x; d < dim; d += blockDim.x) query[d] = to_float(q[d]) * scale;
+  const T* q = qkv + (size_t)token * row_width + head / maps * dim;
+  const int of_map = dim / maps, map_first = head % maps * of_map;
+  for (int d = threadIdx.x; d < dim; d += blockDim.x)
+    query[d] = d >= map_first && d < map_first + of_map ? to_float(q[d]) * scale : 0.f;
   __syncthreads();
 
   const int first = chunk > 0 ? position - position % chunk : window > 0 ? max(0, position - window + 1) : 0;
@@ -60,6 +64,7 @@ __global__ __launch_bounds__(KEYS_PER_TILE) void attention_generic_kernel(
       score = dot;
       if (soft_cap > 0.f) score = soft_cap * tanhf(score / soft_cap);
       score -= slope * (float)(position - key);
+      if (bias) score += bias[(size_t)head * (reach + BIAS_SPARE) + bias_element(position - key, reach)];
     }
     const float tile_max = block_max(score, shared);
     const float next_max = fmaxf(running_max, tile_max);
@@ -102,19 +107,22 @@ extern "C" int llmserve_attention_generic(const void* qkv, int row_width, void* 
                                           const int* token_sequence, const int* positions, int tokens, int heads,
                                           int kv_heads, int dim, int page_size, float scale, int window,
                                           const float* slopes, float soft_cap, const float* sinks, int keep_first,
-                                          int chunk, hipStream_t stream) {
+                                          int chunk, int maps, const float* bias, int reach, hipStream_t stream) {
   if (tokens <= 0) return 0;
   if (dim > MAX_DIM || dim <= 0 || heads % kv_heads || page_size <= 0 || keep_first < 0 || chunk < 0 ||
-      (chunk > 0 && (window > 0 || keep_first > 0)) || out_stride < heads * dim)
+      (chunk > 0 && (window > 0 || keep_first > 0)) || out_stride < heads * dim || maps < 1 || heads % maps || dim % maps ||
+      (bias && reach < 1))
     return ERR_BAD_ARGUMENT;
   dim3 grid(tokens, heads);
   if (is_float)
     hipLaunchKernelGGL(attention_generic_kernel<float>, grid, dim3(KEYS_PER_TILE), 0, stream, (const float*)qkv,
                        row_width, (float*)out, out_stride, (const float*)keys, (const float*)values, block_tables, table_width,
-                       token_sequence, positions, heads, kv_heads, dim, page_size, scale, window, slopes, soft_cap, sinks, keep_first, chunk);
+                       token_sequence, positions, heads, kv_heads, dim, page_size, scale, window, slopes, soft_cap, sinks, keep_first, chunk,
+                       maps, bias, reach);
   else
     hipLaunchKernelGGL(attention_generic_kernel<bf16_t>, grid, dim3(KEYS_PER_TILE), 0, stream, (const bf16_t*)qkv,
                        row_width, (bf16_t*)out, out_stride, (const bf16_t*)keys, (const bf16_t*)values, block_tables, table_width,
-                       token_sequence, positions, heads, kv_heads, dim, page_size, scale, window, slopes, soft_cap, sinks, keep_first, chunk);
+                       token_sequence, positions, heads, kv_heads, dim, page_size, scale, window, slopes, soft_cap, sinks, keep_first, chunk,
+                       maps, bias, reach);
   return LAUNCH_STATUS();
 }

@@ -97,3 +97,10 @@ __device__ __forceinline__ size_t value_element(int d, int offset, int page_size
   const int width = value_piece_width(page_size);
   return ((size_t)(offset / width) * dim + d) * width + offset % width;
 }
+
+// A learned bias by distance: the biases of one head, `reach + 24` floats, lie against the distance, so that consecutive
+// keys are consecutive floats: the bias of distance d (query position - key position, at most reach + 7) is element
+// reach + 7 - d, and the seven behind it are those of the next keys.  Distances from reach - 1 on have the same bias, those
+// below 0 (keys that are masked) nothing.
+#define BIAS_SPARE 24
+__device__ __forceinline__ int bias_element(int distance, int reach) { return reach + 7 - max(min(distance, reach + 7), -8); }

@@ -5,22 +5,33 @@
 
 // ---------------------------------------------------------------------------- embedding
 // out[t, :] = float(table[ids[t], :]) * scale        (reference model.py:293, which has no scale)
+// With `places` (a learned vector a position, [place_rows, hidden], of the table's type) row positions[t] of it is added.
 template <typename T>
 __global__ void embedding_kernel(const T* __restrict__ table, const int* __restrict__ ids,
-                                 float* __restrict__ out, int hidden, float scale) {
+                                 float* __restrict__ out, int hidden, float scale, const T* __restrict__ places,
+                                 const int* __restrict__ positions, int place_rows) {
   const size_t row = (size_t)ids[blockIdx.x];
   const T* src = table + row * hidden;
   float* dst = out + (size_t)blockIdx.x * hidden;
+  if (places) {
+    const T* place = places + (size_t)min(max(positions[blockIdx.x], 0), place_rows - 1) * hidden;
+    for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = to_float(src[i]) * scale + to_float(place[i]);
+    return;
+  }
   for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = to_float(src[i]) * scale;
 }
 
 extern "C" int llmserve_embedding(const void* table, int table_is_float, const int* ids, float* out,
-                                  int tokens, int hidden, float scale, hipStream_t stream) {
+                                  int tokens, int hidden, float scale, const void* places, const int* positions, int place_rows,
+                                  hipStream_t stream) {
   if (tokens <= 0) return 0;
+  if (places && (!positions || place_rows < 1)) return ERR_BAD_ARGUMENT;
   if (table_is_float)
-    hipLaunchKernelGGL(embedding_kernel<float>, dim3(tokens), dim3(256), 0, stream, (const float*)table, ids, out, hidden, scale);
+    hipLaunchKernelGGL(embedding_kernel<float>, dim3(tokens), dim3(256), 0, stream, (const float*)table, ids, out, hidden, scale,
+                       (const float*)places, positions, place_rows);
   else
-    hipLaunchKernelGGL(embedding_kernel<bf16_t>, dim3(tokens), dim3(256), 0, stream, (const bf16_t*)table, ids, out, hidden, scale);
+    hipLaunchKernelGGL(embedding_kernel<bf16_t>, dim3(tokens), dim3(256), 0, stream, (const bf16_t*)table, ids, out, hidden, scale,
+                       (const bf16_t*)places, positions, place_rows);
   return LAUNCH_STATUS();
 }
 

@@ -652,24 +652,29 @@ extern "C" int llmserve_expert_product(const void* x, int is_float, const int* o
 // out[t] = sum_i weight[t, i] * rows[place[t * top + i]], in the order of i; with `shared`, plus
 // sigmoid(gates[t, gate_column]) * shared[t] (an expert that every token uses, behind a gate of its own).
 __global__ void combine_pairs_kernel(const float* __restrict__ rows, const int* __restrict__ place, const float* __restrict__ weight,
-                                     int top, float* __restrict__ out, int width, const float* __restrict__ shared,
+                                     int top, float* __restrict__ out, int width, const float* __restrict__ shared, int parts,
                                      const float* __restrict__ gates, int gate_stride, int gate_column) {
   const int t = blockIdx.x;
   const float gate = shared ? (gates ? 1.f / (1.f + expf(-gates[(size_t)t * gate_stride + gate_column])) : 1.f) : 0.f;
   for (int c = threadIdx.x; c < width; c += blockDim.x) {
     float sum = 0.f;
     for (int i = 0; i < top; ++i) sum += weight[(size_t)t * top + i] * rows[(size_t)place[(size_t)t * top + i] * width + c];
-    if (shared) sum += gate * shared[(size_t)t * width + c];
+    if (shared) {
+      float beside = shared[(size_t)t * width + c];
+      for (int p = 1; p < parts; ++p) beside += shared[((size_t)p * gridDim.x + t) * width + c];
+      sum += gate * beside;
+    }
     out[(size_t)t * width + c] = sum;
   }
 }
 
 extern "C" int llmserve_combine_pairs(const float* rows, const int* place, const float* weight, int top, float* out, int tokens,
-                                      int width, const float* shared, const float* gates, int gate_stride, int gate_column,
+                                      int width, const float* shared, int parts, const float* gates, int gate_stride, int gate_column,
                                       hipStream_t stream) {
   if (tokens <= 0) return 0;
+  if (shared && parts < 1) return ERR_BAD_ARGUMENT;
   if (shared && gates && (gate_column < 0 || gate_column >= gate_stride)) return ERR_BAD_ARGUMENT;  // (no gates: the shared rows are added as they are)
-  hipLaunchKernelGGL(combine_pairs_kernel, dim3(tokens), dim3(256), 0, stream, rows, place, weight, top, out, width, shared, gates,
-                     gate_stride, gate_column);
+  hipLaunchKernelGGL(combine_pairs_kernel, dim3(tokens), dim3(256), 0, stream, rows, place, weight, top, out, width, shared, parts,
+                     gates, gate_stride, gate_column);
   return LAUNCH_STATUS();
 }

@@ -48,7 +48,7 @@ def _pointer(tensor: torch.Tensor | None) -> int | None:
 # Argument types of every entry point: p pointer, i int, f float.  Declared once, so that a call
 # costs no guessing: a decode step is replayed from a graph, but every other step pays per launch.
 _SIGNATURES = {
-    "llmserve_embedding": "pippiifp",
+    "llmserve_embedding": "pippiifppip",
     "llmserve_add_rms_norm": "ppipipiiifp",
     "llmserve_rotary_table": "pppiip",
     "llmserve_rotate_and_store": "piipiiiiipppip",
@@ -69,9 +69,9 @@ _SIGNATURES = {
     "llmserve_gemm_ring": "pppipiiiiiiip",
     "llmserve_gemm_merged": "ppippipiiiip",
     "llmserve_gemm_tiled": "pppipiiiiiip",
-    "llmserve_attention_generic": "pipiipppippiiiiifipfpiip",
-    "llmserve_attention_f32": "pipipppppippiiiiiifiipfpiip",
-    "llmserve_attention_tiles": "pipipppppippiiiiiifiiipippfpiip",
+    "llmserve_attention_generic": "pipiipppippiiiiifipfpiiipip",
+    "llmserve_attention_f32": "pipipppppippiiiiiifiipfpiiipip",
+    "llmserve_attention_tiles": "pipipppppippiiiiiifiiipippfpiipiiifffpiip",
     "llmserve_attention_portions": "pipipppppippiiiiiifiip",
     "llmserve_attention_can_fuse": "i",
     "llmserve_argmax": "ppppiip",
@@ -91,7 +91,7 @@ _SIGNATURES = {
     "llmserve_sort_pairs": "piipppiip",
     "llmserve_expert_product": "pipipiipiipiifp",
     "llmserve_expert_product_gates": "iii",
-    "llmserve_combine_pairs": "pppipiippiip",
+    "llmserve_combine_pairs": "pppipiipipiip",
     "llmserve_conv_gated_delta_rule": "piiipipppppiiiippiiippppppip",
     "llmserve_causal_conv": "piiiipipppipppip",
     "llmserve_gated_delta_rule": "pipppiiiippiiipppppip",
@@ -107,6 +107,10 @@ _SIGNATURES = {
     "llmserve_stream_norm": "ppiippppipipiiifp",
     "llmserve_add_scaled": "pifpifpiip",
     "llmserve_gated_recurrence": "pippppiiiippiippp",
+    "llmserve_convolved_heads_stores": "iiiiiiiiiii",
+    "llmserve_convolved_heads": "piiiiiiiiiiiiifppipiippppipfipipppip",
+    "llmserve_difference_heads": "pipiiiifffp",
+    "llmserve_gate_columns": "piipiiiiipiip",
 }
 _TYPES = {"p": ctypes.c_void_p, "i": ctypes.c_int, "f": ctypes.c_float}
 
@@ -278,11 +282,16 @@ class HipKernels:
 
     # ------------------------------------------------------------------ elementwise
 
-    def embedding(self, table: torch.Tensor, token_ids: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
+    def embedding(self, table: torch.Tensor, token_ids: torch.Tensor, scale: float = 1.0, positions=None, position_table=None) -> torch.Tensor:
         tokens, hidden = token_ids.shape[0], table.shape[1]
+        if (positions is None) != (position_table is None):
+            raise KernelError("embedding: positions and a table for them come together")
+        if position_table is not None and (position_table.dtype != table.dtype or position_table.shape[1:] != (hidden,) or positions.shape != (tokens,)):
+            raise KernelError("embedding: the table of positions has rows like the embedding's, and every token a position")
         out = self._empty((tokens, hidden), torch.float32)
         status = self._elementwise.llmserve_embedding(
-            _pointer(table), _is_float(table), _pointer(token_ids), _pointer(out), tokens, hidden, float(scale), self._stream
+            _pointer(table), _is_float(table), _pointer(token_ids), _pointer(out), tokens, hidden, float(scale), _pointer(position_table),
+            _pointer(positions), position_table.shape[0] if position_table is not None else 0, self._stream,
         )
         _check(status, "embedding")
         return out
@@ -834,14 +843,136 @@ class HipKernels:
     def paged_attention(
         self, qkv, layout, batch, cell, scale: float, window: int | None, *,
         score_slopes: torch.Tensor | None = None, soft_cap: float | None = None, sinks: torch.Tensor | None = None,
-        keep_first: int = 0, chunk: int | None = None, out: torch.Tensor | None = None,
+        keep_first: int = 0, chunk: int | None = None, out: torch.Tensor | None = None, vdim: int | None = None, distance_bias=None,
+        gates=None, maps: int = 1,
     ) -> torch.Tensor:
         """`score_slopes` (float32 [heads]) and `soft_cap` change the scores before the softmax: cap * tanh(score /
         cap), then minus slope * distance; `sinks` (float32 [heads]) add exp(sink) to a head's denominator; with
         `keep_first` a sequence's first so many keys stay visible behind the window, at their own positions.  The
         matrix-core kernels of both precisions take them (in bfloat16 not the forms that fuse the rotation or share
         keys through LDS).  `chunk` is a mask instead of a window: a query sees the keys of its own chunk of so many positions.
-        With `out` (rows of the run dtype, as wide as the heads or wider) the result is its first columns."""
+        With `out` (rows of the run dtype, as wide as the heads or wider) the result is its first columns.  With `vdim`, `distance_bias`
+        or `gates` the results are heads of `vdim` side by side: in bfloat16 the matrix-core kernel adds the bias and writes them
+        gated; elsewhere a kernel of its own brings them together behind the attention.  `maps` (of the kernels that are
+        not for bfloat16 on the matrix cores): a query row holds so many maps side by side, and the result is one head a map."""
+        if vdim is not None or distance_bias is not None or gates is not None:
+            if score_slopes is not None or soft_cap is not None or sinks is not None or keep_first or chunk or maps != 1:
+                raise KernelError("paged_attention: finished results go with no other change of the scores")
+            return self._finished_attention(qkv, layout, batch, cell, scale, window, out, vdim or layout.head_dim, distance_bias, gates)
+        return self._paged_attention(qkv, layout, batch, cell, scale, window, score_slopes, soft_cap, sinks, keep_first, chunk, out, maps=maps)
+
+    def prepare_distance_bias(self, by_distance: torch.Tensor):
+        """(float32 [heads, reach + 24] as the kernels read it (csrc/common.h: bias_element), reach)."""
+        heads, reach = by_distance.shape
+        distances = (reach + 7 - torch.arange(reach + 24)).clamp(max=reach - 1)
+        table = by_distance.float().cpu()[:, distances.clamp(min=0)]
+        table[:, distances < 0] = 0.0
+        return self.to_device(table.contiguous()), reach
+
+    def _finished_attention(self, qkv, layout, batch, cell, scale, window, out, vdim: int, distance_bias, gates):
+        tokens, heads, dim = qkv.shape[0], layout.num_heads, layout.head_dim
+        group = batch.groups[cell.group]
+        if not 0 < vdim <= dim:
+            raise KernelError("paged_attention: a head's result is as wide as a head or narrower")
+        if out is None:
+            out = self._empty((tokens, heads * vdim), qkv.dtype)
+        if out.dtype != qkv.dtype or out.shape[0] != tokens or out.shape[1] < heads * vdim:
+            raise KernelError("paged_attention: the rows to write are of the queries' type, one a token, and wide enough")
+        gate_rows, gate_first = gates if gates is not None else (None, 0)
+        if gate_rows is not None and (gate_rows.dtype != qkv.dtype or gate_rows.shape[0] != tokens or gate_first + heads * vdim > gate_rows.shape[1]):
+            raise KernelError("paged_attention: gates are columns of rows of the queries' type, one a token")
+        if distance_bias is not None and distance_bias[0].shape != (heads, distance_bias[1] + 24):
+            raise KernelError("paged_attention: a bias for every head and distance")
+        if cell.keys.dtype != qkv.dtype or qkv.shape[1] != layout.stride or int(getattr(cell.need, "keep_first", 0) or 0):
+            raise KernelError("paged_attention: queries and pages of one type, rows of the layout's width, no kept first keys")
+        if distance_bias is not None and self._tiles_take(qkv, layout, group) and (out.shape[1] % 4 == 0 or vdim % 4):
+            self._attention_tiles(qkv, out, layout, batch, cell, group, scale, int(window or 0),
+                                  finish=(distance_bias, 1, vdim, 0.0, 0.0, 0.0, gate_rows, gate_first))
+            return out
+        wide = self._paged_attention(qkv, layout, batch, cell, scale, window, None, None, None, 0, None, None, distance_bias=distance_bias)
+        if gate_rows is None and vdim == dim and out.shape[1] == wide.shape[1]:
+            return out.copy_(wide)
+        status = self._library_of("convolved_heads").llmserve_gate_columns(
+            _pointer(wide), _is_float(wide), wide.shape[1], _pointer(out), out.shape[1], tokens, heads, dim, vdim, _pointer(gate_rows),
+            gate_rows.shape[1] if gate_rows is not None else 0, gate_first, self._stream,
+        )
+        _check(status, "gate_columns")
+        return out
+
+    @staticmethod
+    def _tiles_take(qkv, layout, group) -> bool:
+        """Whether the bfloat16 matrix-core kernel takes these queries, heads and pages."""
+        dim = layout.head_dim
+        return qkv.dtype == torch.bfloat16 and group.page_size % 8 == 0 and dim % 16 == 0 and 16 <= dim <= 256 and layout.stride % 8 == 0
+
+    def difference_attention(self, rows, layout, batch, cell, scale: float, vdim: int, factor: float, eps: float, out_scale: float):
+        """In bfloat16 one kernel (and one that merges key splits): both maps of a head walk the keys together, and their
+        normed difference is what is written.  Elsewhere the maps are heads of the plain attention, put together behind it."""
+        tokens, heads, dim = rows.shape[0], layout.num_heads, layout.head_dim
+        group = batch.groups[cell.group]
+        if dim % 2 or not 0 < vdim <= dim:
+            raise KernelError("difference_attention: two maps of one width, and values as wide as both or narrower")
+        if cell.keys.dtype != rows.dtype or rows.shape[1] != layout.stride or int(getattr(cell.need, "keep_first", 0) or 0):
+            raise KernelError("difference_attention: queries and pages of one type, rows of the layout's width, no kept first keys")
+        out = self._empty((tokens, heads * vdim), rows.dtype)
+        if self._tiles_take(rows, layout, group) and dim % 32 == 0 and (heads * vdim % 4 == 0 or vdim % 4):
+            self._attention_tiles(rows, out, layout, batch, cell, group, scale, 0, finish=(None, 2, vdim, factor, eps, out_scale, None, 0))
+            return out
+        maps = self._paged_attention(rows, layout, batch, cell, scale, None, None, None, None, 0, None, None, maps=2)
+        status = self._library_of("convolved_heads").llmserve_difference_heads(
+            _pointer(maps), _is_float(maps), _pointer(out), tokens, heads, dim, vdim, float(factor), float(eps), float(out_scale), self._stream
+        )
+        _check(status, "difference_attention")
+        return out
+
+    def convolved_heads(self, x, q_first: int, k_first: int, v_first: int, heads: int, kv_heads: int, dim: int, vdim: int, width: int, batch,
+                        cell=None, *, maps: int = 1, taps=None, window=None, norm: bool = True, q_weight=None, k_weight=None,
+                        eps: float = 0.0, temperature=None):
+        """With a writable `cell` the keys and values are also stored in its pages: by this kernel in a step of single tokens
+        (sizes that come in 16-byte pieces), by the kernel that stores prompt portions otherwise."""
+        tokens = x.shape[0]
+        if (q_weight is None) != (k_weight is None) and kv_heads or (q_weight is not None and (not norm or q_weight.shape != (dim,))) \
+                or (k_weight is not None and (k_weight.shape != (dim,) or k_weight.dtype != q_weight.dtype)):
+            raise KernelError("convolved_heads: the norms' weights are of one type, as long as a map")
+        if width % maps:
+            raise KernelError("convolved_heads: a head's row is as wide as its maps side by side")
+        channels = 0
+        if taps is not None:
+            channels = heads * maps * dim + kv_heads * (maps * dim + vdim)
+            if taps.dtype != torch.float32 or taps.ndim != 2 or taps.shape[0] != channels or (q_first, k_first, v_first) != (0, heads * maps * dim, heads * maps * dim + kv_heads * maps * dim):
+                raise KernelError("convolved_heads: float32 taps, a row a channel of queries, keys and values side by side")
+            if taps.shape[1] > 1 and (window is None or window.dtype != torch.float32 or window.shape[1:] != (taps.shape[1] - 1, channels)):
+                raise KernelError("convolved_heads: the kept inputs are float32 [slots, taps - 1, channels]")
+        coef, every = temperature if temperature is not None else (0.0, 0)
+        if temperature is not None and not every >= 1:
+            raise KernelError("convolved_heads: a temperature grows every so many positions")
+        out = self._empty((tokens, (heads + 2 * kv_heads) * width), x.dtype)
+        store = cell is not None and cell.writable
+        group = batch.groups[cell.group] if store else None
+        if store and (cell.keys.dtype != x.dtype or cell.values.shape[1:] != cell.need.page_fields(group.page_size)["values"]
+                      or (cell.need.num_kv_heads, cell.need.head_dim) != (kv_heads, width)):
+            raise KernelError("convolved_heads: the cell's pages do not fit the heads")
+        library = self._library_of("convolved_heads")
+        tap_count = taps.shape[1] if taps is not None else 0
+        single = batch.max_query_length == 1
+        here = store and single and bool(library.llmserve_convolved_heads_stores(
+            _is_float(x), x.shape[1], q_first, k_first, v_first, maps, dim, vdim, width, tap_count, channels))
+        status = library.llmserve_convolved_heads(
+            _pointer(x), _is_float(x), tokens, x.shape[1], q_first, k_first, v_first, heads, kv_heads, maps, dim, vdim, width, 1 if norm else 0,
+            float(eps), _pointer(q_weight), _pointer(k_weight), _is_float(q_weight) if q_weight is not None else 0, _pointer(taps), tap_count, channels,
+            _pointer(window if tap_count > 1 else None), _pointer(batch.token_sequence), _pointer(batch.query_start), _pointer(batch.state_slots),
+            batch.state_slots.shape[0], _pointer(batch.positions), float(coef), int(every), _pointer(out), 1 if single else 0,
+            _pointer(cell.keys if here else None), _pointer(cell.values if here else None), _pointer(group.slot_mapping if here else None),
+            group.page_size if here else 1, self._stream,
+        )
+        _check(status, "convolved_heads")
+        if store and not here:
+            layout = types.SimpleNamespace(num_heads=heads, num_kv_heads=kv_heads, head_dim=width, stride=out.shape[1])
+            self.rotate_and_store(out, layout, batch, cell, None, "none")
+        return out
+
+    def _paged_attention(self, qkv, layout, batch, cell, scale, window, score_slopes, soft_cap, sinks, keep_first, chunk, out, *, maps: int = 1,
+                         distance_bias=None):
         tokens = qkv.shape[0]
         group = batch.groups[cell.group]
         if cell.keys.dtype != qkv.dtype:
@@ -860,16 +991,18 @@ class HipKernels:
             raise KernelError("paged_attention: a mask is a window or chunks")
         if qkv.shape[1] != layout.stride:
             raise KernelError("paged_attention: qkv does not have the layout's width")
-        out = self._attention_out(qkv, layout, out)
+        heads = layout.num_heads * maps
+        out = self._attention_out(qkv, layout, out) if maps == 1 else self._empty((tokens, heads * layout.head_dim), qkv.dtype)
         dim = layout.head_dim
+        bias, reach = distance_bias if distance_bias is not None else (None, 0)
         plain_scores = score_slopes is None and soft_cap is None and sinks is None and not keep_first and not chunk
         aligned = layout.stride % 8 == 0 and out.shape[1] % 8 == 0  # (rows are read and written in pieces of 8 or 16 bytes)
-        if qkv.dtype == torch.bfloat16 and group.page_size % 8 == 0 and dim % 16 == 0 and 16 <= dim <= 256 and aligned:
+        if qkv.dtype == torch.bfloat16 and group.page_size % 8 == 0 and dim % 16 == 0 and 16 <= dim <= 256 and aligned and maps == 1 and bias is None:
             changed = None if plain_scores else (score_slopes, float(soft_cap or 0.0), sinks, keep_first, chunk)
             self._attention_tiles(qkv, out, layout, batch, cell, group, scale, int(window or 0), changed=changed)
             return out
         if qkv.dtype == torch.float32 and group.page_size % 4 == 0 and dim % 16 == 0 and 16 <= dim <= 256 and aligned:
-            self._attention_float32(qkv, out, layout, batch, cell, group, scale, int(window or 0), score_slopes, soft_cap, sinks, keep_first, chunk)
+            self._attention_float32(qkv, out, layout, batch, cell, group, scale, int(window or 0), score_slopes, soft_cap, sinks, keep_first, chunk, maps, bias, reach)
             return out
         if qkv.dtype == torch.bfloat16:
             why = f"head size {dim} and pages of {group.page_size}"
@@ -877,8 +1010,9 @@ class HipKernels:
         status = self._attention_generic.llmserve_attention_generic(
             _pointer(qkv), layout.stride, _pointer(out), out.shape[1], _is_float(qkv), _pointer(cell.keys), _pointer(cell.values),
             _pointer(group.block_tables), group.width, _pointer(batch.token_sequence), _pointer(batch.positions),
-            tokens, layout.num_heads, layout.num_kv_heads, dim, group.page_size,
-            scale, int(window or 0), _pointer(score_slopes), float(soft_cap or 0.0), _pointer(sinks), keep_first, chunk, self._stream,
+            tokens, heads, layout.num_kv_heads, dim, group.page_size,
+            scale, int(window or 0), _pointer(score_slopes), float(soft_cap or 0.0), _pointer(sinks), keep_first, chunk, maps, _pointer(bias), reach,
+            self._stream,
         )
         _check(status, "paged_attention")
         return out
@@ -898,14 +1032,14 @@ class HipKernels:
         return min(batch.max_context_length, reach) if reach else batch.max_context_length
 
     def _attention_float32(self, qkv, out, layout, batch, cell, group, scale: float, window: int, score_slopes=None, soft_cap=None, sinks=None,
-                           keep_first: int = 0, chunk: int = 0) -> None:
+                           keep_first: int = 0, chunk: int = 0, maps: int = 1, bias=None, reach: int = 0) -> None:
         """The 32-bit path's attention on the matrix cores: an item is 16 (decoding) or 32 columns of one
         request, (token, head) pairs running through the tokens head by head whatever the number of heads; few
         items over long contexts are cut into key splits that a second kernel merges."""
         dim = layout.head_dim
         if dim not in self._attention_f32:
             self._attention_f32[dim] = _declared(load_module("attention_f32", {"HEAD_DIM": dim}))
-        heads, kv_heads = layout.num_heads, layout.num_kv_heads
+        heads, kv_heads = layout.num_heads * maps, layout.num_kv_heads
         group_size = heads // kv_heads
         column_tiles = 2 if batch.max_query_length * group_size > 16 else 1
         work, items, _ = self._attention_work(batch, group_size, column_tiles, 0, None, True)
@@ -926,11 +1060,11 @@ class HipKernels:
             _pointer(qkv), layout.stride, _pointer(out), out.shape[1], _pointer(partial_acc), _pointer(partial_ml), _pointer(cell.keys),
             _pointer(cell.values), _pointer(group.block_tables), group.width, _pointer(batch.positions), _pointer(work),
             items, column_tiles, tokens, heads, kv_heads, group.page_size, scale, window, splits, _pointer(score_slopes),
-            float(soft_cap or 0.0), _pointer(sinks), keep_first, chunk, self._stream,
+            float(soft_cap or 0.0), _pointer(sinks), keep_first, chunk, maps, _pointer(bias), reach, self._stream,
         )
         _check(status, "paged_attention")
 
-    def _attention_tiles(self, qkv, out, layout, batch, cell, group, scale: float, window: int, fuse=None, unmerged=False, changed=None):
+    def _attention_tiles(self, qkv, out, layout, batch, cell, group, scale: float, window: int, fuse=None, unmerged=False, changed=None, finish=None):
         """The MFMA kernel: requests that bring a few tokens (decoding) one column tile per
         wave, split over the keys when there are few of them; longer portions two tiles
         per wave.  `fuse` = (rotary table, pairing) lets a step of single tokens rotate and
@@ -939,8 +1073,12 @@ class HipKernels:
         (their results in bfloat16, laid out for `gemm_merged`; their maxima and sums in float32; how
         many), instead of `out`.  `changed` = (slopes or None, soft cap or 0.0, sinks or None, kept first keys or 0, chunk or 0): scores
         changed before the softmax, a sink in its denominator, a sequence's first keys kept visible behind the window, or a mask
-        in chunks, which the kernel that shares keys through LDS does not take; `fuse` takes sinks and chunks alone."""
+        in chunks, which the kernel that shares keys through LDS does not take; `fuse` takes sinks and chunks alone.
+        `finish` = (bias by distance or None, maps, vdim, factor, eps, scale of the result, gates or None, their first column): the
+        kinds that write finished results, a bias by distance with gates or the difference of two maps."""
         slopes, soft_cap, sinks, keep_first, chunk = changed if changed is not None else (None, 0.0, None, 0, 0)
+        bias, maps, vdim, factor, eps, out_scale, gates, gate_first = finish if finish is not None else (None, 1, 0, 0.0, 0.0, 0.0, None, 0)
+        bias, reach = bias if bias is not None else (None, 0)
         if fuse is not None and (slopes is not None or soft_cap or keep_first):
             raise KernelError("paged_attention: the fused decode form leaves the scores as they are")
         library = self._attention_library(layout.head_dim)
@@ -953,7 +1091,7 @@ class HipKernels:
         shared = False
         padded = getattr(batch, "padded_to", None) is not None  # a captured step: the same launches whatever it holds
         whole_pages = group.page_size >= 16 and group.page_size & (group.page_size - 1) == 0  # (what that kernel takes)
-        if batch.max_query_length > per_tile and layout.head_dim == 128 and fuse is None and changed is None and self.shared_portions != "never" and not padded and whole_pages:
+        if batch.max_query_length > per_tile and layout.head_dim == 128 and fuse is None and changed is None and finish is None and self.shared_portions != "never" and not padded and whole_pages:
             # Prompt portions at this head size may go to the kernel whose waves share each step's K and V
             # through LDS (a quarter of the cache traffic; what bounds the kernel above over long walks is the
             # path from the caches into the registers).  Its workgroups take 128 columns and walk all their keys,
@@ -1000,7 +1138,7 @@ class HipKernels:
         elif batch.max_query_length > per_tile:
             # two column tiles a wave (heads wider than 128 leave no registers for more than one); four, at
             # one wave a SIMD, were ahead beyond 4,096 keys only while the key pages were whole rows
-            wide = 1 if layout.head_dim > 128 else 2
+            wide = 1 if layout.head_dim > 128 or maps > 1 else 2
             # One launch takes the requests of few tokens along (a decoded token fills part of a tile): in a
             # step of portions beside decoded tokens two launches one after the other cost 11 us each at the
             # 1.5B sizes, and the walk of a decoded token's keys is the same in either kernel.
@@ -1065,14 +1203,16 @@ class HipKernels:
                     splits = max(splits, min(-(-steps // 16), 192 // blocks, 64))
                 if splits > 1:
                     held = 16 if unmerged else tokens  # the product that merges wants 16 rows side by side
-                    partial_acc = self._empty((held * heads * splits * layout.head_dim,), qkv.dtype if unmerged else torch.float32)
-                    partial_ml = self._empty((held * heads * splits * 2,), torch.float32)
+                    partial_acc = self._empty((held * heads * maps * splits * layout.head_dim,), qkv.dtype if unmerged else torch.float32)
+                    partial_ml = self._empty((held * heads * maps * splits * 2,), torch.float32)
             table, pairing = fuse if fuse is not None else (None, "none")
             status = library.llmserve_attention_tiles(
                 _pointer(qkv), layout.stride, _pointer(out), out.shape[1], _pointer(partial_acc), _pointer(partial_ml),
-                _pointer(cell.keys), _pointer(cell.values), _pointer(group.block_tables), group.width, _pointer(batch.positions), _pointer(work), items, column_tiles, tokens, heads, kv_heads,
-                group.page_size, scale, window, splits, (1 if fuse is not None else 0) + (2 if unmerged else 0) + (4 if by_item else 0),
-                _pointer(table), _PAIRINGS[pairing], _pointer(group.slot_mapping), _pointer(slopes), soft_cap, _pointer(sinks), keep_first, chunk, self._stream,
+                _pointer(cell.keys), _pointer(cell.values), _pointer(group.block_tables), group.width, _pointer(batch.positions), _pointer(work), items,
+                column_tiles if maps == 1 else 2, tokens, heads, kv_heads, group.page_size, scale, window, splits, (1 if fuse is not None else 0) + (2 if unmerged else 0) + (4 if by_item else 0),
+                _pointer(table), _PAIRINGS[pairing], _pointer(group.slot_mapping), _pointer(slopes), soft_cap, _pointer(sinks), keep_first, chunk,
+                _pointer(bias), reach, maps, vdim, float(factor), float(eps), float(out_scale), _pointer(gates),
+                gates.shape[1] if gates is not None else 0, gate_first, self._stream,
             )
             _check(status, "paged_attention")
             if unmerged and splits > 1:
@@ -1363,11 +1503,12 @@ class HipKernels:
         _check(library.llmserve_expert_product(
             _pointer(inner), _is_float(inner), _pointer(order), 0, _pointer(downs), hidden, size, _pointer(tiles), capacity, tile_rows, _pointer(rows),
             1, -1, 0.0, self._stream), "experts: second product")
-        if shared is not None and (shared.dtype != torch.float32 or shared.shape != (tokens, hidden) or (gates is not None and gates.dtype != torch.float32)):
+        if shared is not None and (shared.dtype != torch.float32 or shared.shape[-2:] != (tokens, hidden) or (gates is not None and gates.dtype != torch.float32)):
             raise KernelError("experts: the shared rows and their gates are float32")
         out = self._empty((tokens, hidden), torch.float32)
         _check(library.llmserve_combine_pairs(
             _pointer(rows), _pointer(place), _pointer(weights), top, _pointer(out), tokens, hidden, _pointer(shared),
+            shared.shape[0] if shared is not None and shared.ndim == 3 else 1,
             _pointer(gates if shared is not None else None), gates.shape[1] if shared is not None and gates is not None else 1, gate_column,
             self._stream), "experts: sum")
         return out

@@ -23,8 +23,11 @@ class Kernels(Protocol):
     def queued_to_device(self, tensor: torch.Tensor) -> torch.Tensor:
         """As `to_device`, for small per-step inputs: the host does not wait for work queued before."""
 
-    def embedding(self, table: torch.Tensor, token_ids: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
-        """float32 rows [T, hidden] of `table` at `token_ids`, times `scale`."""
+    def embedding(
+        self, table: torch.Tensor, token_ids: torch.Tensor, scale: float = 1.0, positions: torch.Tensor | None = None,
+        position_table: torch.Tensor | None = None,
+    ) -> torch.Tensor:
+        """float32 rows [T, hidden] of `table` at `token_ids`, times `scale` (plus the rows of `position_table` at `positions`)."""
 
     def add_rms_norm(
         self, hidden: torch.Tensor, delta: torch.Tensor | None, weight: torch.Tensor, eps: float
@@ -66,10 +69,14 @@ class Kernels(Protocol):
     def paged_attention(
         self, qkv: torch.Tensor, layout: Any, batch: Any, cell: Any, scale: float, window: int | None, *,
         score_slopes: torch.Tensor | None = None, soft_cap: float | None = None, sinks: torch.Tensor | None = None,
-        keep_first: int = 0, chunk: int | None = None, out: torch.Tensor | None = None,
+        keep_first: int = 0, chunk: int | None = None, out: torch.Tensor | None = None, vdim: int | None = None,
+        distance_bias: Any = None, gates: tuple[torch.Tensor, int] | None = None,
     ) -> torch.Tensor:
         """Attention of the q heads of `qkv` over the cell's pages -> [T, heads * head_dim], or the first columns of `out`'s
-        rows.  With `chunk` (and no window) a query at p sees the keys at k <= p with k // chunk == p // chunk.
+        rows.  With `vdim` a head's result is its first so many columns alone, [T, heads * vdim].  With `distance_bias` (what
+        `prepare_distance_bias` returned) a score has its head's bias of the distance p - k added.  With `gates` = (rows in
+        the run dtype, first column) the result is multiplied element by element with the sigmoid of those rows' columns from
+        there on.  (The three not together with slopes, caps, sinks, kept first keys and chunks.)  With `chunk` (and no window) a query at p sees the keys at k <= p with k // chunk == p // chunk.
         Before the softmax a score s of a query at position p for a key at position k may be changed,
         for encodings and models that want it (Qwen2 wants neither): with `soft_cap`, to
         soft_cap * tanh(s / soft_cap); with `score_slopes` (float32, one per query head), by
@@ -77,6 +84,33 @@ class Kernels(Protocol):
         has exp(sink) more, once, with no value to it.  With `keep_first` (and a window) a query at p sees the keys at
         k <= p with p - k < window or k < keep_first: a sequence's first keys stay visible, at their own positions (the
         cell's need says the same, so their pages are never given back).  A library refuses what it cannot compute."""
+
+    def prepare_distance_bias(self, by_distance: torch.Tensor) -> Any:
+        """float32 [heads, reach], a head's bias at every distance (the last one for all distances from there on), in
+        whatever layout `paged_attention` wants."""
+
+    def convolved_heads(
+        self, x: torch.Tensor, q_first: int, k_first: int, v_first: int, heads: int, kv_heads: int, dim: int, vdim: int, width: int,
+        batch: Any, cell: Any = None, *, maps: int = 1, taps: torch.Tensor | None = None, window: torch.Tensor | None = None,
+        norm: bool = True, q_weight: torch.Tensor | None = None, k_weight: torch.Tensor | None = None, eps: float = 0.0,
+        temperature: tuple[float, int] | None = None,
+    ) -> torch.Tensor:
+        """From rows that hold `heads` queries and `kv_heads` keys of `maps` * `dim` and `kv_heads` values of `vdim` (from the
+        columns q_first, k_first, v_first): rows [T, (heads + 2 kv_heads) * width] of queries, keys and values of `width`; map
+        m of a query or key lies at m * (width / maps), zeros beyond its own size.  With `taps` (float32 [channels, width of
+        the convolution], the last column the current token's; q, k and v are then x's first columns, side by side) every
+        channel goes through a causal convolution over its request's tokens first; `window` float32 [slots, taps - 1,
+        channels] holds each request's last inputs (zeros at its start) and is moved on.  With `norm` every map of every
+        query and key is divided by its root mean square, times `q_weight` / `k_weight` ([dim], None: no weight).  With
+        `temperature` = (coef, every) a query at p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1).  All of it
+        float32, rounded once.  With a writable `cell` the keys and values are also stored in the cell's pages."""
+
+    def difference_attention(
+        self, rows: torch.Tensor, layout: Any, batch: Any, cell: Any, scale: float, vdim: int, factor: float, eps: float, out_scale: float,
+    ) -> torch.Tensor:
+        """Queries and keys are two maps side by side, each half of `layout.head_dim`.  Per head, a1 and a2 the softmax over
+        the cell's keys of (q_m . k_m) * scale of the two maps, applied to the values' first `vdim` columns: d = a1 - factor *
+        a2, and d * rsqrt(mean(d^2) + eps) * out_scale -> [T, heads * vdim] in the run dtype."""
 
     def rotate_store_attend(
         self, qkv: torch.Tensor, layout: Any, batch: Any, cell: Any,
@@ -249,7 +283,7 @@ class Kernels(Protocol):
         gates: torch.Tensor | None = None, gate_column: int = 0,
     ) -> torch.Tensor:
         """sum over a token's chosen experts of weight * down_e(act(up_e x)) (+ sigmoid(gates[:, gate_column]) * shared, or
-        + shared where no gates are given), float32 [T, hidden]; the inner rows are rounded to the run dtype between the
+        + shared where no gates are given), float32 [T, hidden]; `shared` may be partial sums [parts, T, hidden]; the inner rows are rounded to the run dtype between the
         two products."""
 
     # ------------------------------------------------------------------ copies of the stream, a diagonal recurrence, weighted sums

@@ -1,3 +1,3 @@
-from . import dafutar, dolezen, katenex, qwen2, sozavik, vagozen  # register Dafutar, Dolezen, Katenex, Qwen2ForCausalLM, Sozavik and Vagozen
+from . import dafutar, dolezen, dubesun, katenex, qwen2, sozavik, vagozen  # register Dafutar, Dolezen, Dubesun, Katenex, Qwen2ForCausalLM, Sozavik and Vagozen
 
-__all__ = ["dafutar", "dolezen", "katenex", "qwen2", "sozavik", "vagozen"]
+__all__ = ["dafutar", "dolezen", "dubesun", "katenex", "qwen2", "sozavik", "vagozen"]

@@ -17,7 +17,7 @@ from .base import (
     TensorSpec,
 )
 from .norm import LayerNorm, LayerNormSpec, RMSNorm, RMSNormSpec
-from .position import HeadLayout, LinearScaling, NoPositionSpec, PositionEncoding, Rotary, RotarySpec, WavelengthScaling, YarnScaling, rotary_frequencies
+from .position import DistanceBuckets, HeadLayout, LinearScaling, NoPositionSpec, PositionEncoding, Rotary, RotarySpec, WavelengthScaling, YarnScaling, rotary_frequencies
 from .attention import Attention, AttentionSpec, Mixer
 from .feed_forward import DenseMLP, DenseMLPSpec, FeedForward, GatedMLP, GatedMLPSpec
 from .block import Block, OutputNormBlock, OutputNormBlockSpec, ParallelBlock, ParallelBlockSpec, PendingNormed, PreNormBlock, PreNormBlockSpec, SandwichBlock, SandwichBlockSpec
@@ -26,6 +26,7 @@ from .latent_attention import LatentAttention, LatentAttentionSpec
 from .delta import GatedDelta, GatedDeltaSpec
 from .experts import RoutedExperts, RoutedExpertsSpec
 from .normed_attention import NormedAttention, NormedAttentionSpec
+from .difference_attention import DifferenceAttention, DifferenceAttentionSpec
 from .decay_attention import DecayAttention, DecayAttentionSpec
 from .hyper import HyperBlock, HyperBlockSpec, PendingWrite, StreamCopies, StreamCopiesSpec, StreamNorm, StreamNormSpec
 from .recurrent import GatedRecurrence, GatedRecurrenceSpec

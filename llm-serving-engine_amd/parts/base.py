@@ -99,6 +99,17 @@ class SlotNeed(CacheNeed):
     shape: tuple[int, ...] = ()
 
 
+def needs_by_name(need: "CacheNeed | dict[str, CacheNeed] | None") -> "dict[str | None, CacheNeed]":
+    """A run's needs by name: none, one (under None), or the several its block named."""
+    if need is None:
+        return {}
+    if isinstance(need, dict):
+        if any(not isinstance(name, str) for name in need):
+            raise TypeError("several cache needs are named by strings")
+        return {name: value for name, value in need.items() if value is not None}
+    return {None: need}
+
+
 @dataclass(frozen=True)
 class PagedKeyValue(PagedNeed):
     """Cache need of a mixer that keeps a key and a value per token in pages.  Keys lie in pieces of

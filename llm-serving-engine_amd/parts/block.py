@@ -248,8 +248,8 @@ class ParallelBlock(Block):
     """Where mixer and feed-forward both begin and end with a product (`joins`), the two first products are one over the
     weights side by side, and the two last ones are one over the operands side by side, W_o m + W_d a = [W_o | W_d] [m; a]:
     the sum of the sublayers is made in the product's float32 accumulators, and a layer is two launches of products
-    instead of four and no add.  Else (or where the operands side by side make rows of no multiple of eight) the results
-    are added by a kernel."""
+    instead of four and no add.  Else (or where the operands side by side make rows of no multiple of eight) a
+    feed-forward whose last kernel can take the mixer's result along (`adds_beside`) does so, or a kernel adds the two."""
 
     @classmethod
     def _members(cls, spec: ParallelBlockSpec):
@@ -308,4 +308,6 @@ class ParallelBlock(Block):
         mixed = self.mixer.forward(normed, batch, cell)
         if self.feed_forward is None:
             return mixed
+        if getattr(self.feed_forward, "adds_beside", False):
+            return self.feed_forward.forward(normed, batch, beside=mixed)
         return kernels.add_scaled(mixed, 1.0, self.feed_forward.forward(normed, batch), 1.0)

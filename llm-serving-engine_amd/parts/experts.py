@@ -92,6 +92,7 @@ class RoutedExperts(FeedForward):
             gates=[tensors[f"e{index}.gate"] for index in range(spec.num_experts)] if spec.gated else None,
             **({"limit": spec.limit} if spec.limit is not None else {}),
         )
+        self.adds_beside = not shared  # the kernel that adds a token's experts up takes another result along
         self.shared_up = self.shared_down = None
         if shared:
             if spec.gated:
@@ -100,7 +101,8 @@ class RoutedExperts(FeedForward):
                 self.shared_up = kernels.prepare_linear([tensors["shared.up"]], None)
             self.shared_down = kernels.prepare_linear([tensors["shared.down"]], None)
 
-    def forward(self, x: torch.Tensor, batch) -> torch.Tensor:
+    def forward(self, x: torch.Tensor, batch, beside: torch.Tensor | None = None) -> torch.Tensor:
+        """With `beside` (float32 rows, or partial sums of them; for a feed-forward with `adds_beside`): plus those rows."""
         kernels, spec = self.kernels, self.spec
         scores = kernels.linear(x, self.router, out_dtype=torch.float32)  # [T, experts (+ 1)]
         chosen, weights = kernels.route(
@@ -108,7 +110,9 @@ class RoutedExperts(FeedForward):
             groups=spec.groups, keep_groups=spec.keep_groups, renormalise=spec.renormalise,
         )
         if self.shared_up is None:
-            return kernels.expert_feed_forward(x, self.experts, chosen, weights)  # float32 [T, hidden]
+            return kernels.expert_feed_forward(x, self.experts, chosen, weights, shared=beside)  # float32 [T, hidden]
+        if beside is not None:
+            raise ValueError("routed experts: rows beside them are added where there is no shared expert")
         if spec.gated:
             inner = kernels.gated_linear(x, self.shared_up)
         else:

@@ -8,7 +8,7 @@ from typing import Any
 
 import torch
 
-from .base import BLOCKS, LOGIT_PARTS, NORMS, PASS_PARTS, STREAM_PARTS, CacheNeed, PagedNeed, TensorSpec, prefixed, under
+from .base import BLOCKS, LOGIT_PARTS, NORMS, PASS_PARTS, STREAM_PARTS, CacheNeed, PagedNeed, TensorSpec, needs_by_name, prefixed, under
 
 
 @dataclass(frozen=True)
@@ -23,13 +23,19 @@ class LayerRun:
     may be named by several entries (its tensors are shared, each run has a
     cache cell of its own).  With `reads` set, the run uses the cell of that
     earlier entry of the run order instead, and stores nothing (the cell keeps entries as long as the run that
-    fills it or one that reads it asks: they may look back differently far).  With `enters` set, the run is
-    the first of a pass (its number: 0, 1, ...) through layers that the model walks several times, and
+    fills it or one that reads it asks: they may look back differently far).  A run whose block named several needs may
+    read only those named in `reads_only` from there (None: all of them), and keeps the others itself.  With `enters` set,
+    the run is the first of a pass (its number: 0, 1, ...) through layers that the model walks several times, and
     the model's `pass_entry` part acts on the stream before it."""
 
     layer: int
     reads: int | None = None
     enters: int | None = None
+    reads_only: tuple[str, ...] | None = None
+
+    def takes(self, name: str | None) -> bool:
+        """Whether what the run needs under `name` is read from the cell of the run that `reads` names."""
+        return self.reads is not None and (self.reads_only is None or name in self.reads_only)
 
 
 @dataclass(frozen=True)
@@ -59,15 +65,22 @@ class ModelSpec:
     pass_entry: NamedPart | None = None
     # the embedded rows are the table's times this
     embedding_scale: float = 1.0
+    # a table [max_positions, hidden] of learned vectors, one a position, added to the embedded rows (behind their scale)
+    position_name: str | None = None
+    max_positions: int | None = None
     # tensors that a model folder may hold and the model does not use
     ignored_tensors: tuple[str, ...] = ()
 
     def __post_init__(self) -> None:
+        if (self.position_name is None) != (self.max_positions is None):
+            raise ValueError("a table of positions has a name and a length")
         if self.pass_entry is None and any(run.enters is not None for run in self.run_order):
             raise ValueError("a run begins a pass, and the model has no part for that")
         for index, run in enumerate(self.run_order):
             if not 0 <= run.layer < len(self.layers):
                 raise ValueError(f"run {index} names layer {run.layer}, which does not exist")
+            if run.reads is None and run.reads_only is not None:
+                raise ValueError(f"run {index} names what it reads of another's cell, and reads none")
             if run.reads is not None:
                 if not 0 <= run.reads < index:
                     raise ValueError(f"run {index} reads the cache of run {run.reads}, which is not earlier")
@@ -75,23 +88,38 @@ class ModelSpec:
                     raise ValueError(f"run {index} reads run {run.reads}, which owns no cache")
                 self.cell_need(index)  # (refuses runs that cannot share a cell)
 
+    def _own_need(self, run_index: int) -> "CacheNeed | dict[str, CacheNeed] | None":
+        return BLOCKS.cache_need(self.layers[self.run_order[run_index].layer].block)
+
     def cell_need(self, run_index: int) -> "CacheNeed | dict[str, CacheNeed] | None":
-        """What the run's cell has to be: what the run itself needs, joined with what the runs that read its cell need."""
-        owner = self.run_order[run_index].reads
-        owner = run_index if owner is None else owner
-        need = BLOCKS.cache_need(self.layers[self.run_order[owner].layer].block)
-        for index, run in enumerate(self.run_order):
-            if run.reads == owner:
-                other = BLOCKS.cache_need(self.layers[run.layer].block)
-                joined = need.shared_with(other) if isinstance(need, PagedNeed) else need if other == need else None
-                if joined is None and other != need:
-                    raise ValueError(f"run {index} and run {owner} need different caches")
-                need = joined
-        return need
+        """What the run's cell has to be: what the run itself needs, joined with what the runs that read its cell need; for
+        what the run reads from another's cell, what that one has to be."""
+        own = self._own_need(run_index)
+        found: dict[str | None, CacheNeed] = {}
+        for name, need in needs_by_name(own).items():
+            run = self.run_order[run_index]
+            owner = run.reads if run.takes(name) else run_index
+            owned = needs_by_name(self._own_need(owner))
+            if name not in owned:
+                raise ValueError(f"run {run_index} and run {owner} need different caches")
+            need = owned[name]
+            for index, other_run in enumerate(self.run_order):
+                if other_run.reads == owner and other_run.takes(name):
+                    other = needs_by_name(self._own_need(index)).get(name)
+                    joined = need.shared_with(other) if isinstance(need, PagedNeed) else need if other == need else None
+                    if joined is None:
+                        raise ValueError(f"run {index} and run {owner} need different caches")
+                    need = joined
+            found[name] = need
+        if isinstance(own, dict):
+            return found
+        return found.get(None)
 
     def tensors(self) -> dict[str, TensorSpec]:
         """Every tensor of the model by its name in the model folder."""
         found = {self.embedding_name: TensorSpec((self.vocab_size, self.hidden_size), role="embedding")}
+        if self.position_name is not None:
+            found[self.position_name] = TensorSpec((self.max_positions, self.hidden_size), role="embedding")
         for layer in self.layers:
             found.update(prefixed(BLOCKS.tensors(layer.block), layer.prefix))
         found.update(prefixed(NORMS.tensors(self.final_norm), self.final_norm_name))
@@ -116,6 +144,7 @@ class DecoderModel:
         self.kernels = kernels
         self.embedding = tensors[spec.embedding_name]
         self._embedding_scale = (float(spec.embedding_scale),) if spec.embedding_scale != 1.0 else ()
+        self.position_table = tensors[spec.position_name] if spec.position_name is not None else None
         self.layers = [
             BLOCKS.build(layer.block, under(tensors, layer.prefix), kernels) for layer in spec.layers
         ]
@@ -136,7 +165,8 @@ class DecoderModel:
         self.observer = None
 
     def _run_layers(self, batch, cells: list):
-        hidden = self.kernels.embedding(self.embedding, batch.token_ids, *self._embedding_scale)
+        placed = {} if self.position_table is None else {"positions": batch.positions, "position_table": self.position_table}
+        hidden = self.kernels.embedding(self.embedding, batch.token_ids, *self._embedding_scale, **placed)
         for part in self.input_parts:  # (in place, or a new stream of another shape: copies side by side)
             changed = part.forward(hidden, batch)
             hidden = hidden if changed is None else changed

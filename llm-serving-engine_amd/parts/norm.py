@@ -13,13 +13,15 @@ from .base import NORMS, Part, TensorSpec
 class RMSNormSpec:
     """`weight_name` is the tensor's name below the part's prefix (a model whose files call it otherwise says so).
     `weight_scale` multiplies the weight (float32) when the part is built: a constant that a model puts on the normed
-    rows (a scale of the logits behind the last norm) costs nothing that way."""
+    rows (a scale of the logits behind the last norm) costs nothing that way.  `weight_offset` is added to it first
+    (float32): 1 for a model whose files keep the weight's difference from one."""
 
     size: int
     eps: float
     weight_name: str = "weight"
     kind: str = "rmsnorm"
     weight_scale: float = 1.0
+    weight_offset: float = 0.0
 
 
 @NORMS.register("rmsnorm")
@@ -30,13 +32,13 @@ class RMSNorm(Part):
 
     @classmethod
     def tensors(cls, spec: RMSNormSpec) -> dict[str, TensorSpec]:
-        return {spec.weight_name: TensorSpec((spec.size,), role="norm")}
+        return {spec.weight_name: TensorSpec((spec.size,), role="norm" if spec.weight_offset == 0.0 else "bias")}
 
     def __init__(self, spec: RMSNormSpec, tensors, kernels) -> None:
         super().__init__(spec, tensors, kernels)
         self.weight = tensors[spec.weight_name]
-        if spec.weight_scale != 1.0:
-            self.weight = (self.weight.float() * float(spec.weight_scale)).contiguous()
+        if spec.weight_scale != 1.0 or spec.weight_offset != 0.0:
+            self.weight = ((self.weight.float() + float(spec.weight_offset)) * float(spec.weight_scale)).contiguous()
 
     def forward(self, hidden: torch.Tensor, delta: torch.Tensor | None) -> torch.Tensor:
         """Adds `delta` into `hidden` (in place) and returns the normed rows in the run dtype."""

@@ -3,7 +3,10 @@
 from __future__ import annotations
 
 import math
+from bisect import bisect_right
 from dataclasses import dataclass
+from fractions import Fraction
+from functools import cached_property
 
 import torch
 
@@ -158,3 +161,50 @@ def rotary_frequencies(dims: int, theta: float, scaling: "YarnScaling | Waveleng
     ramp = ((index - low) / max(high - low, 0.001)).clamp(0.0, 1.0)
     stretched = plain / scaling.factor * ramp + plain * (1.0 - ramp)
     return stretched.to(torch.float32), 0.1 * math.log(scaling.factor) + 1.0
+
+
+@dataclass(frozen=True)
+class DistanceBuckets:
+    """Distances between a query and a key, sorted into `buckets`: with half = buckets // 2, a distance n below half is a
+    bucket of its own, and from there on bucket half + floor(ln(n / half) / ln(furthest / half) * (buckets - half)), at
+    most the last one."""
+
+    buckets: int
+    furthest: float
+
+    def __post_init__(self) -> None:
+        if self.buckets < 2 or not self.furthest > self.buckets // 2:
+            raise ValueError("distance buckets: two or more, and a furthest distance beyond the buckets of one distance each")
+
+    def of(self, distance: int) -> int:
+        """The bucket, in exact arithmetic: ln(n / half) / ln(furthest / half) * later >= k is n^later half^k >= furthest^k
+        half^later, a comparison of rationals (a logarithm rounded the wrong way would move a bucket's first distance)."""
+        half = self.buckets // 2
+        if distance < half:
+            return distance
+        later = self.buckets - half
+        return half + bisect_right(self._edges, Fraction(distance, half) ** later, 0, later - 1)
+
+    @cached_property
+    def _edges(self) -> list[Fraction]:
+        """(furthest / half)^k for k = 1, 2, ..., where the later buckets begin."""
+        step, edges = Fraction(self.furthest) / (self.buckets // 2), []
+        for _ in range(self.buckets - self.buckets // 2):
+            edges.append(edges[-1] * step if edges else step)
+        return edges
+
+    @property
+    def reach(self) -> int:
+        """Distances from `reach - 1` on all lie in the last bucket."""
+        low, high = 0, max(1, math.ceil(self.furthest))
+        while low < high:
+            middle = (low + high) // 2
+            if self.of(middle) >= self.buckets - 1:
+                high = middle
+            else:
+                low = middle + 1
+        return low + 1
+
+    def by_distance(self) -> torch.Tensor:
+        """int64 [reach]: the bucket of every distance below `reach`."""
+        return torch.tensor([self.of(distance) for distance in range(self.reach)], dtype=torch.int64)

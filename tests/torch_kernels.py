@@ -46,8 +46,9 @@ class TorchKernels:
     def queued_to_device(self, tensor):
         return tensor
 
-    def embedding(self, table, token_ids, scale=1.0):
-        return table[token_ids.long()].float() * scale
+    def embedding(self, table, token_ids, scale=1.0, positions=None, position_table=None):
+        rows = table[token_ids.long()].float() * scale
+        return rows if positions is None else rows + position_table[positions.long()].float()
 
     def add_rms_norm(self, hidden, delta, weight, eps):
         if delta is not None:
@@ -109,7 +110,7 @@ class TorchKernels:
             cell.put_value_rows(pages, offsets, view[:, heads + kv_heads :])  # pages are [kv, offset / v, dim, v]
 
     def paged_attention(self, qkv, layout, batch, cell, scale, window, *, score_slopes=None, soft_cap=None, sinks=None, keep_first=0,
-                        chunk=None, out=None):
+                        chunk=None, out=None, vdim=None, distance_bias=None, gates=None):
         tokens = qkv.shape[0]
         heads, kv_heads, dim = layout.num_heads, layout.num_kv_heads, layout.head_dim
         assert qkv.shape[1] == layout.stride
@@ -135,17 +136,71 @@ class TorchKernels:
                     scores = soft_cap * torch.tanh(scores / soft_cap)
                 if score_slopes is not None:
                     scores = scores - score_slopes.float().view(-1, 1) * (position - where).float()
+                if distance_bias is not None:
+                    scores = scores + distance_bias[:, (position - where).clamp(max=distance_bias.shape[1] - 1)]
                 if sinks is not None:  # a column more in the softmax, with no value
                     scores = torch.cat([scores, sinks.float().view(-1, 1)], dim=1)
                     out[row] = torch.einsum("hn,nhd->hd", torch.softmax(scores, dim=-1)[:, :-1], values)
                 else:
                     out[row] = torch.einsum("hn,nhd->hd", torch.softmax(scores, dim=-1), values)
                 row += 1
-        result = out.reshape(tokens, heads * dim).to(self.dtype)
+        wide = heads * (vdim or dim)
+        result = out[:, :, : vdim or dim].reshape(tokens, wide)
+        if gates is not None:
+            rows, first = gates
+            result = result * torch.sigmoid(rows[:, first : first + wide].float())
+        result = result.to(self.dtype)
         if given is None:
             return result
-        given[:, : heads * dim] = result
+        given[:, :wide] = result
         return given
+
+    def prepare_distance_bias(self, by_distance):
+        return by_distance.float()
+
+    def convolved_heads(self, x, q_first, k_first, v_first, heads, kv_heads, dim, vdim, width, batch, cell=None, *, maps=1, taps=None,
+                        window=None, norm=True, q_weight=None, k_weight=None, eps=0.0, temperature=None):
+        tokens, part = x.shape[0], width // maps
+        if taps is not None:
+            own = self.dtype
+            self.dtype = torch.float32  # (what lies between the convolution and the norm is not rounded)
+            x = self.causal_conv(x, taps.shape[0], taps, "none", batch, window)
+            self.dtype = own
+        out = torch.zeros((tokens, heads + 2 * kv_heads, width))
+        for first, count, weight, at in ((q_first, heads, q_weight, 0), (k_first, kv_heads, k_weight, heads)):
+            rows = x[:, first : first + count * maps * dim].float().reshape(tokens, count, maps, dim)
+            if norm:
+                rows = rows * torch.rsqrt(rows.pow(2).mean(-1, keepdim=True) + eps)
+                rows = rows * weight.float() if weight is not None else rows
+            if temperature is not None and at == 0:
+                coef, every = temperature
+                grown = 1.0 + coef * torch.log(torch.div(batch.positions + 1, every, rounding_mode="floor").float() + 1.0)
+                rows = rows * grown.view(tokens, 1, 1, 1)
+            for m in range(maps):
+                out[:, at : at + count, m * part : m * part + dim] = rows[:, :, m]
+        out[:, heads + kv_heads :, :vdim] = x[:, v_first : v_first + kv_heads * vdim].float().reshape(tokens, kv_heads, vdim)
+        out = out.reshape(tokens, -1).to(self.dtype)
+        if cell is not None and cell.writable:
+            from llmserve_amd.parts import HeadLayout
+
+            self.rotate_and_store(out, HeadLayout(heads, kv_heads, width), batch, cell, None, "none")
+        return out
+
+    def difference_attention(self, rows, layout, batch, cell, scale, vdim, factor, eps, out_scale):
+        from llmserve_amd.parts import HeadLayout
+
+        tokens, heads, width = rows.shape[0], layout.num_heads, layout.head_dim
+        own, maps = self.dtype, []
+        for m in range(2):  # the queries of one map, zeros in place of the other's
+            queries = torch.zeros((tokens, heads, width))
+            half = slice(m * width // 2, (m + 1) * width // 2)
+            queries[:, :, half] = rows[:, : heads * width].float().view(tokens, heads, width)[:, :, half]
+            self.dtype = torch.float32
+            alone = HeadLayout(heads, layout.num_kv_heads, width, heads * width)
+            maps.append(self.paged_attention(queries.view(tokens, -1), alone, batch, cell, scale, None, vdim=vdim).view(tokens, heads, vdim))
+            self.dtype = own
+        d = maps[0] - factor * maps[1]
+        return (d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + eps) * out_scale).reshape(tokens, heads * vdim).to(self.dtype)
 
     def rotate_store_attend(self, qkv, layout, batch, cell, inverse_frequencies, pairing, scale, window, project=None, *, sinks=None, chunk=None,
                             out=None):
@@ -463,6 +518,7 @@ class TorchKernels:
         for slot in range(chosen.shape[1]):
             out += weights[:, slot : slot + 1] * rows[:, slot]
         if shared is not None:
+            shared = shared if shared.ndim == 2 else shared.sum(0)
             out += torch.sigmoid(gates[:, gate_column : gate_column + 1].float()) * shared if gates is not None else shared
         return out
 
