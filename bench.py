@@ -48,6 +48,11 @@ decaying state, norms behind the sublayers), the Dafutar models (latent attentio
 
 measures the sixth (configs/dolezen-w1536.json, configs/dolezen-w3584.json) beside the Sozavik models (window attention with
 a sink), the Vagozen models (latent attention) and the Qwen2 models.
+
+    python bench.py --op dubesun
+
+measures the seventh (configs/dubesun-w1536.json, configs/dubesun-w3584.json) beside the Dolezen models (one norm for two
+sublayers, queries over another layer's keys), the Vagozen models (gated experts with a limit) and the Qwen2 models.
 """
 
 from __future__ import annotations
@@ -89,7 +94,7 @@ def parse() -> argparse.Namespace:
                         help="leave out decoding at contexts of 8k and 30k (batch 8) and 4k (batch 64), and the long prompts")
     parser.add_argument("--skip-other-models", action="store_true",
                         help="leave out the float32 run and the 7B and 32B layer sizes")
-    parser.add_argument("--op", choices=("decode-attention", "prefill-attention", "dafutar", "sozavik", "katenex", "vagozen", "dolezen"), default=None,
+    parser.add_argument("--op", choices=("decode-attention", "prefill-attention", "dafutar", "sozavik", "katenex", "vagozen", "dolezen", "dubesun"), default=None,
                         help="measure one operation alone instead, as the reference's kernel benchmark does")
     return parser.parse_args()
 
@@ -146,6 +151,10 @@ class Bench:
             table = self.tensors[self.spec.embedding_name]
             self.weight_bytes -= table.numel() * table.element_size()
             self.embedding_row_bytes = self.spec.hidden_size * table.element_size()
+        if self.spec.position_name is not None:  # (of a table of positions too only the tokens' rows)
+            table = self.tensors[self.spec.position_name]
+            self.weight_bytes -= table.numel() * table.element_size()
+            self.embedding_row_bytes += self.spec.hidden_size * table.element_size()
         self.kv_bytes_per_token = self.runner.cache.bytes_per_token
         self.generator = torch.Generator().manual_seed(seed)
         self.serial = 0
@@ -448,6 +457,8 @@ def main() -> int:
         return vagozen_table(args)
     if args.op == "dolezen":
         return dolezen_table(args)
+    if args.op == "dubesun":
+        return dubesun_table(args)
 
     import torch
 
@@ -612,6 +623,14 @@ def dolezen_table(args) -> int:
     beside the Sozavik, the Vagozen and the Qwen2 of the same width, number of layer runs and vocabulary, measured as
     `dafutar_table` measures."""
     return beside_qwen2(args, "dolezen", "Dolezen", also=("sozavik", "vagozen"))
+
+
+def dubesun_table(args) -> int:
+    """The Dubesun decoder (one norm for mixer and experts; layers of differential attention behind short convolutions, half of
+    them over an earlier layer's keys and values, and of attention with a learned bias by distance whose values are its keys) at
+    two layer sizes beside the Dolezen, the Vagozen and the Qwen2 of the same width, number of layer runs and vocabulary,
+    measured as `dafutar_table` measures."""
+    return beside_qwen2(args, "dubesun", "Dubesun", also=("dolezen", "vagozen"))
 
 
 def beside_qwen2(args, name: str, title: str, also: tuple[str, ...] = ()) -> int:
