@@ -32,7 +32,8 @@
 // their results finished, heads of `vdim` side by side: CHANGED_BIAS adds a learned bias by distance to the scores and may
 // multiply the results with a gate an element; CHANGED_MAPS is differential attention: a query and a key are two maps side by
 // side, a wave's two column tiles are the two maps of the same columns, each multiplied with its own half of the keys, and the
-// difference of the two results is normed before it is written.
+// difference of the two results is normed before it is written.  In a step of single tokens whose maps fit one column tile (up to
+// eight query heads a kv head) both maps are columns of that tile (COLUMN_TILES 1: `heads` counts maps), each with zeros in the other half.
 #include "common.h"
 
 #ifndef HEAD_DIM
@@ -209,7 +210,7 @@ __device__ __forceinline__ void scores_of(const Columns<COLUMN_TILES>& columns, 
     s_hi[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int s = 0; s < QK_STEPS; ++s) {
-      if (CHANGED == CHANGED_MAPS && (t == 0 ? s * STEP_WIDTH >= D / 2 : (s + 1) * STEP_WIDTH <= D / 2)) continue;
+      if (CHANGED == CHANGED_MAPS && COLUMN_TILES == 2 && (t == 0 ? s * STEP_WIDTH >= D / 2 : (s + 1) * STEP_WIDTH <= D / 2)) continue;
       s_lo[t] = mfma_qk(L.k_lo[s], columns.query[t][s], s_lo[t]);
       s_hi[t] = mfma_qk(L.k_hi[s], columns.query[t][s], s_hi[t]);
     }
@@ -323,7 +324,8 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
     const int* __restrict__ positions, const int* __restrict__ work, int heads, int kv_heads, int tokens_per_tile,
     int page_size, int page_shift, float scale, int window, int splits, FusedDecode fused, ScoreChange change, Finish finish) {
   static_assert(!FUSED || CHANGED == CHANGED_NOT || CHANGED == CHANGED_EDGES, "the fused decode form leaves the scores as they are");
-  static_assert(CHANGED != CHANGED_MAPS || COLUMN_TILES == 2, "a column tile a map");
+  constexpr bool PAIRED = CHANGED == CHANGED_MAPS && COLUMN_TILES == 1;  // a head's two maps are neighbouring columns
+  constexpr bool TILE_A_MAP = CHANGED == CHANGED_MAPS && COLUMN_TILES == 2;
   extern __shared__ float lds[];  // [WAVES][16 columns][D + 4]
   if (FUSED)  // a short kernel: fetch all arguments in one go rather than each before its first use
     asm volatile("" ::"s"(row_width), "s"(table_width), "s"(heads), "s"(kv_heads), "s"(page_size), "s"(page_shift),
@@ -357,7 +359,7 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
   [[maybe_unused]] int early_k = -1, early_k_hi = -1, early_v = -1;
   const bool early_pages = FUSED && splits == 1 && (wave * KEYS + KEYS - 1) / page_size < table_width;
   // (heads up to 128 wide leave the registers for a wave's second step to be asked for together with its first)
-  constexpr bool TWO_STEPS = FUSED && HEAD_DIM <= 128;
+  constexpr bool TWO_STEPS = (FUSED || (WAVES > 4 && COLUMN_TILES == 1 && CHANGED >= CHANGED_BIAS)) && HEAD_DIM <= 128;
   [[maybe_unused]] int second_k = -1, second_k_hi = -1, second_v = -1;
   const bool second_pages = TWO_STEPS && early_pages && ((wave + WAVES) * KEYS + KEYS - 1) / page_size < table_width;
   if (FUSED) {
@@ -411,13 +413,13 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
 #pragma unroll
   for (int t = 0; t < COLUMN_TILES; ++t) {
     int token, head_here;
-    map.of(CHANGED == CHANGED_MAPS ? 0 : t, c, token, head_here, column_live[t]);
+    map.of(TILE_A_MAP ? 0 : t, c, token, head_here, column_live[t]);
     const int safe = min(token, tokens - 1);
     const int head = kv_head * group + head_tile * 16 + head_here;
     column_position[t] = column_live[t] ? position0 + safe : -1;
     column_first[t] = first_seen_from(max(column_position[t], 0));
     if constexpr (CHANGED == CHANGED_SCORES) columns.slope[t] = change.slopes ? change.slopes[head] * 1.44269504088896f : 0.f;
-    const bf16_t* q_row = qkv + (size_t)(row0 + safe) * row_width + (size_t)head * D;
+    const bf16_t* q_row = qkv + (size_t)(row0 + safe) * row_width + (size_t)(PAIRED ? head / 2 : head) * D;
 #pragma unroll
     for (int s = 0; s < QK_STEPS; ++s) query[t][s] = load_qk(q_row, KEY_PIECE, s, q);  // a query's row is in one piece
     if constexpr (CHANGED == CHANGED_BIAS) {
@@ -425,7 +427,12 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
       columns.slope[t] = column_bias[t][0];  // of every distance beyond the table's reach
     }
 #if HEAD_DIM % 32 == 0
-    if constexpr (CHANGED == CHANGED_MAPS && D / 2 % 32 != 0) {  // the step that straddles the middle: zeros in the other map's half
+    if constexpr (PAIRED) {
+#pragma unroll
+      for (int s = 0; s < QK_STEPS; ++s)
+        if ((32 * s + 8 * q >= D / 2) != (head % 2 == 1)) query[t][s].v = (bf16x8){};
+    }
+    if constexpr (TILE_A_MAP && D / 2 % 32 != 0) {  // the step that straddles the middle: zeros in the other map's half
       constexpr int middle = D / 2 / 32;
       if ((q >= 2) != (t == 1)) query[t][middle].v = (bf16x8){};
     }
@@ -594,6 +601,27 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
     for (int d = 0; d < D_TILES; ++d) L.v[d] = *(const bf16x8*)(base + (unsigned)(d * 16 + c) * VALUE_PIECE);
   };
 
+  // CHANGED_BIAS: the biases of a step's keys, by their distances, asked for ahead of the first product
+  auto fetch_bias = [&](int key0, float (*bias)[8]) {
+    if constexpr (CHANGED == CHANGED_BIAS) {
+      if (position0 - (key0 + KEYS - 1) >= change.reach - 1) {  // all of the step's keys lie beyond the table's reach
+#pragma unroll
+        for (int t = 0; t < COLUMN_TILES; ++t)
+#pragma unroll
+          for (int i = 0; i < 8; ++i) bias[t][i] = columns.slope[t];
+      } else {
+        typedef float f32x4_anywhere __attribute__((ext_vector_type(4), aligned(4)));
+#pragma unroll
+        for (int t = 0; t < COLUMN_TILES; ++t) {
+          const float* at = column_bias[t] + bias_element(column_position[t] - (key0 + 8 * q), change.reach);
+          const f32x4_anywhere lo = *(const f32x4_anywhere*)at, hi = *(const f32x4_anywhere*)(at + 4);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) bias[t][i] = i < 4 ? lo[i] : hi[i - 4];
+        }
+      }
+    }
+  };
+
   const float scale_log2 = scale * 1.44269504088896f;
   const int every_first = first_seen_from(last_key);  // every column sees the keys from here on (up to its own)
 
@@ -612,11 +640,13 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
       // own, and each of the two sets is filled again as soon as its step has been multiplied.
       auto multiply = [&](int step, StepLoads& L) {
         f32x4 s_lo[COLUMN_TILES], s_hi[COLUMN_TILES];
-        scores_of(columns, L, s_lo, s_hi);
         const int key0 = step * KEYS;
+        [[maybe_unused]] float bias[COLUMN_TILES][8];
+        fetch_bias(key0, bias);
+        scores_of(columns, L, s_lo, s_hi);
         const bool interior = key0 + KEYS - 1 <= position0 && key0 >= every_first;
-        weigh_and_add(columns, L, s_lo, s_hi, key0, q, interior, last_key,
-                      min(max(key0 + 8 * q, low_limit), high_limit), scale_log2);
+        weigh_and_add<COLUMN_TILES, CHANGED>(columns, L, s_lo, s_hi, key0, q, interior, last_key,
+                                             min(max(key0 + 8 * q, low_limit), high_limit), scale_log2, 0.f, 0, bias);
       };
       StepLoads ahead;
       const int step1 = step0 + WAVES;
@@ -652,23 +682,7 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
       f32x4 s_lo[COLUMN_TILES], s_hi[COLUMN_TILES];
       const int key0 = real_step(step) * KEYS;
       [[maybe_unused]] float bias[COLUMN_TILES][8];
-      if constexpr (CHANGED == CHANGED_BIAS) {
-        if (position0 - (key0 + KEYS - 1) >= change.reach - 1) {  // all of the step's keys lie beyond the table's reach
-#pragma unroll
-          for (int t = 0; t < COLUMN_TILES; ++t)
-#pragma unroll
-            for (int i = 0; i < 8; ++i) bias[t][i] = columns.slope[t];
-        } else {
-          typedef float f32x4_anywhere __attribute__((ext_vector_type(4), aligned(4)));
-#pragma unroll
-          for (int t = 0; t < COLUMN_TILES; ++t) {
-            const float* at = column_bias[t] + bias_element(column_position[t] - (key0 + 8 * q), change.reach);
-            const f32x4_anywhere lo = *(const f32x4_anywhere*)at, hi = *(const f32x4_anywhere*)(at + 4);
-#pragma unroll
-            for (int i = 0; i < 8; ++i) bias[t][i] = i < 4 ? lo[i] : hi[i - 4];
-          }
-        }
-      }
+      fetch_bias(key0, bias);
       scores_of<COLUMN_TILES, CHANGED>(columns, loads, s_lo, s_hi);
       if (more) fetch_keys(step + WAVES, pages, loads);
       const bool interior = key0 + KEYS - 1 <= position0 && key0 >= every_first;
@@ -685,8 +699,31 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
   // (a column's row is D sums, then its maximum and its sum of weights; rows 16 bytes apart in the banks, so that a
   // lane's four sums of a tile go and come as one 16-byte piece)
   constexpr int STRIDE = D + 4;
+  auto merge_waves = [&](int column, int d4, float& best, float& total) {
+    float2 theirs_ml[WAVES];
+    f32x4 theirs_acc[WAVES];
+#pragma unroll
+    for (int w = 0; w < WAVES; ++w) {
+      const float* theirs = lds + ((size_t)w * 16 + column) * STRIDE;
+      theirs_ml[w] = *(const float2*)(theirs + D);
+      theirs_acc[w] = *(const f32x4*)(theirs + d4);
+    }
+    best = -INFINITY;
+#pragma unroll
+    for (int w = 0; w < WAVES; ++w) best = fmaxf(best, theirs_ml[w].x);
+    total = 0.f;
+    f32x4 merged = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int w = 0; w < WAVES; ++w) {
+      const float factor = theirs_ml[w].x == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(theirs_ml[w].x - best);
+      total += theirs_ml[w].y * factor;
+      merged += theirs_acc[w] * factor;
+    }
+    return merged;
+  };
   // (CHANGED_MAPS: a thread's pieces of the first map's results stay here until it has the second's)
-  constexpr int HELD = CHANGED == CHANGED_MAPS ? (16 * (D / 4) + WAVES * 64 - 1) / (WAVES * 64) : 1;
+  constexpr int RESULTS = PAIRED ? 8 : 16;  // columns of the finished result a tile
+  constexpr int HELD = CHANGED == CHANGED_MAPS ? (RESULTS * (D / 4) + WAVES * 64 - 1) / (WAVES * 64) : 1;
   [[maybe_unused]] f32x4 held[HELD];
 #pragma unroll
   for (int t = 0; t < COLUMN_TILES; ++t) {
@@ -698,6 +735,30 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
     for (int d = 0; d < D_TILES; ++d) *(f32x4*)(mine + d * 16 + 4 * q) = acc[t][d];
     if (q == 0) *(float2*)(mine + D) = make_float2(running_max[t], sum);
     __syncthreads();
+    if constexpr (PAIRED) {  // one token: column 2 h and 2 h + 1 are the maps of its head h
+#pragma unroll
+      for (int turn = 0; turn < HELD; ++turn) {
+        const int index = threadIdx.x + turn * WAVES * 64;
+        const int pair = index / (D / 4), d4 = (index % (D / 4)) * 4;
+        if (2 * pair >= map.columns) continue;
+#pragma unroll
+        for (int m = 0; m < 2; ++m) {
+          float best, total;
+          const f32x4 merged = merge_waves(2 * pair + m, d4, best, total);
+          if (splits == 1) {
+            const float inverse = total > 0.f ? 1.f / total : 0.f;
+            if (m == 0) held[turn] = merged * inverse;
+            else held[turn] -= merged * (inverse * finish.factor);
+          } else {
+            const size_t slot = ((size_t)row0 * heads + kv_head * group + 2 * pair + m) * splits + blockIdx.z;
+            *(f32x4*)(partial_acc + slot * D + d4) = merged;
+            if (d4 == 0) *(float2*)(partial_ml + slot * 2) = make_float2(best, total);
+          }
+        }
+      }
+      __syncthreads();
+      continue;
+    }
 #pragma unroll
     for (int turn = 0; turn < (16 * (D / 4) + WAVES * 64 - 1) / (WAVES * 64); ++turn) {
       const int index = threadIdx.x + turn * WAVES * 64;
@@ -705,27 +766,10 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
       const int column = index / (D / 4), d4 = (index % (D / 4)) * 4;
       int token, head_here;
       bool live;
-      map.of(CHANGED == CHANGED_MAPS ? 0 : t, column, token, head_here, live);
+      map.of(TILE_A_MAP ? 0 : t, column, token, head_here, live);
       if (!live) continue;
-      float2 theirs_ml[WAVES];
-      f32x4 theirs_acc[WAVES];
-#pragma unroll
-      for (int w = 0; w < WAVES; ++w) {
-        const float* theirs = lds + ((size_t)w * 16 + column) * STRIDE;
-        theirs_ml[w] = *(const float2*)(theirs + D);
-        theirs_acc[w] = *(const f32x4*)(theirs + d4);
-      }
-      float best = -INFINITY;
-#pragma unroll
-      for (int w = 0; w < WAVES; ++w) best = fmaxf(best, theirs_ml[w].x);
-      float total = 0.f;
-      f32x4 merged = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int w = 0; w < WAVES; ++w) {
-        const float factor = theirs_ml[w].x == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(theirs_ml[w].x - best);
-        total += theirs_ml[w].y * factor;
-        merged += theirs_acc[w] * factor;
-      }
+      float best, total;
+      f32x4 merged = merge_waves(column, d4, best, total);
       const int head = kv_head * group + head_tile * 16 + head_here;
       const size_t row = (size_t)row0 + token;
       if (splits == 1) {
@@ -773,12 +817,12 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
   }
   if constexpr (CHANGED == CHANGED_MAPS) {
     if (splits > 1) return;
-    // a column's sum of squares, over the threads that hold its pieces (dimensions beyond vdim are zeros)
+    // a result's sum of squares, over the threads that hold its pieces (dimensions beyond vdim are zeros)
     constexpr int PIECES = D / 4, SQUARES = PIECES + 1;
 #pragma unroll
     for (int turn = 0; turn < HELD; ++turn) {
       const int index = threadIdx.x + turn * WAVES * 64;
-      if (index >= 16 * PIECES) continue;
+      if (index >= RESULTS * PIECES) continue;
       const f32x4 v = held[turn];
       lds[(index / PIECES) * SQUARES + index % PIECES] = v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
     }
@@ -786,17 +830,20 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
 #pragma unroll
     for (int turn = 0; turn < HELD; ++turn) {
       const int index = threadIdx.x + turn * WAVES * 64;
-      if (index >= 16 * PIECES) continue;
+      if (index >= RESULTS * PIECES) continue;
       const int column = index / PIECES, d4 = (index % PIECES) * 4;
-      int token, head_here;
-      bool live;
-      map.of(0, column, token, head_here, live);
+      int token = 0, head = (kv_head * group + 2 * column) / 2;
+      bool live = 2 * column < map.columns;
+      if constexpr (!PAIRED) {
+        int head_here;
+        map.of(0, column, token, head_here, live);
+        head = kv_head * group + head_tile * 16 + head_here;
+      }
       if (!live) continue;
       float squares = 0.f;
       for (int i = 0; i < PIECES; ++i) squares += lds[column * SQUARES + i];
       const float normed = finish.out_scale * rsqrtf(squares / (float)finish.vdim + finish.eps);
-      write_finished(finish, out + ((size_t)row0 + token) * out_stride, nullptr, kv_head * group + head_tile * 16 + head_here, d4,
-                     held[turn] * normed);
+      write_finished(finish, out + ((size_t)row0 + token) * out_stride, nullptr, head, d4, held[turn] * normed);
     }
   }
 }
@@ -1207,6 +1254,7 @@ extern "C" int llmserve_attention_portions(const void*, int, void*, int, float*,
 #ifndef FUSED_WAVES
 #define FUSED_WAVES (HEAD_DIM > 128 ? 4 : 8)
 #endif
+#define EIGHT_WAVES (HEAD_DIM > 128 ? 4 : 8)  // (of the kinds that write finished results, in a step of single tokens)
 template <int COLUMN_TILES, bool FUSED, int WAVES, int CHANGED = CHANGED_NOT>
 static int launch_tiles(const void* qkv, int row_width, void* out, int out_stride, float* partial_acc, float* partial_ml,
                         void* keys, void* values, const int* block_tables, int table_width,
@@ -1264,8 +1312,10 @@ extern "C" int llmserve_attention_can_fuse(int pairing) {
 // positions; slopes, cap and kept keys not together with `fuse` & 1, sinks not with `fuse` & 2.
 // `bias` (float32 [heads][reach + BIAS_SPARE], common.h: bias_element, or null) adds a bias by distance to the scores, `gates`
 // (bfloat16 rows of `gate_stride`, or null) multiplies a result's element with the sigmoid of column gate_first + its own;
-// `maps` 2: differential attention, column_tiles 2 with work items made for one column tile, partial results twice as many
-// ([rows * heads * 2 * splits ..]); each of the three writes heads of `vdim` side by side, and goes with no other change.
+// `maps` 2: differential attention, column_tiles 2 with work items made for one column tile, or, in a step of single tokens with up
+// to eight query heads a kv head, column_tiles 1 with work items of both maps of a token; partial results twice as many
+// ([rows * heads * 2 * splits ..]); `fuse` 8 says that they are for a step of single tokens, whose keys eight waves a workgroup
+// walk; each of the three writes heads of `vdim` side by side, and goes with no other change.
 // A row of `out` begins every `out_stride` elements (a multiple of 4 from heads * D, or heads * vdim, on).
 extern "C" int llmserve_attention_tiles(const void* qkv, int row_width, void* out, int out_stride, float* partial_acc,
                                         float* partial_ml, void* keys, void* values,
@@ -1281,8 +1331,11 @@ extern "C" int llmserve_attention_tiles(const void* qkv, int row_width, void* ou
   const bool finished = vdim > 0;
   if (out_stride < heads * (finished ? vdim : D) || (out_stride % 4 && (!finished || vdim % 4 == 0))) return ERR_BAD_ARGUMENT;
   if (vdim > D || (maps != 1 && maps != 2) || (!finished && (bias || gates || maps == 2)) || (bias && reach < 1)) return ERR_BAD_ARGUMENT;
-  if (finished && ((maps == 1) == (bias == nullptr) || fuse || slopes || soft_cap != 0.f || sinks || keep_first > 0 || chunk > 0)) return ERR_BAD_ARGUMENT;
-  if (maps == 2 && (D % 32 || gates || column_tiles != 2 || window > 0)) return ERR_BAD_ARGUMENT;
+  if (finished && ((maps == 1) == (bias == nullptr) || (fuse & ~8) || slopes || soft_cap != 0.f || sinks || keep_first > 0 || chunk > 0)) return ERR_BAD_ARGUMENT;
+  const bool eight_waves = finished && fuse == 8;  // (a step of single tokens)
+  if (finished) fuse &= ~8;
+  if (maps == 2 && (D % 32 || gates || window > 0)) return ERR_BAD_ARGUMENT;
+  if (maps == 2 && column_tiles == 1 && (tiles != rows || !eight_waves || heads / kv_heads > 8)) return ERR_BAD_ARGUMENT;
   if (gates && (gate_first < 0 || gate_first + heads * vdim > gate_stride)) return ERR_BAD_ARGUMENT;
   const Finish finish = {vdim, (const bf16_t*)gates, gate_stride, gate_first, factor, eps, out_scale};
   if (window <= 0) keep_first = 0;  // (without a window every key is seen anyway)
@@ -1311,10 +1364,15 @@ extern "C" int llmserve_attention_tiles(const void* qkv, int row_width, void* ou
     status = edges ? LAUNCH_TILES(1, true, FUSED_WAVES, CHANGED_EDGES) : LAUNCH_TILES(1, true, FUSED_WAVES, CHANGED_NOT);
   } else if (finished) {
 #if HEAD_DIM % 32 == 0
-    if (maps == 2) status = LAUNCH_TILES(2, false, 4, CHANGED_MAPS);
+    if (maps == 2 && column_tiles == 1) {  // both maps of a head in one column tile
+      heads *= 2;
+      status = LAUNCH_TILES(1, false, EIGHT_WAVES, CHANGED_MAPS);
+      heads /= 2;
+    } else if (maps == 2) status = LAUNCH_TILES(2, false, 4, CHANGED_MAPS);
     else
 #endif
-    status = column_tiles == 1 ? LAUNCH_TILES(1, false, 4, CHANGED_BIAS) : LAUNCH_TILES(2, false, 4, CHANGED_BIAS);
+    status = column_tiles == 1 && eight_waves ? LAUNCH_TILES(1, false, EIGHT_WAVES, CHANGED_BIAS)
+             : column_tiles == 1        ? LAUNCH_TILES(1, false, 4, CHANGED_BIAS) : LAUNCH_TILES(2, false, 4, CHANGED_BIAS);
     if (status != 0 || splits == 1) return status;
     if (maps == 2)
       hipLaunchKernelGGL(attention_merge_finish_kernel<true>, dim3((unsigned)rows * heads), dim3(MERGE_THREADS), 0, stream, partial_acc,

@@ -166,7 +166,8 @@ __global__ __launch_bounds__(256) void convolved_heads_vector_kernel(
 #pragma unroll
       for (int e = 0; e < 8; ++e) value[e] = (float)raw[e];
     } else {
-      const int request = token_request[token], inside = token - start[request];
+      // (a step of single tokens: token i is request i's, its first in the step)
+      const int request = TOKENS == 1 ? token : token_request[token], inside = TOKENS == 1 ? 0 : token - start[request];
       if constexpr (TAPS > 1) kept = window + (size_t)slots[request] * (TAPS - 1) * z.channels + (live ? column : 0);
       float input[TAPS][8];
 #pragma unroll

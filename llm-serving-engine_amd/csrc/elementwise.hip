@@ -21,11 +21,39 @@ __global__ void embedding_kernel(const T* __restrict__ table, const int* __restr
   for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = to_float(src[i]) * scale;
 }
 
+// the same in pieces of four (a width that is a multiple of four): a thread a piece
+template <typename T>
+__global__ __launch_bounds__(256) void embedding_pieces_kernel(const T* __restrict__ table, const int* __restrict__ ids, float* __restrict__ out,
+                                                               int quads, float scale, const T* __restrict__ places,
+                                                               const int* __restrict__ positions, int place_rows) {
+  typedef T four __attribute__((ext_vector_type(4)));
+  const int c = blockIdx.y * blockDim.x + threadIdx.x;
+  if (c >= quads) return;
+  const four v = ((const four*)table)[(size_t)ids[blockIdx.x] * quads + c];
+  float4 r = make_float4((float)v[0] * scale, (float)v[1] * scale, (float)v[2] * scale, (float)v[3] * scale);
+  if (places) {
+    const four p = ((const four*)places)[(size_t)min(max(positions[blockIdx.x], 0), place_rows - 1) * quads + c];
+    r.x += (float)p[0]; r.y += (float)p[1]; r.z += (float)p[2]; r.w += (float)p[3];
+  }
+  ((float4*)out)[(size_t)blockIdx.x * quads + c] = r;
+}
+
 extern "C" int llmserve_embedding(const void* table, int table_is_float, const int* ids, float* out,
                                   int tokens, int hidden, float scale, const void* places, const int* positions, int place_rows,
                                   hipStream_t stream) {
   if (tokens <= 0) return 0;
   if (places && (!positions || place_rows < 1)) return ERR_BAD_ARGUMENT;
+  if (hidden % 4 == 0) {
+    const int quads = hidden / 4, threads = quads <= 64 ? 64 : quads <= 128 ? 128 : 256;
+    const dim3 grid(tokens, (quads + threads - 1) / threads);
+    if (table_is_float)
+      hipLaunchKernelGGL(embedding_pieces_kernel<float>, grid, dim3(threads), 0, stream, (const float*)table, ids, out, quads, scale,
+                         (const float*)places, positions, place_rows);
+    else
+      hipLaunchKernelGGL(embedding_pieces_kernel<bf16_t>, grid, dim3(threads), 0, stream, (const bf16_t*)table, ids, out, quads, scale,
+                         (const bf16_t*)places, positions, place_rows);
+    return LAUNCH_STATUS();
+  }
   if (table_is_float)
     hipLaunchKernelGGL(embedding_kernel<float>, dim3(tokens), dim3(256), 0, stream, (const float*)table, ids, out, hidden, scale,
                        (const float*)places, positions, place_rows);

@@ -381,26 +381,25 @@ extern "C" int llmserve_headwise_linear(const void* x, int is_float, int rows, i
 // chosen[t, i] and weight[t, i] = scale * s_e, with `renormalise` scale * s_e / (sum of the chosen s + 1e-20).  Lane l
 // keeps the experts l, l + 64, ...; a pick is the wave's best of the lanes' best, which is then struck out.
 #define ROUTE_PER_LANE 16
-__global__ __launch_bounds__(WAVE) void route_kernel(const float* __restrict__ z, int z_stride, int experts,
-                                                     const float* __restrict__ correction, int top, float scale,
-                                                     int* __restrict__ chosen, float* __restrict__ weight, int softmax,
-                                                     int groups, int keep, int renormalise) {
-  __shared__ float by_expert[ROUTE_PER_LANE * WAVE];
-  __shared__ float by_group[ROUTE_PER_LANE * WAVE];
-  const int t = blockIdx.x, lane = threadIdx.x;
-  const float* row = z + (size_t)t * z_stride;
-  float score[ROUTE_PER_LANE], choice[ROUTE_PER_LANE];
+// One wave and one token: `row` its scores, `chosen` and `weight` where its choice goes (at most PER_LANE * 64 experts); by_expert
+// and by_group have room for as many floats as experts and are the wave's own.  All waves of a workgroup call it together.
+template <int PER_LANE>
+__device__ __forceinline__ void route_one(const float* row, int experts, const float* __restrict__ correction, int top, float scale,
+                                          int* chosen, float* weight, int softmax, int groups, int keep, int renormalise,
+                                          float* by_expert, float* by_group) {
+  const int lane = threadIdx.x & (WAVE - 1);
+  float score[PER_LANE], choice[PER_LANE];
   float top_z = -INFINITY, total = 1.f;
   if (softmax) {  // over all experts: exp(z - max) / sum
 #pragma unroll
-    for (int j = 0; j < ROUTE_PER_LANE; ++j) {
+    for (int j = 0; j < PER_LANE; ++j) {
       const int e = lane + j * WAVE;
       if (e < experts) top_z = fmaxf(top_z, row[e]);
     }
     top_z = wave_max(top_z);
     total = 0.f;
 #pragma unroll
-    for (int j = 0; j < ROUTE_PER_LANE; ++j) {
+    for (int j = 0; j < PER_LANE; ++j) {
       const int e = lane + j * WAVE;
       score[j] = e < experts ? expf(row[e] - top_z) : 0.f;
       total += score[j];
@@ -408,7 +407,7 @@ __global__ __launch_bounds__(WAVE) void route_kernel(const float* __restrict__ z
     total = wave_sum(total);
   }
 #pragma unroll
-  for (int j = 0; j < ROUTE_PER_LANE; ++j) {
+  for (int j = 0; j < PER_LANE; ++j) {
     const int e = lane + j * WAVE;
     if (softmax) score[j] = score[j] / total;
     else score[j] = e < experts ? 1.f / (1.f + expf(-row[e])) : 0.f;
@@ -419,7 +418,7 @@ __global__ __launch_bounds__(WAVE) void route_kernel(const float* __restrict__ z
     // among equals, as everywhere here).
     const int size = experts / groups;
 #pragma unroll
-    for (int j = 0; j < ROUTE_PER_LANE; ++j)
+    for (int j = 0; j < PER_LANE; ++j)
       if (lane + j * WAVE < experts) by_expert[lane + j * WAVE] = choice[j];
     __syncthreads();
     for (int g = lane; g < groups; g += WAVE) {
@@ -430,7 +429,7 @@ __global__ __launch_bounds__(WAVE) void route_kernel(const float* __restrict__ z
     __syncthreads();
     // group g stays if fewer than `keep` groups come before it in the order (score descending, index ascending)
 #pragma unroll
-    for (int j = 0; j < ROUTE_PER_LANE; ++j) {
+    for (int j = 0; j < PER_LANE; ++j) {
       const int e = lane + j * WAVE;
       if (e >= experts) continue;
       const int g = e / size;
@@ -445,7 +444,7 @@ __global__ __launch_bounds__(WAVE) void route_kernel(const float* __restrict__ z
     float best = -INFINITY, best_score = 0.f;
     int best_expert = 0x7fffffff;
 #pragma unroll
-    for (int j = 0; j < ROUTE_PER_LANE; ++j) {
+    for (int j = 0; j < PER_LANE; ++j) {
       const int e = lane + j * WAVE;
       if (e < experts && (choice[j] > best || best_expert == 0x7fffffff)) { best = choice[j]; best_score = score[j]; best_expert = e; }
     }
@@ -459,15 +458,26 @@ __global__ __launch_bounds__(WAVE) void route_kernel(const float* __restrict__ z
     }
     sum += best_score;
     if (lane == 0) {
-      chosen[(size_t)t * top + i] = best_expert;
-      weight[(size_t)t * top + i] = renormalise ? best_score : scale * best_score;
+      chosen[i] = best_expert;
+      weight[i] = renormalise ? best_score : scale * best_score;
     }
 #pragma unroll
-    for (int j = 0; j < ROUTE_PER_LANE; ++j)
+    for (int j = 0; j < PER_LANE; ++j)
       if (lane + j * WAVE == best_expert) choice[j] = -INFINITY;
   }
   if (renormalise && lane == 0)  // (the lane reads back what it wrote itself)
-    for (int i = 0; i < top; ++i) weight[(size_t)t * top + i] = weight[(size_t)t * top + i] / (sum + 1e-20f) * scale;
+    for (int i = 0; i < top; ++i) weight[i] = weight[i] / (sum + 1e-20f) * scale;
+}
+
+__global__ __launch_bounds__(WAVE) void route_kernel(const float* __restrict__ z, int z_stride, int experts,
+                                                     const float* __restrict__ correction, int top, float scale,
+                                                     int* __restrict__ chosen, float* __restrict__ weight, int softmax,
+                                                     int groups, int keep, int renormalise) {
+  __shared__ float by_expert[ROUTE_PER_LANE * WAVE];
+  __shared__ float by_group[ROUTE_PER_LANE * WAVE];
+  const size_t t = blockIdx.x;
+  route_one<ROUTE_PER_LANE>(z + t * z_stride, experts, correction, top, scale, chosen + t * top, weight + t * top, softmax, groups, keep,
+                            renormalise, by_expert, by_group);
 }
 
 // `correction` may be null (the choice is by score alone).  softmax 0: sigmoid of each score; 1: softmax over all experts.
@@ -489,44 +499,71 @@ extern "C" int llmserve_route(const float* z, int z_stride, int experts, const f
 // there is room for ceil(pairs / tile_rows) + experts of them, and those not needed have no rows.
 #define SORT_THREADS 1024
 #define MAX_EXPERTS 1024
-__global__ __launch_bounds__(SORT_THREADS) void sort_pairs_kernel(const int* __restrict__ chosen, int pairs, int experts,
-                                                                  int* __restrict__ place, int* __restrict__ order,
-                                                                  int* __restrict__ tiles, int capacity, int tile_rows) {
-  __shared__ int count[MAX_EXPERTS], first[MAX_EXPERTS], first_tile[MAX_EXPERTS + 1];
-  for (int e = threadIdx.x; e < experts; e += SORT_THREADS) count[e] = 0;
+// All SORT_THREADS threads of a workgroup; `chosen` and `place` may lie in LDS.
+struct SortSpace { int count[MAX_EXPERTS], first[MAX_EXPERTS], first_tile[MAX_EXPERTS + 1]; };
+
+__device__ __forceinline__ void sort_pairs(const int* chosen, int pairs, int experts, int* place, int* order, int* tiles, int capacity,
+                                           int tile_rows, SortSpace& s) {
+  for (int e = threadIdx.x; e < experts; e += SORT_THREADS) s.count[e] = 0;
   __syncthreads();
-  for (int p = threadIdx.x; p < pairs; p += SORT_THREADS) place[p] = atomicAdd(&count[chosen[p]], 1);
+  for (int p = threadIdx.x; p < pairs; p += SORT_THREADS) place[p] = atomicAdd(&s.count[chosen[p]], 1);
   __syncthreads();
-  if (threadIdx.x == 0) {
+  if (experts <= WAVE) {  // running sums over the experts: a lane an expert
+    if (threadIdx.x < WAVE) {
+      const int lane = threadIdx.x;
+      const int mine = lane < experts ? s.count[lane] : 0, mine_tiles = (mine + tile_rows - 1) / tile_rows;
+      int rows = mine, tile = mine_tiles;
+#pragma unroll
+      for (int offset = 1; offset < WAVE; offset <<= 1) {
+        const int before = __shfl_up(rows, offset, WAVE), tiles_before = __shfl_up(tile, offset, WAVE);
+        if (lane >= offset) {
+          rows += before;
+          tile += tiles_before;
+        }
+      }
+      if (lane < experts) {
+        s.first[lane] = rows - mine;
+        s.first_tile[lane] = tile - mine_tiles;
+      }
+      if (lane == experts - 1) s.first_tile[experts] = tile;
+    }
+  } else if (threadIdx.x == 0) {
     int rows = 0, tile = 0;
     for (int e = 0; e < experts; ++e) {
-      first[e] = rows;
-      first_tile[e] = tile;
-      rows += count[e];
-      tile += (count[e] + tile_rows - 1) / tile_rows;
+      s.first[e] = rows;
+      s.first_tile[e] = tile;
+      rows += s.count[e];
+      tile += (s.count[e] + tile_rows - 1) / tile_rows;
     }
-    first_tile[experts] = tile;
+    s.first_tile[experts] = tile;
   }
   __syncthreads();
   for (int p = threadIdx.x; p < pairs; p += SORT_THREADS) {
-    const int where = first[chosen[p]] + place[p];
+    const int where = s.first[chosen[p]] + place[p];
     place[p] = where;
     order[where] = p;
   }
   for (int e = threadIdx.x; e < experts; e += SORT_THREADS) {
-    const int n = (count[e] + tile_rows - 1) / tile_rows;
+    const int n = (s.count[e] + tile_rows - 1) / tile_rows;
     for (int i = 0; i < n; ++i) {
-      int* tile = tiles + 3 * (size_t)(first_tile[e] + i);
+      int* tile = tiles + 3 * (size_t)(s.first_tile[e] + i);
       tile[0] = e;
-      tile[1] = first[e] + i * tile_rows;
-      tile[2] = min(tile_rows, count[e] - i * tile_rows);
+      tile[1] = s.first[e] + i * tile_rows;
+      tile[2] = min(tile_rows, s.count[e] - i * tile_rows);
     }
   }
-  for (int i = first_tile[experts] + threadIdx.x; i < capacity; i += SORT_THREADS) {
+  for (int i = s.first_tile[experts] + threadIdx.x; i < capacity; i += SORT_THREADS) {
     tiles[3 * (size_t)i] = 0;
     tiles[3 * (size_t)i + 1] = 0;
     tiles[3 * (size_t)i + 2] = 0;
   }
+}
+
+__global__ __launch_bounds__(SORT_THREADS) void sort_pairs_kernel(const int* __restrict__ chosen, int pairs, int experts,
+                                                                  int* __restrict__ place, int* __restrict__ order,
+                                                                  int* __restrict__ tiles, int capacity, int tile_rows) {
+  __shared__ SortSpace space;
+  sort_pairs(chosen, pairs, experts, place, order, tiles, capacity, tile_rows, space);
 }
 
 extern "C" int llmserve_sort_pairs(const int* chosen, int pairs, int experts, int* place, int* order, int* tiles,
@@ -537,6 +574,111 @@ extern "C" int llmserve_sort_pairs(const int* chosen, int pairs, int experts, in
     return ERR_BAD_ARGUMENT;
   hipLaunchKernelGGL(sort_pairs_kernel, dim3(1), dim3(SORT_THREADS), 0, stream, chosen, pairs, experts, place, order, tiles, capacity,
                      tile_rows);
+  return LAUNCH_STATUS();
+}
+
+// ---------------------------------------------------------------------------- router, choice and sort of a few tokens
+// A step of up to 16 tokens (decoding) and up to 64 experts: the router's product, the choice and the sort by expert in one
+// launch of one workgroup, where three launches take longer to start than to run.  The product is made on the matrix cores
+// (16 rows of the router by the tokens, K dealt out to the waves in 32-wide steps, their partial sums added in wave order);
+// the scores lie in LDS between (and go to memory for whoever else reads them).  Then wave t chooses for token t.  A token
+// names an expert once at most, so an expert has no more rows than there are tokens: one tile; and a pair's place is the
+// number of pairs before it by (expert, number), counted by its own lane.
+#define FEW_TOKENS 16
+#define FEW_EXPERTS 64
+#define FEW_TILES 5   // of 16 router rows: the experts' and a row or more of something else
+#define FEW_PAIRS 256
+#define FEW_WAVES 16
+
+__global__ __launch_bounds__(FEW_WAVES * WAVE) void route_few_kernel(
+    const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, const void* __restrict__ bias, int bias_is_float, int tokens, int outputs,
+    int inner, int experts, const float* __restrict__ correction, int top, float scale, int softmax, int groups, int keep, int renormalise,
+    float* __restrict__ scores, int* __restrict__ chosen, float* __restrict__ weight, int* __restrict__ place, int* __restrict__ order,
+    int* __restrict__ tiles, int capacity) {
+  __shared__ f32x4 partial[FEW_WAVES][WAVE];
+  __shared__ float z[FEW_TOKENS][FEW_TILES * 16];
+  __shared__ float by_expert[FEW_TOKENS][FEW_EXPERTS], by_group[FEW_TOKENS][FEW_EXPERTS];
+  __shared__ int picked[FEW_PAIRS + FEW_TOKENS * FEW_EXPERTS];
+  __shared__ float shares[FEW_TOKENS][FEW_EXPERTS];
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
+  const int row_tiles = (outputs + 15) / 16, slices = FEW_WAVES / row_tiles;
+  const int my_tile = wave / slices, my_slice = wave % slices;
+  f32x4 acc = (f32x4){0.f, 0.f, 0.f, 0.f};
+  if (my_tile < row_tiles) {
+    const bf16_t* a_row = w + (size_t)min(my_tile * 16 + r, outputs - 1) * inner + g * 8;
+    const bf16_t* b_row = x + (size_t)min(r, tokens - 1) * inner + g * 8;
+#pragma unroll 8
+    for (int step = my_slice; step < inner / 32; step += slices)
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(a_row + step * 32), *(const bf16x8*)(b_row + step * 32), acc, 0, 0, 0);
+  }
+  partial[wave][lane] = acc;
+  __syncthreads();
+  if (wave < row_tiles) {  // lane (r, g) holds token r and rows 16 wave + 4 g .. + 3
+    f32x4 total = partial[wave * slices][lane];
+    for (int s = 1; s < slices; ++s) total += partial[wave * slices + s][lane];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int n = wave * 16 + g * 4 + e;
+      const float v = total[e] + (bias && n < outputs ? load_as_float(bias, bias_is_float, n) : 0.f);
+      z[r][n] = v;
+      if (r < tokens && n < outputs) scores[(size_t)r * outputs + n] = v;
+    }
+  }
+  __syncthreads();
+  // (waves without a token of their own choose for the last one once more, to a place of their own)
+  int* mine = picked + (wave < tokens ? wave * top : FEW_PAIRS + wave * FEW_EXPERTS);
+  route_one<1>(z[min(wave, tokens - 1)], experts, correction, top, scale, mine, shares[wave], softmax, groups, keep, renormalise,
+               by_expert[wave], by_group[wave]);
+  __syncthreads();
+  const int pairs = tokens * top;
+  for (int p = threadIdx.x; p < pairs; p += FEW_WAVES * WAVE) {
+    const int expert = picked[p];
+    int before = 0;
+    for (int q = 0; q < pairs; ++q) before += picked[q] < expert || (picked[q] == expert && q < p) ? 1 : 0;
+    chosen[p] = expert;
+    weight[p] = shares[p / top][p % top];
+    place[p] = before;
+    order[before] = p;
+  }
+  if (wave == FEW_WAVES - 1) {  // a lane an expert
+    int count = 0, before = 0;
+    for (int q = 0; q < pairs; ++q) {
+      count += picked[q] == lane ? 1 : 0;
+      before += picked[q] < lane ? 1 : 0;
+    }
+    const unsigned long long named = __ballot(count > 0);
+    if (count > 0) {
+      int* tile = tiles + 3 * (size_t)__popcll(named & ((1ull << lane) - 1));
+      tile[0] = lane;
+      tile[1] = before;
+      tile[2] = count;
+    }
+    for (int i = __popcll(named) + lane; i < capacity; i += WAVE) {
+      tiles[3 * (size_t)i] = 0;
+      tiles[3 * (size_t)i + 1] = 0;
+      tiles[3 * (size_t)i + 2] = 0;
+    }
+  }
+}
+
+extern "C" int llmserve_route_few_takes(int tokens, int outputs, int inner, int experts, int top) {
+  return tokens >= 1 && tokens <= FEW_TOKENS && experts <= FEW_EXPERTS && outputs <= FEW_TILES * 16 && inner % 32 == 0 && tokens * top <= FEW_PAIRS ? 1 : 0;
+}
+
+// bias (bfloat16 or float32 [outputs]) and correction (float32 [experts]) may be null; outputs >= experts rows of w, of which the
+// first `experts` are the experts'; `capacity` tiles, of 16 rows or more.
+extern "C" int llmserve_route_few(const void* x, const void* w, const void* bias, int bias_is_float, int tokens, int outputs, int inner,
+                                  int experts, const float* correction, int top, float scale, int softmax, int groups, int keep,
+                                  int renormalise, float* scores, int* chosen, float* weight, int* place, int* order, int* tiles,
+                                  int capacity, int tile_rows, hipStream_t stream) {
+  if (tokens <= 0) return 0;
+  if (!llmserve_route_few_takes(tokens, outputs, inner, experts, top) || experts < 1 || top < 1 || top > experts || experts > outputs)
+    return ERR_BAD_ARGUMENT;
+  if (groups < 1 || experts % groups || keep < 1 || keep > groups || top > keep * (experts / groups)) return ERR_BAD_ARGUMENT;
+  if (tile_rows < FEW_TOKENS || capacity < min(experts, tokens * top)) return ERR_BAD_ARGUMENT;
+  hipLaunchKernelGGL(route_few_kernel, dim3(1), dim3(FEW_WAVES * WAVE), 0, stream, (const bf16_t*)x, (const bf16_t*)w, bias, bias_is_float,
+                     tokens, outputs, inner, experts, correction, top, scale, softmax, groups, keep, renormalise, scores, chosen, weight,
+                     place, order, tiles, capacity);
   return LAUNCH_STATUS();
 }
 
@@ -651,6 +793,55 @@ extern "C" int llmserve_expert_product(const void* x, int is_float, const int* o
 // ---------------------------------------------------------------------------- the tokens' weighted sums
 // out[t] = sum_i weight[t, i] * rows[place[t * top + i]], in the order of i; with `shared`, plus
 // sigmoid(gates[t, gate_column]) * shared[t] (an expert that every token uses, behind a gate of its own).
+template <int AT_ONCE>
+__device__ __forceinline__ void add_choices(float4& sum, const float4* rows, const int* place, const float* weight, int first, int top,
+                                            int quads, int c) {
+  float4 row[AT_ONCE];
+  float share[AT_ONCE];
+#pragma unroll
+  for (int i = 0; i < AT_ONCE; ++i) {  // (all asked for before the first is used; those beyond the last choice read it again)
+    const int choice = min(first + i, top - 1);
+    share[i] = weight[choice];
+    row[i] = rows[(size_t)place[choice] * quads + c];
+  }
+#pragma unroll
+  for (int i = 0; i < AT_ONCE; ++i) {
+    if (first + i >= top) continue;
+    sum.x += share[i] * row[i].x; sum.y += share[i] * row[i].y; sum.z += share[i] * row[i].z; sum.w += share[i] * row[i].w;
+  }
+}
+
+// rows whose length is a multiple of four: a thread a 16-byte piece
+__global__ __launch_bounds__(256) void combine_pairs_vector_kernel(const float4* __restrict__ rows, const int* __restrict__ place,
+                                                                   const float* __restrict__ weight, int top, float4* __restrict__ out,
+                                                                   int quads, const float4* __restrict__ shared, int parts,
+                                                                   const float* __restrict__ gates, int gate_stride, int gate_column) {
+  const int t = blockIdx.x, c = blockIdx.y * blockDim.x + threadIdx.x;
+  if (c >= quads) return;
+  float4 beside = make_float4(0.f, 0.f, 0.f, 0.f);
+  if (shared) {
+    beside = shared[(size_t)t * quads + c];
+    for (int p = 1; p < parts; ++p) {
+      const float4 more = shared[((size_t)p * gridDim.x + t) * quads + c];
+      beside.x += more.x; beside.y += more.y; beside.z += more.z; beside.w += more.w;
+    }
+    if (gates) {
+      const float gate = 1.f / (1.f + expf(-gates[(size_t)t * gate_stride + gate_column]));
+      beside.x *= gate; beside.y *= gate; beside.z *= gate; beside.w *= gate;
+    }
+  }
+  float4 sum = make_float4(0.f, 0.f, 0.f, 0.f);
+  const int* mine = place + (size_t)t * top;
+  const float* shares = weight + (size_t)t * top;
+  if (top <= 2) {
+    add_choices<2>(sum, rows, mine, shares, 0, top, quads, c);
+  } else {
+    for (int first = 0; first < top; first += 4) add_choices<4>(sum, rows, mine, shares, first, top, quads, c);
+  }
+  sum.x += beside.x; sum.y += beside.y; sum.z += beside.z; sum.w += beside.w;
+  out[(size_t)t * quads + c] = sum;
+}
+
 __global__ void combine_pairs_kernel(const float* __restrict__ rows, const int* __restrict__ place, const float* __restrict__ weight,
                                      int top, float* __restrict__ out, int width, const float* __restrict__ shared, int parts,
                                      const float* __restrict__ gates, int gate_stride, int gate_column) {
@@ -674,6 +865,12 @@ extern "C" int llmserve_combine_pairs(const float* rows, const int* place, const
   if (tokens <= 0) return 0;
   if (shared && parts < 1) return ERR_BAD_ARGUMENT;
   if (shared && gates && (gate_column < 0 || gate_column >= gate_stride)) return ERR_BAD_ARGUMENT;  // (no gates: the shared rows are added as they are)
+  if (width % 4 == 0) {
+    const int quads = width / 4, threads = quads <= 64 ? 64 : quads <= 128 ? 128 : 256;
+    hipLaunchKernelGGL(combine_pairs_vector_kernel, dim3(tokens, (quads + threads - 1) / threads), dim3(threads), 0, stream, (const float4*)rows,
+                       place, weight, top, (float4*)out, quads, (const float4*)shared, parts, gates, gate_stride, gate_column);
+    return LAUNCH_STATUS();
+  }
   hipLaunchKernelGGL(combine_pairs_kernel, dim3(tokens), dim3(256), 0, stream, rows, place, weight, top, out, width, shared, parts,
                      gates, gate_stride, gate_column);
   return LAUNCH_STATUS();

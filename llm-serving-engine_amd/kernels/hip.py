@@ -88,6 +88,8 @@ _SIGNATURES = {
     "llmserve_add_gated_rows": "pppiiiip",
     "llmserve_headwise_linear": "piiiiipiiipiiip",
     "llmserve_route": "piipifppiiiiip",
+    "llmserve_route_few_takes": "iiiii",
+    "llmserve_route_few": "pppiiiiipifiiiippppppiip",
     "llmserve_sort_pairs": "piipppiip",
     "llmserve_expert_product": "pipipiipiipiifp",
     "llmserve_expert_product_gates": "iii",
@@ -1087,7 +1089,11 @@ class HipKernels:
         head_tiles = -(-(heads // kv_heads) // 16)
         tokens = qkv.shape[0]
         group_size = heads // kv_heads
-        launches = [(1, *self._attention_work(batch, group_size, 1, 0, per_tile)[:2])]
+        paired = maps == 2 and batch.max_query_length == 1 and group_size <= 8  # both maps of a token's heads in one column tile
+        if paired:
+            launches = [(1, *self._attention_work(batch, 2 * group_size, 1, 0, None)[:2])]
+        else:
+            launches = [(1, *self._attention_work(batch, group_size, 1, 0, per_tile)[:2])]
         shared = False
         padded = getattr(batch, "padded_to", None) is not None  # a captured step: the same launches whatever it holds
         whole_pages = group.page_size >= 16 and group.page_size & (group.page_size - 1) == 0  # (what that kernel takes)
@@ -1209,7 +1215,7 @@ class HipKernels:
             status = library.llmserve_attention_tiles(
                 _pointer(qkv), layout.stride, _pointer(out), out.shape[1], _pointer(partial_acc), _pointer(partial_ml),
                 _pointer(cell.keys), _pointer(cell.values), _pointer(group.block_tables), group.width, _pointer(batch.positions), _pointer(work), items,
-                column_tiles if maps == 1 else 2, tokens, heads, kv_heads, group.page_size, scale, window, splits, (1 if fuse is not None else 0) + (2 if unmerged else 0) + (4 if by_item else 0),
+                column_tiles if maps == 1 or paired else 2, tokens, heads, kv_heads, group.page_size, scale, window, splits, (1 if fuse is not None else 0) + (2 if unmerged else 0) + (4 if by_item else 0) + (8 if finish is not None and batch.max_query_length == 1 else 0),
                 _pointer(table), _PAIRINGS[pairing], _pointer(group.slot_mapping), _pointer(slopes), soft_cap, _pointer(sinks), keep_first, chunk,
                 _pointer(bias), reach, maps, vdim, float(factor), float(eps), float(out_scale), _pointer(gates),
                 gates.shape[1] if gates is not None else 0, gate_first, self._stream,
@@ -1447,6 +1453,48 @@ class HipKernels:
         _check(status, "route")
         return chosen, weights
 
+    @staticmethod
+    def _expert_tiles(x, experts, pairs: int) -> tuple[int, int, bool]:
+        """(rows a tile of the grouped products, tiles at most, whether the matrix-core kernels take them)."""
+        ups, _, _, gated = experts
+        count, size, hidden = ups.shape
+        # tiles of 64 rows for the matrix cores where an expert has that many rows or so, else of 16
+        width = size // 2 if gated else size  # (the second product's inner size)
+        on_cores = x.dtype == torch.bfloat16 and hidden % 32 == 0 and width % 32 == 0
+        tile_rows = 64 if on_cores and pairs >= 32 * count else 16
+        if on_cores and pairs >= 96 * count and hidden % 64 == 0 and width % 64 == 0:
+            tile_rows = 128  # many rows an expert: both operands through LDS
+        return tile_rows, -(-pairs // tile_rows) + count, on_cores
+
+    def route_product(self, x, router: LinearWeights, experts, count: int, correction, top: int, scale: float, scoring: str, groups: int = 1,
+                      keep_groups: int = 1, renormalise: bool = False):
+        """For up to 16 tokens in bfloat16 the product, the choice and the sort by expert are one launch."""
+        tokens = x.shape[0]
+        if (
+            x.dtype == torch.bfloat16
+            and router.weight.dtype == torch.bfloat16
+            and scoring in ("sigmoid", "softmax")
+            and self._library_of("gemm_rows").llmserve_route_few_takes(tokens, router.out_features, router.in_features, count, top)
+        ):
+            if x.shape[1] != router.in_features or (correction is not None and (correction.dtype != torch.float32 or correction.shape != (count,))):
+                raise KernelError("route_product: rows as wide as the router's weight, and one float32 correction an expert")
+            pairs = tokens * top
+            tile_rows, capacity, _ = self._expert_tiles(x, experts, pairs)
+            scores = self._empty((tokens, router.out_features), torch.float32)
+            chosen, weights = self._empty((tokens, top), torch.int32), self._empty((tokens, top), torch.float32)
+            place, order, tiles = (self._empty(shape, torch.int32) for shape in ((pairs,), (pairs,), (capacity, 3)))
+            bias = router.bias
+            status = self._library_of("gemm_rows").llmserve_route_few(
+                _pointer(x), _pointer(router.weight), _pointer(bias), _is_float(bias) if bias is not None else 0, tokens, router.out_features,
+                router.in_features, count, _pointer(correction), top, float(scale), 1 if scoring == "softmax" else 0, groups, keep_groups,
+                1 if renormalise else 0, _pointer(scores), _pointer(chosen), _pointer(weights), _pointer(place), _pointer(order), _pointer(tiles),
+                capacity, tile_rows, self._stream,
+            )
+            _check(status, "route_product")
+            return scores, chosen, weights, (place, order, tiles)
+        scores = self.linear(x, router, out_dtype=torch.float32)
+        return scores, *self.route(scores, count, correction, top, scale, scoring, groups, keep_groups, renormalise), None
+
     def prepare_experts(self, ups: list[torch.Tensor], downs: list[torch.Tensor], activation: str, gates: list[torch.Tensor] | None = None,
                         limit: float | None = None):
         """The experts' weights stacked: ([experts, size, hidden], [experts, hidden, size], activation, gated).  With `gates`
@@ -1461,7 +1509,7 @@ class HipKernels:
         both = torch.stack([torch.stack([gate, up], dim=1).reshape(2 * up.shape[0], up.shape[1]) for gate, up in zip(gates, ups)])
         return both.contiguous(), torch.stack(list(downs)).contiguous(), (activation, float(limit)) if limit is not None else activation, True
 
-    def expert_feed_forward(self, x, experts, chosen, weights, shared=None, gates=None, gate_column: int = 0) -> torch.Tensor:
+    def expert_feed_forward(self, x, experts, chosen, weights, shared=None, gates=None, gate_column: int = 0, sorted_pairs=None) -> torch.Tensor:
         """sum over a token's chosen experts of weight * down(act(up x)), float32 [T, hidden].  The (token, choice)
         pairs are sorted by expert on the device, the two products run over tiles of one expert's rows, and a last
         kernel adds each token's rows up in the order of its choices; with `shared` (float32 [T, hidden]) it adds
@@ -1474,17 +1522,13 @@ class HipKernels:
             raise KernelError("experts: rows and weights are of one type")
         library = self._library_of("gemm_rows")
         pairs = tokens * top
-        # tiles of 64 rows for the matrix cores where an expert has that many rows or so, else of 16
         width = size // 2 if gated else size  # (the second product's inner size)
-        on_cores = x.dtype == torch.bfloat16 and hidden % 32 == 0 and width % 32 == 0
-        tile_rows = 64 if on_cores and pairs >= 32 * count else 16
-        if on_cores and pairs >= 96 * count and hidden % 64 == 0 and width % 64 == 0:
-            tile_rows = 128  # many rows an expert: both operands through LDS
-        capacity = -(-pairs // tile_rows) + count
-        place = self._empty((pairs,), torch.int32)
-        order = self._empty((pairs,), torch.int32)
-        tiles = self._empty((capacity, 3), torch.int32)
-        _check(library.llmserve_sort_pairs(_pointer(chosen), pairs, count, _pointer(place), _pointer(order), _pointer(tiles), capacity, tile_rows, self._stream), "experts: sort")
+        tile_rows, capacity, on_cores = self._expert_tiles(x, experts, pairs)
+        if sorted_pairs is not None:
+            place, order, tiles = sorted_pairs
+        else:
+            place, order, tiles = (self._empty(shape, torch.int32) for shape in ((pairs,), (pairs,), (capacity, 3)))
+            _check(library.llmserve_sort_pairs(_pointer(chosen), pairs, count, _pointer(place), _pointer(order), _pointer(tiles), capacity, tile_rows, self._stream), "experts: sort")
         # the matrix-core kernels gate their result themselves (act(gate) * up of neighbouring columns); behind the others a
         # kernel of its own does
         fused = gated and bool(library.llmserve_expert_product_gates(_is_float(x), hidden, tile_rows))

@@ -272,6 +272,13 @@ class Kernels(Protocol):
         neighbours (a group's score is its largest); -> (int32 [T, top] experts, float32 [T, top] weights = scale * s of the
         chosen, with `renormalise` scale * s / (sum of the chosen s + 1e-20))."""
 
+    def route_product(
+        self, x: torch.Tensor, router: Any, experts: Any, count: int, correction: torch.Tensor | None, top: int, scale: float, scoring: str,
+        groups: int = 1, keep_groups: int = 1, renormalise: bool = False,
+    ):
+        """`scores = linear(x, router, float32)` and `route(scores, count, ...)` for the experts that `prepare_experts` returned
+        -> (scores, chosen, weights, whatever `expert_feed_forward` takes as `sorted_pairs`, or None)."""
+
     def prepare_experts(
         self, ups: list[torch.Tensor], downs: list[torch.Tensor], activation: str, gates: list[torch.Tensor] | None = None, limit: float | None = None,
     ) -> Any:
@@ -280,7 +287,7 @@ class Kernels(Protocol):
 
     def expert_feed_forward(
         self, x: torch.Tensor, experts: Any, chosen: torch.Tensor, weights: torch.Tensor, shared: torch.Tensor | None = None,
-        gates: torch.Tensor | None = None, gate_column: int = 0,
+        gates: torch.Tensor | None = None, gate_column: int = 0, sorted_pairs: Any = None,
     ) -> torch.Tensor:
         """sum over a token's chosen experts of weight * down_e(act(up_e x)) (+ sigmoid(gates[:, gate_column]) * shared, or
         + shared where no gates are given), float32 [T, hidden]; `shared` may be partial sums [parts, T, hidden]; the inner rows are rounded to the run dtype between the

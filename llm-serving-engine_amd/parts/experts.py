@@ -104,13 +104,13 @@ class RoutedExperts(FeedForward):
     def forward(self, x: torch.Tensor, batch, beside: torch.Tensor | None = None) -> torch.Tensor:
         """With `beside` (float32 rows, or partial sums of them; for a feed-forward with `adds_beside`): plus those rows."""
         kernels, spec = self.kernels, self.spec
-        scores = kernels.linear(x, self.router, out_dtype=torch.float32)  # [T, experts (+ 1)]
-        chosen, weights = kernels.route(
-            scores, spec.num_experts, self.correction, spec.top, spec.route_scale, spec.scoring,
+        # scores float32 [T, experts (+ 1)]
+        scores, chosen, weights, ordered = kernels.route_product(
+            x, self.router, self.experts, spec.num_experts, self.correction, spec.top, spec.route_scale, spec.scoring,
             groups=spec.groups, keep_groups=spec.keep_groups, renormalise=spec.renormalise,
         )
         if self.shared_up is None:
-            return kernels.expert_feed_forward(x, self.experts, chosen, weights, shared=beside)  # float32 [T, hidden]
+            return kernels.expert_feed_forward(x, self.experts, chosen, weights, shared=beside, sorted_pairs=ordered)  # float32 [T, hidden]
         if beside is not None:
             raise ValueError("routed experts: rows beside them are added where there is no shared expert")
         if spec.gated:
@@ -120,5 +120,5 @@ class RoutedExperts(FeedForward):
         shared = kernels.linear(inner, self.shared_down, out_dtype=torch.float32)
         # the kernel that adds a token's experts up adds the (gated) shared expert too
         if not spec.shared_gate:
-            return kernels.expert_feed_forward(x, self.experts, chosen, weights, shared=shared)
-        return kernels.expert_feed_forward(x, self.experts, chosen, weights, shared=shared, gates=scores, gate_column=spec.num_experts)
+            return kernels.expert_feed_forward(x, self.experts, chosen, weights, shared=shared, sorted_pairs=ordered)
+        return kernels.expert_feed_forward(x, self.experts, chosen, weights, shared=shared, gates=scores, gate_column=spec.num_experts, sorted_pairs=ordered)

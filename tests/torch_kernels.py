@@ -483,6 +483,10 @@ class TorchKernels:
             weights = weights / (weights.sum(-1, keepdim=True) + 1e-20)
         return chosen.to(torch.int32), (weights * scale).float()
 
+    def route_product(self, x, router, experts, count, correction, top, scale, scoring, groups=1, keep_groups=1, renormalise=False):
+        scores = self.linear(x, router, out_dtype=torch.float32)
+        return scores, *self.route(scores, count, correction, top, scale, scoring, groups, keep_groups, renormalise), None
+
     def prepare_experts(self, ups, downs, activation, gates=None, limit=None):
         stacked = torch.stack([w.float() for w in gates]) if gates is not None else None
         if activation == "limited_swish":
@@ -496,7 +500,7 @@ class TorchKernels:
         mixed = self.causal_conv(projected, channels, taps, activation, batch, window)
         return self.gated_delta_rule(mixed, controls, rate, step_bias, heads, kv_heads, dim, vdim, batch, state, channel_steps=channel_steps)
 
-    def expert_feed_forward(self, x, experts, chosen, weights, shared=None, gates=None, gate_column=0):
+    def expert_feed_forward(self, x, experts, chosen, weights, shared=None, gates=None, gate_column=0, sorted_pairs=None):
         ups, downs, activation, gate_weights = experts
         out = torch.zeros((x.shape[0], downs.shape[1]))
         rows = torch.zeros((x.shape[0], chosen.shape[1], downs.shape[1]))  # every (token, choice) pair's row, then added in the order of the choices
