@@ -127,15 +127,18 @@ struct Finish {               // how CHANGED_BIAS and CHANGED_MAPS write a resul
 };
 
 // four results of one head, from dimension d4 on, to their row (16-byte aligned where vdim is a multiple of 4)
-__device__ __forceinline__ void write_finished(const Finish& f, bf16_t* row_out, const bf16_t* row_gates, int head, int d4, f32x4 v) {
+// (`early`: the four gates, if they have been asked for ahead; null: they are read here)
+__device__ __forceinline__ bool gates_in_pieces(const Finish& f) { return f.gates && f.vdim % 4 == 0 && (f.gate_stride | f.gate_first) % 4 == 0; }
+__device__ __forceinline__ void write_finished(const Finish& f, bf16_t* row_out, const bf16_t* row_gates, int head, int d4, f32x4 v,
+                                               const bf16x4* early = nullptr) {
   if (d4 >= f.vdim) return;
   const int column = head * f.vdim + d4;
   const bool whole = f.vdim % 4 == 0;
   if (row_gates) {
     const bf16_t* g = row_gates + column;
     float gate[4];
-    if (whole && (f.gate_stride | f.gate_first) % 4 == 0) {
-      const bf16x4 raw = *(const bf16x4*)g;
+    if (gates_in_pieces(f)) {
+      const bf16x4 raw = early ? *early : *(const bf16x4*)g;
 #pragma unroll
       for (int i = 0; i < 4; ++i) gate[i] = (float)raw[i];
     } else {
@@ -622,6 +625,19 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
     }
   };
 
+  // (a step of single tokens: the gates of this thread's piece of the result are asked for here, not when it is written)
+  constexpr bool EARLY_GATES = CHANGED == CHANGED_BIAS && TWO_STEPS && 16 * (D / 4) <= WAVES * 64;
+  [[maybe_unused]] bf16x4 early_gate = (bf16x4){};
+  if constexpr (EARLY_GATES) {
+    const int d4 = (threadIdx.x % (D / 4)) * 4;
+    int token, head_here;
+    bool live;
+    map.of(0, threadIdx.x / (D / 4), token, head_here, live);
+    if (live && gates_in_pieces(finish) && splits == 1 && d4 < finish.vdim)
+      early_gate = *(const bf16x4*)(finish.gates + ((size_t)row0 + token) * finish.gate_stride + finish.gate_first +
+                                    (kv_head * group + head_tile * 16 + head_here) * finish.vdim + d4);
+  }
+
   const float scale_log2 = scale * 1.44269504088896f;
   const int every_first = first_seen_from(last_key);  // every column sees the keys from here on (up to its own)
 
@@ -638,19 +654,21 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
       // A step of single tokens is a few trips to memory in a row, and a wave has two or three steps to
       // walk: its second step's K and V are asked for together with the first's, into registers of their
       // own, and each of the two sets is filled again as soon as its step has been multiplied.
-      auto multiply = [&](int step, StepLoads& L) {
+      auto multiply = [&](int step, StepLoads& L, const float (*bias)[8]) {
         f32x4 s_lo[COLUMN_TILES], s_hi[COLUMN_TILES];
         const int key0 = step * KEYS;
-        [[maybe_unused]] float bias[COLUMN_TILES][8];
-        fetch_bias(key0, bias);
         scores_of(columns, L, s_lo, s_hi);
         const bool interior = key0 + KEYS - 1 <= position0 && key0 >= every_first;
         weigh_and_add<COLUMN_TILES, CHANGED>(columns, L, s_lo, s_hi, key0, q, interior, last_key,
                                              min(max(key0 + 8 * q, low_limit), high_limit), scale_log2, 0.f, 0, bias);
       };
       StepLoads ahead;
+      // (CHANGED_BIAS: a step's biases are asked for with its keys)
+      [[maybe_unused]] float bias_even[COLUMN_TILES][8], bias_odd[COLUMN_TILES][8];
+      fetch_bias(step0 * KEYS, bias_even);
       const int step1 = step0 + WAVES;
       if (step1 < step_end) {
+        fetch_bias(step1 * KEYS, bias_odd);
         const StepPages pages1 =
             second_pages && first_key == 0 && step1 < step_last ? StepPages{second_k, second_k_hi, second_v} : pages_of(step1);
         fetch_keys(step1, pages1, ahead);
@@ -660,15 +678,17 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
       if (step0 + 2 * WAVES < step_end) pages_even = pages_of(step0 + 2 * WAVES);
       if (step0 + 3 * WAVES < step_end) pages_odd = pages_of(step0 + 3 * WAVES);
       for (int step = step0; step < step_end; step += 2 * WAVES) {
-        multiply(step, loads);
+        multiply(step, loads, bias_even);
         if (step + 2 * WAVES < step_end) {
+          fetch_bias((step + 2 * WAVES) * KEYS, bias_even);
           fetch_keys(step + 2 * WAVES, pages_even, loads);
           fetch_values(step + 2 * WAVES, pages_even, loads);
           if (step + 4 * WAVES < step_end) pages_even = pages_of(step + 4 * WAVES);
         }
         if (step + WAVES < step_end) {
-          multiply(step + WAVES, ahead);
+          multiply(step + WAVES, ahead, bias_odd);
           if (step + 3 * WAVES < step_end) {
+            fetch_bias((step + 3 * WAVES) * KEYS, bias_odd);
             fetch_keys(step + 3 * WAVES, pages_odd, ahead);
             fetch_values(step + 3 * WAVES, pages_odd, ahead);
             if (step + 5 * WAVES < step_end) pages_odd = pages_of(step + 5 * WAVES);
@@ -787,7 +807,7 @@ __global__ __launch_bounds__(WAVES * 64, (COLUMN_TILES > 2 || HEAD_DIM > 192 || 
           else held[turn] -= merged * (inverse * finish.factor);
         } else if constexpr (CHANGED == CHANGED_BIAS) {
           write_finished(finish, out + row * out_stride, finish.gates ? finish.gates + row * finish.gate_stride + finish.gate_first : nullptr,
-                         head, d4, merged * inverse);
+                         head, d4, merged * inverse, EARLY_GATES ? &early_gate : nullptr);
         } else {
           const bf16x4 rounded = {(bf16_t)(merged[0] * inverse), (bf16_t)(merged[1] * inverse), (bf16_t)(merged[2] * inverse),
                                   (bf16_t)(merged[3] * inverse)};
