@@ -42,7 +42,7 @@ HEADS = [
     (6, 2, 2, 24, 40, 64),
     (12, 2, 2, 64, 128, 128),
     (3, 3, 2, 40, 8, 96),
-    (4, 1, 2, 48, 96, 96),
+    (4, 1, 2, 40, 88, 96),
     (2, 1, 2, 5, 7, 32),
     (8, 2, 1, 128, 128, 128),
     (3, 1, 1, 80, 80, 80),
@@ -229,7 +229,7 @@ def test_finished_results_that_do_not_fit_are_refused(kernels):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("tokens,experts,top,hidden,size", [(3, 5, 2, 40, 24), (70, 8, 4, 256, 96), (33, 7, 1, 96, 33), (1, 4, 4, 1536, 64), (600, 5, 2, 192, 128), (400, 3, 3, 64, 320)])
+@pytest.mark.parametrize("tokens,experts,top,hidden,size", [(3, 5, 2, 40, 24), (70, 9, 4, 320, 160), (33, 7, 1, 96, 33), (1, 4, 4, 1536, 64), (600, 5, 2, 192, 128), (400, 3, 3, 64, 320)])
 @pytest.mark.parametrize("parts", [None, 1, 3])
 def test_experts_with_a_limit_beside_another_result(kernels, dtype, tokens, experts, top, hidden, size, parts):
     torch.manual_seed(tokens + experts)
