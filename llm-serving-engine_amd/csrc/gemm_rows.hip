@@ -199,73 +199,71 @@ __global__ __launch_bounds__(256) void expert_product_mfma_kernel(const bf16_t* 
   }
 }
 
-// The experts' products of a step of many rows (prompts): tiles of 128 rows of one expert by 128 columns, K in steps of 64
-// through LDS.  All 256 threads bring the two operand tiles from memory sixteen bytes at a time, eight threads a row (128
-// bytes in a row, where the kernel above asks for sixteen rows of 64 bytes an instruction and is bound by the address
-// path), two steps ahead in registers; the four waves (2 x 2) each make 64 x 64 of the result out of LDS.  Rows of LDS are
+// The experts' products of a step of many rows (prompts): tiles of 128 rows of one expert by COLS (128 or 64) columns, K in
+// steps of 64 through LDS.  All 256 threads bring the two operand tiles from memory sixteen bytes at a time, eight threads a
+// row (128 bytes in a row, where the kernel above asks for sixteen rows of 64 bytes an instruction and is bound by the
+// address path), a step ahead in registers; the four waves (2 x 2) each make 64 x COLS / 2 of the result out of LDS.  One step
+// ahead leaves the registers for four workgroups a CU, which hide a step's trip to memory behind each other: two steps ahead
+// and two workgroups took 96 us where this takes 61 (4,096 rows over 16 experts, K 1,536, 2,048 columns).  Rows of LDS are
 // 144 bytes apart (banks).  Rows and columns beyond the tile's are read from the last valid one and never stored.
 #define TILED_ROWS 128
 #define TILED_K 64
 #define TILED_LINE 72  // elements: 64 and 8 of padding
-template <typename TO>
-__global__ __launch_bounds__(256) void expert_tiled_kernel(const bf16_t* __restrict__ x, const int* __restrict__ order, int top,
+template <int COLS, typename TO>
+__global__ __launch_bounds__(256, 3) void expert_tiled_kernel(const bf16_t* __restrict__ x, const int* __restrict__ order, int top,
                                                            const bf16_t* __restrict__ w, int outputs, int inner,
                                                            const int* __restrict__ tiles, TO* __restrict__ out, int activation, float limit) {
-  __shared__ __attribute__((aligned(16))) bf16_t xs[TILED_ROWS * TILED_LINE], ws[TILED_ROWS * TILED_LINE];
+  __shared__ __attribute__((aligned(16))) bf16_t xs[TILED_ROWS * TILED_LINE], ws[COLS * TILED_LINE];
+  constexpr int WAVE_COLS = COLS / 2, CT = WAVE_COLS / 16;  // a wave makes 64 rows by so many columns
   const int* tile = tiles + 3 * (size_t)blockIdx.y;
   const int expert = tile[0], first = tile[1], rows = tile[2];
   if (rows == 0) return;
   const int t = threadIdx.x, wave = t >> 6, lane = t & 63, r = lane & 15, g = lane >> 4;
-  const int wave_row = (wave >> 1) * 64, wave_col = (wave & 1) * 64;
-  const int col0 = blockIdx.x * TILED_ROWS;
+  const int wave_row = (wave >> 1) * 64, wave_col = (wave & 1) * WAVE_COLS;
+  const int col0 = blockIdx.x * COLS;
   const int piece = t % 8;  // which sixteen bytes of a row's 128 a step
   const bf16_t* x_from[4];
-  const bf16_t* w_from[4];
+  const bf16_t* w_from[COLS / 32];
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
     const int row = min(t / 8 + 32 * j, rows - 1), place = first + row;
     x_from[j] = x + (size_t)(top > 0 ? order[place] / top : place) * inner + piece * 8;
+  }
+#pragma unroll
+  for (int j = 0; j < COLS / 32; ++j) {
     const int n = min(col0 + t / 8 + 32 * j, outputs - 1);
     w_from[j] = w + ((size_t)expert * outputs + n) * inner + piece * 8;
   }
-  bf16x8 x_next[4], w_next[4], x_after[4], w_after[4];  // the next step's pieces, and the one's after it
-  const int second = min(TILED_K, inner - TILED_K);
+  bf16x8 x_next[4], w_next[COLS / 32];  // the next step's pieces
 #pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    x_next[j] = *(const bf16x8*)x_from[j];
-    w_next[j] = *(const bf16x8*)w_from[j];
-    x_after[j] = *(const bf16x8*)(x_from[j] + second);
-    w_after[j] = *(const bf16x8*)(w_from[j] + second);
-  }
-  f32x4 acc[4][4];
+  for (int j = 0; j < 4; ++j) x_next[j] = *(const bf16x8*)x_from[j];
 #pragma unroll
-  for (int s = 0; s < 4; ++s)
+  for (int j = 0; j < COLS / 32; ++j) w_next[j] = *(const bf16x8*)w_from[j];
+  f32x4 acc[CT][4];
+#pragma unroll
+  for (int s = 0; s < CT; ++s)
 #pragma unroll
     for (int u = 0; u < 4; ++u) acc[s][u] = (f32x4){0.f, 0.f, 0.f, 0.f};
   for (int k0 = 0; k0 < inner; k0 += TILED_K) {
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      *(bf16x8*)&xs[(t / 8 + 32 * j) * TILED_LINE + piece * 8] = x_next[j];
-      *(bf16x8*)&ws[(t / 8 + 32 * j) * TILED_LINE + piece * 8] = w_next[j];
-      x_next[j] = x_after[j];
-      w_next[j] = w_after[j];
-    }
-    __syncthreads();
-    const int ahead = min(k0 + 2 * TILED_K, inner - TILED_K);  // (in no branch; the last steps ask for the last again)
+    for (int j = 0; j < 4; ++j) *(bf16x8*)&xs[(t / 8 + 32 * j) * TILED_LINE + piece * 8] = x_next[j];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      x_after[j] = *(const bf16x8*)(x_from[j] + ahead);
-      w_after[j] = *(const bf16x8*)(w_from[j] + ahead);
-    }
+    for (int j = 0; j < COLS / 32; ++j) *(bf16x8*)&ws[(t / 8 + 32 * j) * TILED_LINE + piece * 8] = w_next[j];
+    __syncthreads();
+    const int ahead = min(k0 + TILED_K, inner - TILED_K);  // (in no branch; the last step asks for itself again)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) x_next[j] = *(const bf16x8*)(x_from[j] + ahead);
+#pragma unroll
+    for (int j = 0; j < COLS / 32; ++j) w_next[j] = *(const bf16x8*)(w_from[j] + ahead);
 #pragma unroll
     for (int half = 0; half < 2; ++half) {
-      bf16x8 a[4], b[4];
+      bf16x8 a[CT], b[4];
 #pragma unroll
-      for (int s = 0; s < 4; ++s) a[s] = *(const bf16x8*)&ws[(wave_col + s * 16 + r) * TILED_LINE + half * 32 + g * 8];
+      for (int s = 0; s < CT; ++s) a[s] = *(const bf16x8*)&ws[(wave_col + s * 16 + r) * TILED_LINE + half * 32 + g * 8];
 #pragma unroll
       for (int u = 0; u < 4; ++u) b[u] = *(const bf16x8*)&xs[(wave_row + u * 16 + r) * TILED_LINE + half * 32 + g * 8];
 #pragma unroll
-      for (int s = 0; s < 4; ++s)
+      for (int s = 0; s < CT; ++s)
 #pragma unroll
         for (int u = 0; u < 4; ++u) acc[s][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[s], b[u], acc[s][u], 0, 0, 0);
     }
@@ -276,7 +274,7 @@ __global__ __launch_bounds__(256) void expert_tiled_kernel(const bf16_t* __restr
     const int m = wave_row + u * 16 + r;
     if (m >= rows) continue;
 #pragma unroll
-    for (int s = 0; s < 4; ++s) store_four<TO>(out, (size_t)(first + m), col0 + wave_col + s * 16 + g * 4, outputs, activation, acc[s][u], limit);
+    for (int s = 0; s < CT; ++s) store_four<TO>(out, (size_t)(first + m), col0 + wave_col + s * 16 + g * 4, outputs, activation, acc[s][u], limit);
   }
 }
 
@@ -732,13 +730,18 @@ extern "C" int llmserve_expert_product(const void* x, int is_float, const int* o
   if (activation >= ACT_GATED && (outputs % 2 || !llmserve_expert_product_gates(is_float, inner, tile_rows))) return ERR_BAD_ARGUMENT;
   if (!is_float && tile_rows == TILED_ROWS) {
     if (inner % TILED_K) return ERR_BAD_ARGUMENT;
-    const dim3 through_lds((outputs + TILED_ROWS - 1) / TILED_ROWS, capacity);
-    if (out_is_float)
-      hipLaunchKernelGGL(expert_tiled_kernel<float>, through_lds, dim3(256), 0, stream, (const bf16_t*)x, order, top, (const bf16_t*)w,
-                         outputs, inner, tiles, (float*)out, activation, limit);
-    else
-      hipLaunchKernelGGL(expert_tiled_kernel<bf16_t>, through_lds, dim3(256), 0, stream, (const bf16_t*)x, order, top, (const bf16_t*)w,
-                         outputs, inner, tiles, (bf16_t*)out, activation, limit);
+    // (half as wide where the workgroups of 128 columns would not fill the chip's 1,024 places)
+    const int cols = capacity * ((outputs + 127) / 128) <= 1024 ? 64 : 128;
+    const dim3 through_lds((outputs + cols - 1) / cols, capacity);
+#define LAUNCH_TILED(COLS, TO)                                                                                                  \
+  hipLaunchKernelGGL((expert_tiled_kernel<COLS, TO>), through_lds, dim3(256), 0, stream, (const bf16_t*)x, order, top, (const bf16_t*)w, \
+                     outputs, inner, tiles, (TO*)out, activation, limit)
+    if (out_is_float) {
+      if (cols == 128) LAUNCH_TILED(128, float); else LAUNCH_TILED(64, float);
+    } else {
+      if (cols == 128) LAUNCH_TILED(128, bf16_t); else LAUNCH_TILED(64, bf16_t);
+    }
+#undef LAUNCH_TILED
     return LAUNCH_STATUS();
   }
   if (!is_float && inner % 32 == 0) {
