@@ -250,3 +250,34 @@ def test_experts_with_a_limit_beside_another_result(kernels, dtype, tokens, expe
     prepared = mine.prepare_experts([gpu(w) for w in ups], [gpu(w) for w in downs], "limited_swish", gates=[gpu(w) for w in gates], limit=0.9)
     got = mine.expert_feed_forward(gpu(x), prepared, chosen, weights, shared=None if beside is None else gpu(beside))
     close(got, want, dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("tokens", [1, 3, 8, 16, 17])
+@pytest.mark.parametrize("experts,top,extra,hidden,groups,keep", [(5, 2, 0, 64, 1, 1), (16, 2, 0, 1536, 1, 1), (16, 4, 1, 352, 4, 2), (64, 8, 1, 96, 8, 3), (64, 16, 0, 96, 1, 1), (65, 3, 0, 64, 1, 1), (4, 4, 2, 40, 1, 1)])
+@pytest.mark.parametrize("scoring,with_bias,with_correction,renormalise", [("softmax", False, False, True), ("sigmoid", True, True, False), ("softmax", True, True, True)])
+def test_router_choice_and_sort_of_a_few_tokens(kernels, dtype, tokens, experts, top, extra, hidden, groups, keep, scoring, with_bias, with_correction, renormalise):
+    """In one launch where the sizes allow it: scores, choices and weights as apart, and pairs sorted so that the experts'
+    products find every token's rows."""
+    torch.manual_seed(tokens * 100 + experts)
+    plain, mine = TorchKernels(dtype), kernels[dtype]
+    x = torch.randn(tokens, hidden).to(dtype)
+    rows = [(3.0 * torch.randn(count, hidden) / hidden**0.5).to(dtype) for count in (experts, extra) if count]
+    biases = [torch.randn(len(row)).to(dtype) for row in rows] if with_bias else None
+    correction = 0.3 * torch.randn(experts) if with_correction else None
+    size = 32
+    gates, ups = ([(torch.randn(size, hidden) / hidden**0.5).to(dtype) for _ in range(experts)] for _ in range(2))
+    downs = [(torch.randn(hidden, size) / size**0.5).to(dtype) for _ in range(experts)]
+    options = (experts, None if correction is None else correction, top, 1.3, scoring, groups, keep, renormalise)
+    prepared = plain.prepare_experts(ups, downs, "silu", gates=gates)
+    scores, chosen, weights, _ = plain.route_product(x, plain.prepare_linear(rows, biases), prepared, *options)
+    on = [gpu(w) for w in rows], [gpu(b) for b in biases] if with_bias else None
+    there = mine.prepare_experts([gpu(w) for w in ups], [gpu(w) for w in downs], "silu", gates=[gpu(w) for w in gates])
+    got_scores, got_chosen, got_weights, ordered = mine.route_product(
+        gpu(x), mine.prepare_linear(*on), there, experts, None if correction is None else gpu(correction), *options[2:])
+    assert (ordered is not None) == (dtype == torch.bfloat16 and tokens <= 16 and experts <= 64 and hidden % 32 == 0)
+    torch.testing.assert_close(got_scores.cpu(), scores, atol=2e-4, rtol=2e-4)
+    assert torch.equal(got_chosen.cpu(), chosen)
+    torch.testing.assert_close(got_weights.cpu(), weights, atol=2e-4, rtol=2e-4)
+    want = plain.expert_feed_forward(x, prepared, chosen, weights)
+    close(mine.expert_feed_forward(gpu(x), there, got_chosen, got_weights, sorted_pairs=ordered), want, dtype)
